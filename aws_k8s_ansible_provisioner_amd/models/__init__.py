@@ -19,6 +19,10 @@ def model_class(cfg: ModelConfig):
         from .mudepel import MudepelLM
 
         return MudepelLM
+    if cfg.arch == "papivik":
+        from .papivik import PapivikLM
+
+        return PapivikLM
     from .transformer import DecoderLM
 
     return DecoderLM

@@ -10,6 +10,7 @@ from __future__ import annotations
 
 import dataclasses
 import json
+import math
 import os
 from typing import Optional
 
@@ -144,6 +145,11 @@ class AttentionSpec:
     pool: int = 0
     unit_sink: bool = False
     bias: bool = False
+    # conv > 0: each channel of the projected q, k and v passes a causal convolution of that many
+    # taps (no bias, no activation) before anything else; qk_norm_w: the per-head norms of q and
+    # k carry a weight vector of `dim` entries shared by the heads
+    conv: int = 0
+    qk_norm_w: bool = False
 
 
 @dataclasses.dataclass
@@ -158,6 +164,14 @@ class RetentionSpec:
     vdim: int
     decay: tuple
     rot: Optional[RotarySpec] = None
+    # act "silu": q, k and v pass silu after their projection; k_scaled: k carries dim^-1/2;
+    # out_norm "head": each head's output is divided by its own root mean square, "all": the
+    # concatenated heads by theirs and multiplied by a weight vector; gate: the activation of
+    # the output gate
+    act: str = "none"
+    k_scaled: bool = True
+    out_norm: str = "head"
+    gate: str = "silu"
     # sizing fields shared with AttentionSpec: a retention mixer caches no keys
     kv_heads: int = 0
     chunk: int = 0
@@ -208,11 +222,64 @@ class StateSpaceSpec:
 
 
 @dataclasses.dataclass
+class MatrixMemorySpec:
+    """Linear attention with exponential gates (mLSTM form): per head and live sequence a state
+    S [dim, vdim], a normaliser n [dim] and a running maximum m (fp32, all starting at zero).
+    With the log gates i and f, each soft-capped at `cap` and f through logsigmoid:
+    m' = max(f + m, i), S <- e^(f + m - m') S + e^(i - m') k v^T, n likewise with k alone, and
+    o = S^T q / (max(|n . q|, e^(-m')) + 1e-6), q scaled by dim^-1/2; each head's output is
+    RMS-normed, weighted and gated by a sigmoid."""
+    heads: int
+    dim: int
+    vdim: int
+    cap: float
+    # sizing fields shared with AttentionSpec: nothing is cached per token
+    kv_heads: int = 0
+    chunk: int = 0
+    window: int = 0
+
+    @property
+    def state_floats(self) -> int:
+        return self.heads * (self.dim * self.vdim + self.dim + 1)
+
+
+@dataclasses.dataclass
+class DeltaRuleSpec:
+    """Gated delta rule: q and k (`qk_heads` heads of `dim`, shared by neighbouring heads) and v
+    (`heads` heads of `vdim`) pass a causal per-channel convolution of `conv` taps and silu, q
+    and k are made unit vectors; with a step size beta and a decay g per head and token,
+    S <- g S, S <- S + k (beta (v - S^T k))^T, o = S^T q dim^-1/2 on the fp32 state S
+    [dim, vdim]; each head's output is RMS-normed with one weight vector for all heads and gated
+    by silu."""
+    heads: int
+    qk_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    # sizing fields shared with AttentionSpec: nothing is cached per token
+    kv_heads: int = 0
+    chunk: int = 0
+    window: int = 0
+
+    @property
+    def state_floats(self) -> int:
+        return self.heads * self.dim * self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.qk_heads * self.dim + self.heads * self.vdim
+
+
+@dataclasses.dataclass
 class ParallelMixerSpec:
-    """Two mixers side by side on the same input; the layer's mixer output is half the sum of
-    their outputs, each RMS-normed over the model width with a weight vector of its own."""
+    """Two mixers side by side on the same input.  combine "norm": the layer's mixer output is
+    half the sum of their outputs, each RMS-normed over the model width with a weight vector of
+    its own; "scale": left_scale * left + right_scale * right."""
     left: AttentionSpec
-    right: RetentionSpec
+    right: object                # RetentionSpec | DeltaRuleSpec
+    combine: str = "norm"
+    left_scale: float = 1.0
+    right_scale: float = 1.0
 
     @property
     def heads(self) -> int:
@@ -289,8 +356,8 @@ class RouterSpec:
 class MlpSpec:
     kind: str   # "dense": down(act(up h)) | "moe": routed experts of that form
     ff: int
-    # "relu2" | "xielu" (two learned numbers per layer) | "swiglu" | "geglu" (gated, tanh form
-    # of gelu on the gate)
+    # "relu2" | "xielu" (two learned numbers per layer) | "gelu" (tanh form) | "swiglu" |
+    # "geglu" (gated, tanh form of gelu on the gate)
     act: str = "relu2"
     bias: bool = False
     router: Optional[RouterSpec] = None
@@ -299,9 +366,11 @@ class MlpSpec:
 
 @dataclasses.dataclass
 class LayerSpec:
-    # "attention" | "latent_attention[_2]" | "retention" | "parallel" | "mamba2"
+    # "attention" | "latent_attention[_2]" | "retention" | "lightning" | "mlstm" | "parallel" |
+    # "mamba2"
     type: str
-    # AttentionSpec | LatentAttentionSpec | RetentionSpec | ParallelMixerSpec | StateSpaceSpec
+    # AttentionSpec | LatentAttentionSpec | RetentionSpec | MatrixMemorySpec |
+    # ParallelMixerSpec | StateSpaceSpec
     mixer: object
     mlp: Optional[MlpSpec] = None   # None: the layer has no feed-forward
 
@@ -339,7 +408,7 @@ class LayeredConfig(ModelConfig):
             m = self.layer_specs[i].mixer
             if isinstance(m, LatentAttentionSpec):
                 n += 0 if m.kv_from is not None else m.cache_dim * es
-            elif isinstance(m, (RetentionSpec, StateSpaceSpec)):
+            elif isinstance(m, (RetentionSpec, StateSpaceSpec, MatrixMemorySpec)):
                 pass
             elif isinstance(m, ParallelMixerSpec):
                 n += m.left.kv_heads * (m.left.dim + m.left.vdim) * es
@@ -355,6 +424,8 @@ class LayeredConfig(ModelConfig):
         if self.arch == "mudepel":
             return self.vocab_size * d + d + sum(_mudepel_layer_params(d, max(self.streams, 0), ls)
                                                  for ls in self.layer_specs)
+        if self.arch == "papivik":
+            return n + sum(_papivik_layer_params(d, ls) for ls in self.layer_specs)
         for ls in self.layer_specs:
             m = ls.mixer
             if isinstance(m, (RetentionSpec, ParallelMixerSpec)):
@@ -406,6 +477,24 @@ def _mudepel_layer_params(d: int, streams: int, ls: "LayerSpec") -> int:
     if ml is not None:
         e = ml.router.experts if ml.router else 1
         n += d + hc + 3 * d * ml.ff * e + 3 * d * ml.shared_ff + (e * d if ml.router else 0)
+    return n
+
+
+def _papivik_layer_params(d: int, ls: "LayerSpec") -> int:
+    m = ls.mixer
+    if isinstance(m, ParallelMixerSpec):
+        a, r = m.left, m.right
+        qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
+        n = qkv * (d + a.conv) + 2 * a.dim + d * a.heads * a.vdim
+        n += r.conv_channels * (d + r.conv) + 2 * r.heads * (d + 1) + r.vdim \
+            + 2 * d * r.heads * r.vdim
+    else:
+        n = m.heads * (2 * m.dim + 3 * m.vdim) * d + m.heads * m.vdim
+        if isinstance(m, MatrixMemorySpec):
+            n += 2 * m.heads * (d + 1)
+    n += d
+    if ls.mlp is not None:
+        n += d + 2 * d * ls.mlp.ff
     return n
 
 
@@ -764,9 +853,112 @@ def mudepel_dict(width: int, layers: list, vocab: int = 32000, eps: float = 1e-6
     return d
 
 
+def _papivik_attention(m: dict) -> AttentionSpec:
+    rot = m.get("rot")
+    rs = None
+    if rot and int(rot.get("dims") or 0) > 0:
+        rs = RotarySpec(int(rot["dims"]), float(rot["base"]), layout="half")
+        if rs.dims % 2 or rs.dims > int(m["dim"]):
+            raise ValueError("Papivik: rot.dims must be even and at most dim")
+    spec = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]),
+                         vdim=int(m["vdim"]), scale=float(m["scale"]), rot=rs, sink=False,
+                         gate=False, shared_kv=False, head_norm=True, qk_norm_w=True,
+                         conv=int(m["conv"]))
+    if spec.heads % spec.kv_heads or spec.conv < 1:
+        raise ValueError("Papivik: heads must be a multiple of kv_heads, and conv at least 1")
+    return spec
+
+
+def _papivik_delta(m: dict) -> DeltaRuleSpec:
+    spec = DeltaRuleSpec(heads=int(m["heads"]), qk_heads=int(m["kv_heads"]), dim=int(m["dim"]),
+                         vdim=int(m["vdim"]), conv=int(m["conv"]))
+    if spec.heads % spec.qk_heads or spec.conv < 1:
+        raise ValueError("Papivik: heads must be a multiple of kv_heads, and conv at least 1")
+    return spec
+
+
+def papivik_config(name: str, d: dict, max_position: int = 1 << 20) -> LayeredConfig:
+    """A Papivik config.json: layers that norm only their sublayers' OUTPUTS, mixers "mlstm"
+    (matrix memory with exponential gates), "lightning" (linear attention with a fixed decay per
+    head over silu-activated q, k, v) or "parallel" (a convolved, qk-normed softmax attention
+    beside a gated delta rule, added with two constants), dense gelu feed-forwards or none,
+    separate output head."""
+    specs = []
+    for ly in d["layers"]:
+        m = ly["mixer"]
+        if ly["type"] == "mlstm":
+            mixer = MatrixMemorySpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                     cap=float(m["gate_cap"]))
+        elif ly["type"] == "lightning":
+            mixer = RetentionSpec(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                  decay=tuple(float(g) for g in m["decay"]), act="silu",
+                                  k_scaled=False, out_norm="all", gate="sigmoid")
+            if len(mixer.decay) != mixer.heads or not all(0.0 <= g <= 1.0 for g in mixer.decay):
+                raise ValueError("Papivik: one decay in [0, 1] per lightning head")
+        elif ly["type"] == "parallel":
+            mixer = ParallelMixerSpec(_papivik_attention(m["left"]), _papivik_delta(m["right"]),
+                                      combine="scale", left_scale=float(m["left_scale"]),
+                                      right_scale=float(m["right_scale"]))
+        else:
+            raise ValueError(f"Papivik: unknown mixer type {ly['type']!r}")
+        ml = ly.get("mlp")
+        if ml is not None and ml.get("kind") != "dense":
+            raise ValueError(f"Papivik: unknown feed-forward kind {ml.get('kind')!r}")
+        mlp = MlpSpec("dense", int(ml["ff"]), act="gelu") if ml is not None else None
+        specs.append(LayerSpec(ly["type"], mixer, mlp))
+    par = [ls.mixer for ls in specs if isinstance(ls.mixer, ParallelMixerSpec)]
+    return LayeredConfig(
+        name=name, hf_id=name, arch="papivik", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]),
+        intermediate_size=max([ls.mlp.ff for ls in specs if ls.mlp is not None] or [0]),
+        num_layers=len(specs), num_heads=max(ls.mixer.heads for ls in specs),
+        num_kv_heads=max([p.left.kv_heads for p in par] + [1]),
+        head_dim=max([ls.mixer.dim for ls in specs]), rms_eps=float(d["norm"]["eps"]),
+        max_position=max_position, bos_id=0, eos_id=-1, layer_specs=specs,
+        embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)))
+
+
+def papivik_dict(width: int, layers: list, vocab: int = 32000, eps: float = 1e-6,
+                 embed_scale: float = 1.0) -> dict:
+    """A Papivik config.json dictionary from short layer dicts (random-init benchmarks and
+    tests).  A layer gives `mlstm` = (heads, dim, vdim) with optional cap, or `lightning` =
+    (heads, dim, vdim) with optional decay (list), or `att` = (heads, kv_heads, dim, vdim) and
+    `delta` = (heads, kv_heads, dim, vdim) with optional rot_dims, base, scale, conv (two
+    numbers), scales (two numbers); and optionally `ff`."""
+    out = []
+    for ly in layers:
+        if "mlstm" in ly:
+            h, dd, vv = ly["mlstm"]
+            kind, m = "mlstm", {"heads": h, "dim": dd, "vdim": vv,
+                                "gate_cap": float(ly.get("cap", 15.0))}
+        elif "lightning" in ly:
+            h, dd, vv = ly["lightning"]
+            decay = ly.get("decay") or [math.exp(-(2.0 ** (-8.0 * (i + 1) / h)))
+                                        for i in range(h)]
+            kind, m = "lightning", {"heads": h, "dim": dd, "vdim": vv,
+                                    "decay": [float(g) for g in decay]}
+        else:
+            h, g, dd, vv = ly["att"]
+            rh, rg, rd, rv = ly["delta"]
+            cl, cr = ly.get("conv", (4, 4))
+            sl, sr = ly.get("scales", (1.0, 1.0))
+            kind = "parallel"
+            m = {"left": {"heads": h, "kv_heads": g, "dim": dd, "vdim": vv, "conv": cl,
+                          "scale": float(ly.get("scale", dd ** -0.5)),
+                          "rot": {"base": float(ly.get("base", 10000.0)),
+                                  "dims": int(ly.get("rot_dims", dd))}},
+                 "right": {"heads": rh, "kv_heads": rg, "dim": rd, "vdim": rv, "conv": cr},
+                 "left_scale": float(sl), "right_scale": float(sr)}
+        out.append({"type": kind, "mixer": m,
+                    "mlp": {"kind": "dense", "ff": ly["ff"]} if ly.get("ff") else None})
+    return {"architecture": "Papivik", "embedding": {"scale": embed_scale}, "layers": out,
+            "norm": {"eps": eps}, "vocab": vocab, "width": width}
+
+
 # config.json readers of designs that do not use the HF key set, by their "architecture" value
 _NATIVE_READERS = {"Bidetar": bidetar_config, "Puputar": puputar_config,
-                   "Sazepel": sazepel_config, "Mudepel": mudepel_config}
+                   "Sazepel": sazepel_config, "Mudepel": mudepel_config,
+                   "Papivik": papivik_config}
 
 _REGISTRY: dict[str, ModelConfig] = {}
 
@@ -1026,6 +1218,44 @@ TINY_MUDEPEL = register(_mudepel_stack(
     expert_ff=64, top=2, window=24, pool=8, vocab=512, streams=3, groups=3, keep=2,
     norm_groups=2, loop=(1, 3, 2), rot_dims=16,
     yarn={"factor": 2.0, "original": 64, "fast": 8.0, "slow": 1.0}))
+
+
+def _papivik_stack(name: str, width: int, n: int, att: tuple, delta: tuple, mlstm: tuple,
+                   lightning: tuple, ff: int, vocab: int = 32000, rot_dims: Optional[int] = None,
+                   scales: tuple = (1.0, 1.0), conv: tuple = (4, 4), embed_scale: float = 1.0
+                   ) -> LayeredConfig:
+    """n layers in turns of four: mLSTM, parallel, lightning, parallel; all with a dense
+    feed-forward except the last."""
+    layers = []
+    for i in range(n):
+        if i % 2:
+            ly = dict(att=att, delta=delta, base=500000.0, scales=scales, conv=conv)
+            if rot_dims is not None:
+                ly["rot_dims"] = rot_dims
+        else:
+            ly = dict(mlstm=mlstm) if i % 4 == 0 else dict(lightning=lightning)
+        if i + 1 < n:
+            ly["ff"] = ff
+        layers.append(ly)
+    cfg = papivik_config(name, papivik_dict(width, layers, vocab=vocab, embed_scale=embed_scale))
+    cfg.hf_id = "test/" + name
+    return cfg
+
+
+# Papivik at layer sizes of real models (random weights; bench.py --compare-design papivik):
+# 16 / 4 attention heads of 128 beside 16 delta-rule heads with 128 x 128 states over 8 key
+# heads, mLSTM layers of 8 heads with 128 x 256 states, lightning layers of 16 heads with
+# 128 x 128 states
+PAPIVIK_W2048 = register(_papivik_stack(
+    "papivik-w2048", width=2048, n=16, att=(16, 4, 128, 128), delta=(16, 8, 128, 128),
+    mlstm=(8, 128, 256), lightning=(16, 128, 128), ff=8192, rot_dims=64))
+PAPIVIK_W4096 = register(_papivik_stack(
+    "papivik-w4096", width=4096, n=8, att=(32, 8, 128, 128), delta=(32, 16, 128, 128),
+    mlstm=(16, 128, 256), lightning=(32, 128, 128), ff=16384, rot_dims=64))
+TINY_PAPIVIK = register(_papivik_stack(
+    "tiny-papivik", width=128, n=5, att=(4, 2, 32, 16), delta=(4, 2, 16, 32), mlstm=(2, 16, 24),
+    lightning=(3, 16, 32), ff=192, vocab=512, rot_dims=16, scales=(1.2, 0.8), conv=(3, 4),
+    embed_scale=0.5))
 
 
 def get_config(name: str) -> ModelConfig:

@@ -109,6 +109,15 @@ def relu2(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     return out
 
 
+def gelu_tanh(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3))) (fp32 arithmetic); x and out are
+    [T, F] views that may be column slices of wider rows."""
+    if _native(x):
+        torch.ops.akap_stream.gelu_tanh(out, x)
+        return
+    out.copy_(torch.nn.functional.gelu(x.float(), approximate="tanh").to(out.dtype))
+
+
 # ----------------------------------------------------------------------------- rotary, cache
 def rotary_table(max_pos: int, dims: int, base: float, scaling: Optional[dict] = None,
                  device=None) -> torch.Tensor:
@@ -641,11 +650,12 @@ def _w(w: torch.Tensor) -> torch.Tensor:
 
 def stream_post_norm_add_norm(x: torch.Tensor, ya: torch.Tensor, yb: Optional[torch.Tensor],
                               wa: Optional[torch.Tensor], wb: Optional[torch.Tensor],
-                              post_w: torch.Tensor, next_w: torch.Tensor, eps: float,
+                              post_w: torch.Tensor, next_w: Optional[torch.Tensor], eps: float,
                               out: torch.Tensor, fresh: bool = False) -> None:
     """The residual update of a sublayer whose OUTPUT is normed, fused with the norm that feeds
     the next sublayer:  m = ya, or with two branches m = (rms(ya) wa + rms(yb) wb) / 2;
-    x <- x + rms(m) post_w (fresh: x <- rms(m) post_w, x is not read);  out = rms(x) next_w.
+    x <- x + rms(m) post_w (fresh: x <- rms(m) post_w, x is not read);  out = rms(x) next_w
+    (next_w None: out = x, for a sublayer that reads the stream itself).
     rms(v) = v / sqrt(mean(v^2) + eps) over the row.  x fp32 [T, d] (the stream, updated in
     place); ya / yb [T, d] in the activation type or fp32; every weight is fp32 with d entries
     or ONE (a single number for all coordinates).  All arithmetic is fp32; out is rounded
@@ -662,23 +672,28 @@ def stream_post_norm_add_norm(x: torch.Tensor, ya: torch.Tensor, yb: Optional[to
         x.copy_(upd)
     else:
         x.add_(upd)
-    out.copy_((_rms(x, eps) * _w(next_w)).to(out.dtype))
+    out.copy_((_rms(x, eps) * _w(next_w) if next_w is not None else x).to(out.dtype))
 
 
 # ----------------------------------------------------------------------------- head-mixed attention
 def head_norm_cache(proj: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor,
                     v_cache: torch.Tensor, slots: torch.Tensor, H: int, G: int, D: int, Dv: int,
                     q_off: int, k_off: int, v_off: int, eps: float, norm_qk: bool = True,
-                    norm_v: bool = True) -> None:
+                    norm_v: bool = True, q_w: Optional[torch.Tensor] = None,
+                    k_w: Optional[torch.Tensor] = None, cos_sin: Optional[torch.Tensor] = None,
+                    positions: Optional[torch.Tensor] = None) -> None:
     """Per token t of the fused projection proj [T, N]: the H query heads
     proj[t, q_off : q_off + H D] go to q_out [T, H, D], the G key heads (from k_off) to k_cache
     [NB, G, BS, D] and the G value heads (from v_off, size Dv) to v_cache [NB, G, BS / 8, Dv, 8]
-    (groups of 8 tokens, dimension-major inside a group) at slots[t] (-1: nothing is cached).  norm_qk / norm_v: each head is first divided by its own
-    root mean square (fp32, eps inside the root, no weights)."""
+    (groups of 8 tokens, dimension-major inside a group) at slots[t] (-1: nothing is cached).
+    norm_qk / norm_v: each head is first divided by its own root mean square (fp32, eps inside
+    the root); q_w / k_w (fp32 [D], shared by the heads): the norms' weights.  cos_sin: q and k
+    are then rotated on their first cos_sin.shape[1] dimensions in the rotate-half layout
+    (entry i with i + dims/2) by the table row of positions[t]."""
     if _native(proj):
         torch.ops.akap_stream.head_norm_cache(proj, q_out, k_cache, v_cache, slots, H, G, D, Dv,
                                               q_off, k_off, v_off, float(eps), bool(norm_qk),
-                                              bool(norm_v))
+                                              bool(norm_v), q_w, k_w, cos_sin, positions)
         return
     T = proj.shape[0]
     q = proj[:, q_off:q_off + H * D].float().view(T, H, D)
@@ -686,6 +701,13 @@ def head_norm_cache(proj: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tens
     v = proj[:, v_off:v_off + G * Dv].float().view(T, G, Dv)
     if norm_qk:
         q, k = _rms(q, eps), _rms(k, eps)
+    if q_w is not None:
+        q = q * q_w.float()
+    if k_w is not None:
+        k = k * k_w.float()
+    if cos_sin is not None:
+        cs = cos_sin[positions.long()]
+        q, k = rotate_half_(q.clone(), cs), rotate_half_(k.clone(), cs)
     if norm_v:
         v = _rms(v, eps)
     q_out.copy_(q.to(q_out.dtype))
@@ -893,6 +915,211 @@ def retention(out: torch.Tensor, proj: torch.Tensor, q_off: int, k_off: int, v_o
         state[slot] = S.transpose(1, 2)
         on = _rms(o[r0:r1], eps) * torch.nn.functional.silu(g[r0:r1])
         out[r0:r1] = on.reshape(r1 - r0, H * V).to(out.dtype)
+
+
+# ----------------------------------------------------------------------------- matrix-state recurrences
+def norm_gate(out: torch.Tensor, y: torch.Tensor, gate: torch.Tensor, w: torch.Tensor,
+              groups: int, eps: float, act: str = "sigmoid", den: Optional[torch.Tensor] = None,
+              floor: Optional[torch.Tensor] = None) -> None:
+    """out = gnorm(y) w act(gate): y [T, n] fp32 RMS-normed in `groups` equal consecutive parts
+    (each by its own root mean square), times the fp32 weights w [n], times act ("sigmoid" |
+    "silu") of gate [T, n] (a column slice of a projection); the gate comes after the norm.  den
+    and floor (fp32 [T, groups]): a part of y is first divided by max(|den|, floor) + 1e-6.  out
+    may be a column slice of wider rows.  fp32 arithmetic."""
+    if _native(y):
+        torch.ops.akap_stream.norm_gate(out, y, gate, w, int(groups), float(eps),
+                                        1 if act == "silu" else 0, den, floor)
+        return
+    T, n = y.shape
+    v = y.float()
+    if den is not None:
+        d = torch.maximum(den.abs(), floor) + 1e-6
+        v = (v.view(T, groups, n // groups) / d[:, :, None]).view(T, n)
+    g = gate.float()
+    g = torch.nn.functional.silu(g) if act == "silu" else torch.sigmoid(g)
+    out.copy_((_group_rms(v, groups, eps) * w.float() * g).to(out.dtype))
+
+
+_REC_MODE = {"decay": 0, "mlstm": 1, "delta": 2}
+
+
+def _recurrence(mode: str, out, qkv, q_off, k_off, v_off, act, proj, gates: tuple, pa, pb, cap,
+                q_scale, state, n_state, m_state, norm_w, g_off, gate_act, norm_all, eps,
+                seq_slot, positions, q_start, H, G, D, V) -> None:
+    """GPU form of the recurrences below: the scan kernel (one workgroup per sequence, head and
+    block of state columns, state in registers) with the head norm and the gate fused where a
+    workgroup holds a whole head, else followed by norm_gate."""
+    T = qkv.shape[0]
+    fuse = not norm_all and torch.ops.akap_stream.recurrence_fused(D, V)
+    raw = None if fuse else torch.empty(T, H * V, dtype=torch.float32, device=qkv.device)
+    torch.ops.akap_stream.recurrence(_REC_MODE[mode], out, raw, qkv, q_off, k_off, v_off, act,
+                                     proj, gates[0], gates[1], pa, pb, float(cap), float(q_scale),
+                                     state, n_state, m_state, norm_w, g_off,
+                                     1 if gate_act == "silu" else 0, float(eps), seq_slot,
+                                     positions, q_start, H, G, D, V)
+    if raw is not None:
+        norm_gate(out, raw, proj[:, g_off:g_off + H * V], norm_w, 1 if norm_all else H, eps,
+                  gate_act)
+
+
+def _heads(x: torch.Tensor, off: int, n: int, size: int) -> torch.Tensor:
+    return x[:, off:off + n * size].float().reshape(x.shape[0], n, size)
+
+
+def _live_sequences(T, q_start, seq_slot):
+    for r0, r1 in _row_sequences(T, q_start):
+        if r1 > r0 and int(seq_slot[r0]) >= 0:
+            yield r0, r1, int(seq_slot[r0])
+
+
+def linear_attention(out: torch.Tensor, proj: torch.Tensor, q_off: int, k_off: int, v_off: int,
+                     g_off: int, decay: torch.Tensor, state: torch.Tensor, norm_w: torch.Tensor,
+                     seq_slot: torch.Tensor, positions: torch.Tensor,
+                     q_start: Optional[torch.Tensor], H: int, D: int, V: int, eps: float,
+                     act: str = "silu", norm: str = "all", gate: str = "sigmoid",
+                     first_seq: int = 0) -> None:
+    """Linear attention with a fixed decay per head, for the token rows of a step.  From the
+    fused projection proj [T, N]: q, k (H heads of D from q_off / k_off) and v (H heads of V from
+    v_off), each through act ("silu" | "none"); S <- decay[h] S + k v^T, o = S^T q; the outputs
+    are RMS-normed per head (norm "head") or over all heads together ("all"), times norm_w
+    [H V], times gate(proj[t, g_off ...]), to out [T, H V] (may be a column slice).  decay fp32
+    [H].  The state of a sequence lives transposed in state[slot, h] (fp32 [V, D]).  Sequences,
+    slots and fresh starts as in `retention`.  first_seq: the sequences before it are single
+    rows (the decode rows of a mixed step)."""
+    if _native(proj):
+        _recurrence("decay", out, proj, q_off, k_off, v_off, 1 if act == "silu" else 0, proj,
+                    (0, 0), decay, None, 0.0, 1.0, state, None, None, norm_w, g_off, gate,
+                    norm == "all", eps, seq_slot, positions, q_start, H, H, D, V)
+        return
+    T = proj.shape[0]
+    q, k, v = _heads(proj, q_off, H, D), _heads(proj, k_off, H, D), _heads(proj, v_off, H, V)
+    if act == "silu":
+        q, k, v = (torch.nn.functional.silu(t) for t in (q, k, v))
+    o = torch.zeros(T, H, V)
+    for r0, r1, slot in _live_sequences(T, q_start, seq_slot):
+        S = state[slot].transpose(1, 2).clone() if int(positions[r0]) > 0 else torch.zeros(H, D, V)
+        for t in range(r0, r1):
+            S = decay.float()[:, None, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S.transpose(1, 2)
+    norm_gate(out, o.view(T, H * V), proj[:, g_off:g_off + H * V], norm_w,
+              1 if norm == "all" else H, eps, gate)
+
+
+def matrix_memory(out: torch.Tensor, proj: torch.Tensor, q_off: int, k_off: int, v_off: int,
+                  g_off: int, i_off: int, f_off: int, i_b: torch.Tensor, f_b: torch.Tensor,
+                  cap: float, state: tuple, norm_w: torch.Tensor, seq_slot: torch.Tensor,
+                  positions: torch.Tensor, q_start: Optional[torch.Tensor], H: int, D: int,
+                  V: int, eps: float, first_seq: int = 0) -> None:
+    """The mLSTM recurrence for the token rows of a step.  q (scaled by D^-1/2), k, v and the
+    output gate from the fused projection as in linear_attention (no activation); log gates
+    i = cap tanh((proj[t, i_off + h] + i_b[h]) / cap) and f = logsigmoid(cap tanh((proj[t, f_off
+    + h] + f_b[h]) / cap)).  With m' = max(f + m, i): S <- e^(f + m - m') S + e^(i - m') k v^T,
+    n <- e^(f + m - m') n + e^(i - m') k, o = S^T q / (max(|n . q|, e^(-m')) + 1e-6); each
+    head's o is RMS-normed over V, times norm_w [H V], times sigmoid(gate).  state = (S^T [slots,
+    H, V, D], n [slots, H, D], m [slots, H]), all fp32 and zero at position 0."""
+    S_st, n_st, m_st = state
+    if _native(proj):
+        _recurrence("mlstm", out, proj, q_off, k_off, v_off, 0, proj, (f_off, i_off), f_b, i_b,
+                    cap, D ** -0.5, S_st, n_st, m_st, norm_w, g_off, "sigmoid", False, eps,
+                    seq_slot, positions, q_start, H, H, D, V)
+        return
+    T = proj.shape[0]
+    q, k, v = _heads(proj, q_off, H, D), _heads(proj, k_off, H, D), _heads(proj, v_off, H, V)
+    q = q * D ** -0.5
+    ig = cap * torch.tanh((proj[:, i_off:i_off + H].float() + i_b) / cap)
+    fg = torch.nn.functional.logsigmoid(
+        cap * torch.tanh((proj[:, f_off:f_off + H].float() + f_b) / cap))
+    o = torch.zeros(T, H, V)
+    for r0, r1, slot in _live_sequences(T, q_start, seq_slot):
+        if int(positions[r0]) > 0:
+            S, n, m = S_st[slot].transpose(1, 2).clone(), n_st[slot].clone(), m_st[slot].clone()
+        else:
+            S, n, m = torch.zeros(H, D, V), torch.zeros(H, D), torch.zeros(H)
+        for t in range(r0, r1):
+            m2 = torch.maximum(fg[t] + m, ig[t])
+            keep, add = torch.exp(fg[t] + m - m2), torch.exp(ig[t] - m2)
+            m = m2
+            ka = add[:, None] * k[t]
+            S = keep[:, None, None] * S + ka[:, :, None] * v[t][:, None, :]
+            n = keep[:, None] * n + ka
+            den = torch.maximum((n * q[t]).sum(dim=-1).abs(), torch.exp(-m)) + 1e-6
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t]) / den[:, None]
+        S_st[slot], n_st[slot], m_st[slot] = S.transpose(1, 2), n, m
+    norm_gate(out, o.view(T, H * V), proj[:, g_off:g_off + H * V], norm_w, H, eps, "sigmoid")
+
+
+def gated_delta(out: torch.Tensor, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int,
+                proj: torch.Tensor, g_off: int, b_off: int, a_off: int, a_log: torch.Tensor,
+                dt_bias: torch.Tensor, state: torch.Tensor, norm_w: torch.Tensor,
+                seq_slot: torch.Tensor, positions: torch.Tensor, q_start: Optional[torch.Tensor],
+                H: int, G: int, D: int, V: int, eps: float, first_seq: int = 0) -> None:
+    """The gated delta rule for the token rows of a step.  qkv [T, .]: q and k (G heads of D; head
+    h of the H value heads uses h // (H / G)) and v (H heads of V), already convolved and
+    activated; q and k are made unit vectors, x / sqrt(sum x^2 + 1e-6), and q scaled by D^-1/2.
+    From proj [T, N]: beta = sigmoid(proj[t, b_off + h]), g = exp(-exp(a_log[h])
+    softplus(proj[t, a_off + h] + dt_bias[h])).  S <- g S; u = beta (v - S^T k); S <- S + k u^T;
+    o = S^T q.  Each head's o is RMS-normed over V, times norm_w [H V], times silu(proj[t,
+    g_off + h V ...]).  State, sequences and out as in linear_attention."""
+    if _native(qkv):
+        _recurrence("delta", out, qkv, q_off, k_off, v_off, 0, proj, (a_off, b_off), a_log,
+                    dt_bias, 0.0, D ** -0.5, state, None, None, norm_w, g_off, "silu", False, eps,
+                    seq_slot, positions, q_start, H, G, D, V)
+        return
+    T = qkv.shape[0]
+    q, k, v = _heads(qkv, q_off, G, D), _heads(qkv, k_off, G, D), _heads(qkv, v_off, H, V)
+    q = q * torch.rsqrt((q * q).sum(dim=-1, keepdim=True) + 1e-6) * D ** -0.5
+    k = k * torch.rsqrt((k * k).sum(dim=-1, keepdim=True) + 1e-6)
+    q, k = q.repeat_interleave(H // G, dim=1), k.repeat_interleave(H // G, dim=1)
+    beta = torch.sigmoid(proj[:, b_off:b_off + H].float())
+    g = torch.exp(-torch.exp(a_log.float()) * torch.nn.functional.softplus(
+        proj[:, a_off:a_off + H].float() + dt_bias.float(), threshold=30.0))
+    o = torch.zeros(T, H, V)
+    for r0, r1, slot in _live_sequences(T, q_start, seq_slot):
+        S = state[slot].transpose(1, 2).clone() if int(positions[r0]) > 0 else torch.zeros(H, D, V)
+        for t in range(r0, r1):
+            S = g[t][:, None, None] * S
+            u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S.transpose(1, 2)
+    norm_gate(out, o.view(T, H * V), proj[:, g_off:g_off + H * V], norm_w, H, eps, "silu")
+
+
+# ----------------------------------------------------------------------------- plain causal attention
+def causal_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
+                     v_cache: torch.Tensor, batch, scale: float, max_len: int,
+                     workspace=None) -> None:
+    """Causal grouped-query softmax attention of the rows of a step (batch: the runner's
+    AttnBatch) over the paged cache, no window, sink or gate; out may be a column slice of wider
+    rows.  Heads whose keys and values have the same size go through the sink attention kernels
+    (without a sink), which split long key ranges of decode rows; others through the pooled
+    window kernels (without window and pooled entries).  workspace: callable (rows, parts) ->
+    decode_workspace buffers."""
+    T, H, D = q.shape
+    G, Dv = k_cache.shape[1], v_cache.shape[3]
+    nd = batch.num_decode if batch.is_prefill else T
+    if D != Dv:
+        if batch.is_prefill:
+            pooled_window_attention_prefill(
+                out, q, k_cache, v_cache, None, None, batch.block_tables, batch.q_start,
+                batch.positions, batch.slots, batch.tile_seq, batch.tile_row, batch.tile_rows,
+                scale, 0, 0, False, first_seq=nd)
+        else:
+            pooled_window_attention_decode(out, q, k_cache, v_cache, None, None,
+                                           batch.block_tables, batch.positions, batch.slots,
+                                           scale, 0, 0, False)
+        return
+    if nd:
+        wgs = max(1, nd * G)
+        parts = 1 if wgs >= 1024 else min(max(1, -(-max_len // DECODE_PART)), 64, -(-1024 // wgs))
+        ws = workspace(nd, parts) if (parts > 1 and q.is_cuda) else None
+        sink_attention_decode(out[:nd], q[:nd], k_cache, v_cache, batch.block_tables[:nd],
+                              batch.seq_lens[:nd], None, None, scale, 0, 0, ws, parts)
+    if batch.is_prefill:
+        sink_attention_prefill(out, q, k_cache, v_cache, batch.block_tables, batch.seq_lens,
+                               batch.q_start, batch.tile_seq, batch.tile_row, batch.tile_rows,
+                               None, None, scale, 0, 0, first_seq=nd)
 
 
 # ----------------------------------------------------------------------------- logit-top-k routing
@@ -1201,19 +1428,21 @@ def pooled_window_attention_prefill(out: torch.Tensor, q: torch.Tensor, k_cache:
 
 # ----------------------------------------------------------------------------- selective state space
 def conv_silu(out: torch.Tensor, proj: torch.Tensor, off: int, conv_w: torch.Tensor,
-              conv_b: torch.Tensor, state: torch.Tensor, seq_slot: torch.Tensor,
-              positions: torch.Tensor, q_start: Optional[torch.Tensor]) -> None:
+              conv_b: Optional[torch.Tensor], state: torch.Tensor, seq_slot: torch.Tensor,
+              positions: torch.Tensor, q_start: Optional[torch.Tensor],
+              silu_from: int = 0) -> None:
     """Causal per-channel convolution + silu over the columns [off, off + C) of proj [T, N]:
-    out[t, c] = silu(conv_b[c] + sum_j conv_w[c, j] u[t - (taps - 1 - j), c]) (fp32 [T, C]),
-    u the column of the sequence's earlier tokens: rows of this step, before them what an
+    out[t, c] = act(conv_b[c] + sum_j conv_w[c, j] u[t - (taps - 1 - j), c]) ([T, C], fp32 or
+    proj's type), act = silu for the channels from silu_from on and nothing before it; u is the
+    column of the sequence's earlier tokens: rows of this step, before them what an
     earlier step left in state[slot] ([slots, taps - 1, C], proj's type, oldest first), zeros
     before position 0.  After the step state[slot] holds the sequence's last taps - 1 inputs.
     Sequences as in `retention`: rows [q_start[b], q_start[b + 1]) (None: one row each), slot =
     seq_slot of the first row (-1: padding), fresh when that row has position 0.  conv_w
-    [C, taps], conv_b [C] fp32."""
+    [C, taps], conv_b [C] (None: no bias) fp32."""
     if _native(proj):
         torch.ops.akap_stream.conv_silu(out, proj, int(off), conv_w, conv_b, state, seq_slot,
-                                        positions, q_start)
+                                        positions, q_start, int(silu_from))
         return
     C, taps = conv_w.shape
     for r0, r1 in _row_sequences(proj.shape[0], q_start):
@@ -1223,10 +1452,12 @@ def conv_silu(out: torch.Tensor, proj: torch.Tensor, off: int, conv_w: torch.Ten
         prev = state[slot, :taps - 1].float() if int(positions[r0]) > 0 \
             else torch.zeros(taps - 1, C)
         u = torch.cat([prev, proj[r0:r1, off:off + C].float()])      # [taps - 1 + n, C]
-        acc = conv_b.float()[None, :].repeat(r1 - r0, 1)
+        acc = torch.zeros(r1 - r0, C) if conv_b is None else \
+            conv_b.float()[None, :].repeat(r1 - r0, 1)
         for j in range(taps):
             acc = acc + conv_w[:, j].float()[None, :] * u[j:j + r1 - r0]
-        out[r0:r1] = torch.nn.functional.silu(acc)
+        acc[:, silu_from:] = torch.nn.functional.silu(acc[:, silu_from:])
+        out[r0:r1] = acc.to(out.dtype)
         if taps > 1:
             state[slot, :taps - 1] = u[-(taps - 1):].to(state.dtype)
 
