@@ -225,19 +225,29 @@ void launch_add_norm(void* out, bool out_f32, float* x, const void* y, bool y_f3
     add_norm_t<bf16, bf16>(out, x, y, y_stride, bias, mult, w, rows, d, out_stride, eps, s);
 }
 
-template <typename T>
-__global__ __launch_bounds__(256) void relu2_kernel(T* __restrict__ out, const T* __restrict__ x,
-                                                    int F, int x_stride, int out_stride) {
+template <int ACT>   // 0: relu(z)^2, 1: gelu in its tanh form
+__device__ __forceinline__ float activate(float z) {
+  if (ACT == 0) {
+    const float f = fmaxf(z, 0.f);
+    return f * f;
+  }
+  // 0.5 (1 + tanh(u)) = 1 / (1 + exp(-2 u))
+  const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z / (1.0f + __expf(-2.0f * u));
+}
+
+template <typename T, int ACT>
+__global__ __launch_bounds__(256) void act_kernel(T* __restrict__ out, const T* __restrict__ x,
+                                                  int F, int x_stride, int out_stride) {
   const int row = blockIdx.y;
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= F) return;
-  const float f = fmaxf(ldf(x + (size_t)row * x_stride + c), 0.f);
-  stf(out + (size_t)row * out_stride + c, f * f);
+  stf(out + (size_t)row * out_stride + c, activate<ACT>(ldf(x + (size_t)row * x_stride + c)));
 }
 
 // 16 bytes per thread and access
-template <typename T, int V>
-__global__ __launch_bounds__(256) void relu2_vec_kernel(T* __restrict__ out,
+template <typename T, int V, int ACT>
+__global__ __launch_bounds__(256) void act_vec_kernel(T* __restrict__ out,
                                                         const T* __restrict__ x, int F,
                                                         int x_stride, int out_stride) {
   const int row = blockIdx.y;
@@ -246,33 +256,31 @@ __global__ __launch_bounds__(256) void relu2_vec_kernel(T* __restrict__ out,
   float v[V];
   ldv(v, x + (size_t)row * x_stride + c);
 #pragma unroll
-  for (int e = 0; e < V; ++e) {
-    const float f = fmaxf(v[e], 0.f);
-    v[e] = f * f;
-  }
+  for (int e = 0; e < V; ++e) v[e] = activate<ACT>(v[e]);
   stv(out + (size_t)row * out_stride + c, v);
 }
 
-void launch_relu2(void* out, const void* x, bool f32, int rows, int F, int x_stride,
-                  int out_stride, hipStream_t s) {
+void launch_activation(void* out, const void* x, bool f32, int act, int rows, int F, int x_stride,
+                       int out_stride, hipStream_t s) {
   if (rows <= 0 || F <= 0) return;
   const int V = f32 ? 4 : 8;
-  if (F % V == 0 && x_stride % V == 0 && out_stride % V == 0 && aligned(x, 16) &&
-      aligned(out, 16)) {
-    const dim3 vgrid((F / V + 255) / 256, rows);
-    if (f32)
-      relu2_vec_kernel<float, 4><<<vgrid, 256, 0, s>>>((float*)out, (const float*)x, F, x_stride,
-                                                       out_stride);
-    else
-      relu2_vec_kernel<bf16, 8><<<vgrid, 256, 0, s>>>((bf16*)out, (const bf16*)x, F, x_stride,
-                                                      out_stride);
-    return;
+  const bool vec = F % V == 0 && x_stride % V == 0 && out_stride % V == 0 && aligned(x, 16) &&
+                   aligned(out, 16);
+  const dim3 vgrid((F / V + 255) / 256, rows), grid((F + 255) / 256, rows);
+#define AKAP_ACT(TY, VV, A)                                                                     \
+  do {                                                                                          \
+    if (vec)                                                                                    \
+      act_vec_kernel<TY, VV, A><<<vgrid, 256, 0, s>>>((TY*)out, (const TY*)x, F, x_stride,      \
+                                                      out_stride);                              \
+    else                                                                                        \
+      act_kernel<TY, A><<<grid, 256, 0, s>>>((TY*)out, (const TY*)x, F, x_stride, out_stride);  \
+  } while (0)
+  if (f32) {
+    if (act == 1) AKAP_ACT(float, 4, 1); else AKAP_ACT(float, 4, 0);
+  } else {
+    if (act == 1) AKAP_ACT(bf16, 8, 1); else AKAP_ACT(bf16, 8, 0);
   }
-  const dim3 grid((F + 255) / 256, rows);
-  if (f32)
-    relu2_kernel<float><<<grid, 256, 0, s>>>((float*)out, (const float*)x, F, x_stride, out_stride);
-  else
-    relu2_kernel<bf16><<<grid, 256, 0, s>>>((bf16*)out, (const bf16*)x, F, x_stride, out_stride);
+#undef AKAP_ACT
 }
 
 // One workgroup per token: sums of squares over the WHOLE q and the WHOLE k projection, then

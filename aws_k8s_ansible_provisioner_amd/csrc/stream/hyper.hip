@@ -311,20 +311,21 @@ __global__ __launch_bounds__(256) void route_sigmoid_kernel(int32_t* __restrict_
 constexpr int kMaxTaps = 8;
 
 struct ConvArgs {
-  float* out;              // [T, C]
+  void* out;               // [T, C]
   const void* proj;        // rows of proj_stride; the convolution's columns start at off
   void* state;             // [slots, taps - 1, C] of proj's type, oldest first
   const float* w;          // [C, taps]
-  const float* b;          // [C]
+  const float* b;          // [C] or null
   const int32_t* seq_slot; // [T]
   const int64_t* positions;
   const int32_t* q_start;  // [B + 1] or null (a row is a sequence)
   int proj_stride, off, C, taps, T, B;
+  int silu_from;           // silu on the channels from here on
 };
 
 // a thread per (row, channel): inputs before the step's first row of the sequence come from the
 // slot (zeros before position 0)
-template <typename TY>
+template <typename TY, typename TO>
 __global__ __launch_bounds__(256) void conv_silu_kernel(const ConvArgs a) {
   const int t = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
   if (c >= a.C) return;
@@ -334,7 +335,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const ConvArgs a) {
   const int64_t pos0 = a.positions[r0];
   const TY* proj = (const TY*)a.proj;
   const TY* st = (const TY*)a.state + (size_t)slot * (a.taps - 1) * a.C;
-  float acc = a.b[c];
+  float acc = a.b ? a.b[c] : 0.f;
   for (int j = 0; j < a.taps; ++j) {
     const int src = t - (a.taps - 1 - j);
     float u = 0.f;
@@ -346,7 +347,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const ConvArgs a) {
     }
     acc += a.w[(size_t)c * a.taps + j] * u;
   }
-  a.out[(size_t)t * a.C + c] = siluf(acc);
+  stf((TO*)a.out + (size_t)t * a.C + c, c >= a.silu_from ? siluf(acc) : acc);
 }
 
 // four channels per thread over a tile of RB rows (kConvRows for prompt chunks, 1 for steps of
@@ -356,7 +357,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(const ConvArgs a) {
 // history comes from its slot
 constexpr int kConvRows = 16;
 
-template <typename TY>
+template <typename TY, typename TO>
 __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const ConvArgs a, const int RB) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 4;
   if (c >= a.C) return;
@@ -364,7 +365,9 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const ConvArgs a, co
   constexpr bool F32 = sizeof(TY) == 4;
   const TY* proj = (const TY*)a.proj;
   float bias[4], w[4][kMaxTaps], hist[kMaxTaps][4];   // hist[j]: the input taps - 1 - j rows back
-  ld4v(a.b, true, c, bias);
+#pragma unroll
+  for (int k = 0; k < 4; ++k) bias[k] = 0.f;
+  if (a.b) ld4v(a.b, true, c, bias);
 #pragma unroll
   for (int k = 0; k < 4; ++k)
 #pragma unroll
@@ -422,9 +425,10 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const ConvArgs a, co
 #pragma unroll
       for (int j = 0; j < kMaxTaps; ++j)
         if (j == a.taps - 1) wl = w[k][j];
-      o[k] = siluf(acc[k] + wl * cur[k]);
+      const float z = acc[k] + wl * cur[k];
+      o[k] = c + k >= a.silu_from ? siluf(z) : z;
     }
-    if (slot >= 0) st4(a.out + (size_t)t * a.C + c, o);
+    if (slot >= 0) st4((TO*)a.out + (size_t)t * a.C + c, o);
 #pragma unroll
     for (int j = 0; j < kMaxTaps - 2; ++j)
       if (j < a.taps - 2) {
@@ -838,23 +842,29 @@ void launch_route_sigmoid(int32_t* ids, float* w, const void* h, int h_stride, b
                                                       E, top, groups, keep, group_top);
 }
 
-void launch_conv_silu(float* out, const void* proj, int proj_stride, int off, bool f32,
-                      void* state, const float* w, const float* b, const int32_t* seq_slot,
-                      const int64_t* positions, const int32_t* q_start, int T, int B, int C,
-                      int taps, hipStream_t s) {
+void launch_conv_silu(void* out, bool out_f32, const void* proj, int proj_stride, int off, bool f32,
+                      int silu_from, void* state, const float* w, const float* b,
+                      const int32_t* seq_slot, const int64_t* positions, const int32_t* q_start,
+                      int T, int B, int C, int taps, hipStream_t s) {
   if (T <= 0) return;
-  ConvArgs a{out, proj, state, w, b, seq_slot, positions, q_start, proj_stride, off, C, taps, T, B};
-  const dim3 g1(T, (C + 255) / 256), g2(B, (C + 255) / 256), g4((T + (q_start ? kConvRows : 1) - 1) / (q_start ? kConvRows : 1), (C / 4 + 255) / 256);
+  ConvArgs a{out, proj, state, w, b, seq_slot, positions, q_start, proj_stride, off, C, taps, T, B,
+             silu_from};
   const int RB = q_start ? kConvRows : 1;
+  const dim3 g1(T, (C + 255) / 256), g2(B, (C + 255) / 256),
+      g4((T + RB - 1) / RB, (C / 4 + 255) / 256);
   const int es = f32 ? 4 : 2;
   const bool vec = C % 4 == 0 && off % 4 == 0 && proj_stride % 4 == 0 &&
                    (uintptr_t)proj % (4 * es) == 0 && (uintptr_t)state % (4 * es) == 0 &&
                    (uintptr_t)out % 16 == 0 && (uintptr_t)b % 16 == 0;
-  if (vec) {
-    if (f32) conv_silu_vec_kernel<float><<<g4, 256, 0, s>>>(a, RB);
-    else conv_silu_vec_kernel<bf16><<<g4, 256, 0, s>>>(a, RB);
-  } else if (f32) conv_silu_kernel<float><<<g1, 256, 0, s>>>(a);
-  else conv_silu_kernel<bf16><<<g1, 256, 0, s>>>(a);
+#define AKAP_CONV(TY, TO)                                              \
+  do {                                                                 \
+    if (vec) conv_silu_vec_kernel<TY, TO><<<g4, 256, 0, s>>>(a, RB);   \
+    else conv_silu_kernel<TY, TO><<<g1, 256, 0, s>>>(a);               \
+  } while (0)
+  if (f32) AKAP_CONV(float, float);
+  else if (out_f32) AKAP_CONV(bf16, float);
+  else AKAP_CONV(bf16, bf16);
+#undef AKAP_CONV
   if (taps > 1) {
     if (f32) conv_state_kernel<float><<<g2, 256, 0, s>>>(a);
     else conv_state_kernel<bf16><<<g2, 256, 0, s>>>(a);

@@ -140,9 +140,12 @@ SeqArgs seq_args(int64_t T, const Tensor& seq_slot, const Tensor& positions,
   return a;
 }
 
-void conv_silu(Tensor out, Tensor proj, int64_t off, Tensor conv_w, Tensor conv_b, Tensor state,
-               Tensor seq_slot, Tensor positions, std::optional<Tensor> q_start) {
-  CHECK_GPU(out); CHECK_GPU(proj); CHECK_GPU(state); CHECK_F32(out); CHECK_CONTIG(out);
+void conv_silu(Tensor out, Tensor proj, int64_t off, Tensor conv_w, std::optional<Tensor> conv_b,
+               Tensor state, Tensor seq_slot, Tensor positions, std::optional<Tensor> q_start,
+               int64_t silu_from) {
+  CHECK_GPU(out); CHECK_GPU(proj); CHECK_GPU(state); CHECK_CONTIG(out);
+  TORCH_CHECK(out.scalar_type() == at::kFloat || out.scalar_type() == proj.scalar_type(),
+              "conv_silu: out must be fp32 or of proj's type");
   CHECK_LAST_CONTIG(proj); CHECK_CONTIG(state);
   TORCH_CHECK(conv_w.dim() == 2 && out.dim() == 2 && proj.dim() == 2, "conv_silu: shapes");
   const int64_t T = proj.size(0), C = conv_w.size(0), taps = conv_w.size(1);
@@ -154,8 +157,9 @@ void conv_silu(Tensor out, Tensor proj, int64_t off, Tensor conv_w, Tensor conv_
                   (taps == 1 || state.size(1) == taps - 1), "conv_silu: state [slots, taps - 1, C]");
   const SeqArgs sa = seq_args(T, seq_slot, positions, q_start);
   const c10::DeviceGuard g(proj.device());
-  akap_stream::launch_conv_silu(out.data_ptr<float>(), proj.data_ptr(), (int)proj.stride(0),
-                                (int)off, is_f32(proj, "proj"), state.data_ptr(),
+  akap_stream::launch_conv_silu(out.data_ptr(), is_f32(out, "out"), proj.data_ptr(),
+                                (int)proj.stride(0), (int)off, is_f32(proj, "proj"),
+                                (int)silu_from, state.data_ptr(),
                                 f32_vec(conv_w, C * taps, "conv_w"), f32_vec(conv_b, C, "conv_b"),
                                 sa.slot, sa.pos, sa.q_start, sa.T, sa.B, (int)C, (int)taps,
                                 cur_stream());
@@ -393,8 +397,9 @@ TORCH_LIBRARY_FRAGMENT(akap_stream, m) {
         "-> ()");
   m.def("route_sigmoid(Tensor(a!) ids, Tensor(b!) w, Tensor h, Tensor router, int groups, "
         "int keep, int group_top) -> ()");
-  m.def("conv_silu(Tensor(a!) out, Tensor proj, int off, Tensor conv_w, Tensor conv_b, "
-        "Tensor(b!) state, Tensor seq_slot, Tensor positions, Tensor? q_start) -> ()");
+  m.def("conv_silu(Tensor(a!) out, Tensor proj, int off, Tensor conv_w, Tensor? conv_b, "
+        "Tensor(b!) state, Tensor seq_slot, Tensor positions, Tensor? q_start, "
+        "int silu_from=0) -> ()");
   m.def("selective_scan(Tensor(a!) y, Tensor xbc, Tensor proj, int dt_off, Tensor dt_bias, "
         "Tensor a_log, Tensor d_skip, Tensor(b!) state, Tensor seq_slot, Tensor positions, "
         "Tensor? q_start, int H, int V, int N, int G) -> ()");

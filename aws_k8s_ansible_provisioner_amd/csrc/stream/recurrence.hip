@@ -1,0 +1,448 @@
+// Recurrences over a matrix state S [D, V] per head and live sequence: linear attention with a
+// fixed decay per head, matrix memory with exponential gates (mLSTM), and the gated delta rule;
+// and the head norm + output gate that follows them.
+//
+// Gates, decays, step sizes, unit norms, the running maximum and the whole state are fp32
+// whatever the storage type; every size is a run-time argument.
+#include "../kernels/common.h"
+#include "stream.h"
+
+namespace akap_stream {
+
+using akap::bf16;
+using akap::block_sum;
+
+namespace {
+
+template <typename T>
+__device__ __forceinline__ float ldf(const T* p) { return (float)*p; }
+template <typename T>
+__device__ __forceinline__ void stf(T* p, float v) { *p = (T)v; }
+
+__device__ __forceinline__ void ld4(const float* p, float (&v)[4]) {
+  const float4 a = *(const float4*)p;
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+__device__ __forceinline__ void ld4(const bf16* p, float (&v)[4]) {
+  const akap::bf16x4 a = *(const akap::bf16x4*)p;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] = (float)a[i];
+}
+
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __expf(-z)); }
+__device__ __forceinline__ float gatef(float z, int silu) { return silu ? z * sigmoidf(z) : sigmoidf(z); }
+__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+// ------------------------------------------------------------------ scan
+// One workgroup per (sequence, head, VB state columns), at most 256 threads.  A thread keeps
+// VR = 4 neighbouring state columns and, of their D rows, DREG / 4 groups of four (group j of lane
+// part `part` covers d = 4 (j DP + part) ..+4, so the DP lanes of a column group read and write
+// consecutive 16-byte pieces of the stored state and of the staged rows).  Rows are staged TC at
+// a time; the recurrence then runs over them without a barrier: the DP lanes of a column group
+// add their partial sums by lane exchange.  The normaliser of the matrix memory is one more
+// column that every column group carries along (its D entries are spread over the same lanes).
+// For the delta rule q and k stay as staged: the reciprocals of their lengths, which are scalars
+// per token, multiply the sums and the update.
+constexpr int kVR = 4;
+constexpr int kDreg = 16;
+constexpr int kTokens = 16;
+
+template <typename T, int MODE>
+__global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
+  extern __shared__ __align__(16) float lds[];
+  constexpr int NJ = kDreg / 4;
+  const int DP = p.DP, DPD = DP * kDreg, TC = p.TC, VP = (p.VB + 3) & ~3;
+  float* qs = lds;                        // [TC][DPD]
+  float* ks = qs + TC * DPD;              // [TC][DPD]
+  float* vs = ks + TC * DPD;              // [TC][VP]
+  float* os = vs + TC * VP;               // [TC][VP]
+  float* g0 = os + TC * VP;               // [TC] decay of the state
+  float* g1 = g0 + TC;                    // [TC] input scale | beta
+  float* g2 = g1 + TC;                    // [TC] e^-m | 1 / |q|
+  float* g3 = g2 + TC;                    // [TC] 1 / |k|
+  float* mrun = g3 + TC;                  // [4] running maximum
+  const int b = blockIdx.x, h = blockIdx.y, c_lo = blockIdx.z * p.VB;
+  const int nv = min(p.VB, p.V - c_lo);   // columns of this workgroup
+  const int r0 = p.q_start ? p.q_start[b] : b;
+  const int r1 = p.q_start ? p.q_start[b + 1] : b + 1;
+  if (r1 <= r0) return;
+  const int slot = p.seq_slot[r0];
+  if (slot < 0 || slot >= p.num_slots) return;
+  const int tid = threadIdx.x, nt = blockDim.x;
+  const int hq = h / (p.H / p.G);
+  const int v0 = (tid / DP) * kVR, part = tid % DP;
+  const bool fresh = p.positions[r0] == 0;
+  float* sbase = p.state + (((size_t)slot * p.H + h) * p.V + c_lo) * p.D;
+  float* nbase = MODE == kMatrixMemory ? p.n_state + ((size_t)slot * p.H + h) * p.D : nullptr;
+  const bool vec = (p.D & 3) == 0;
+  auto load4 = [&](const float* sp, int d) {
+    float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (vec) {
+      if (d < p.D) t = *(const float4*)sp;
+    } else {
+      if (d < p.D) t.x = sp[0];
+      if (d + 1 < p.D) t.y = sp[1];
+      if (d + 2 < p.D) t.z = sp[2];
+      if (d + 3 < p.D) t.w = sp[3];
+    }
+    return t;
+  };
+  auto store4 = [&](float* sp, int d, float x, float y, float z, float w) {
+    if (vec) {
+      if (d < p.D) *(float4*)sp = make_float4(x, y, z, w);
+    } else {
+      if (d < p.D) sp[0] = x;
+      if (d + 1 < p.D) sp[1] = y;
+      if (d + 2 < p.D) sp[2] = z;
+      if (d + 3 < p.D) sp[3] = w;
+    }
+  };
+  float S[kVR][kDreg], N[kDreg];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int d = 4 * (j * DP + part);
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) {
+      float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (!fresh && v0 + r < nv) t = load4(sbase + (size_t)(v0 + r) * p.D + d, d);
+      S[r][4 * j] = t.x; S[r][4 * j + 1] = t.y; S[r][4 * j + 2] = t.z; S[r][4 * j + 3] = t.w;
+    }
+    float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (MODE == kMatrixMemory && !fresh) t = load4(nbase + d, d);
+    N[4 * j] = t.x; N[4 * j + 1] = t.y; N[4 * j + 2] = t.z; N[4 * j + 3] = t.w;
+  }
+  if (MODE == kMatrixMemory && tid == 0)
+    mrun[0] = fresh ? 0.f : p.m_state[(size_t)slot * p.H + h];
+  const float pa = p.pa[h], pb = MODE == kDecay ? 0.f : p.pb[h];
+  const float ea = MODE == kDelta ? expf(pa) : 0.f;
+  // 16-byte staging: every slice starts and every row strides at a multiple of 4 elements
+  const bool vstage = ((p.D | p.V | c_lo | p.qkv_stride | p.q_off | p.k_off | p.v_off) & 3) == 0 &&
+                      ((uintptr_t)p.qkv & 15) == 0;
+  const float qsc = MODE == kDelta ? 1.0f : p.q_scale;   // the delta rule scales with 1 / |q|
+  const bool act = p.act != 0;
+  auto on = [&](float z) { return act ? z * sigmoidf(z) : z; };
+  int LPT = 64;                           // lanes per token of the per-token phases
+  while (LPT * TC > nt && LPT > 1) LPT >>= 1;
+  for (int c0 = r0; c0 < r1; c0 += TC) {
+    const int n = min(TC, r1 - c0);
+    if (vstage) {
+      const int Q4 = DPD >> 2;
+      for (int e = tid; e < n * Q4; e += nt) {
+        const int tk = e / Q4, d = (e - tk * Q4) << 2;
+        const T* row = (const T*)p.qkv + (size_t)(c0 + tk) * p.qkv_stride;
+        float q4[4] = {0.f, 0.f, 0.f, 0.f}, k4[4] = {0.f, 0.f, 0.f, 0.f};
+        if (d < p.D) {
+          ld4(row + p.q_off + hq * p.D + d, q4);
+          ld4(row + p.k_off + hq * p.D + d, k4);
+        }
+        *(float4*)(qs + tk * DPD + d) =
+            make_float4(on(q4[0]) * qsc, on(q4[1]) * qsc, on(q4[2]) * qsc, on(q4[3]) * qsc);
+        *(float4*)(ks + tk * DPD + d) = make_float4(on(k4[0]), on(k4[1]), on(k4[2]), on(k4[3]));
+      }
+      const int V4 = VP >> 2;
+      for (int e = tid; e < n * V4; e += nt) {
+        const int tk = e / V4, c = (e - tk * V4) << 2;
+        float v4[4] = {0.f, 0.f, 0.f, 0.f};
+        if (c < nv)
+          ld4((const T*)p.qkv + (size_t)(c0 + tk) * p.qkv_stride + p.v_off + h * p.V + c_lo + c, v4);
+        *(float4*)(vs + tk * VP + c) = make_float4(on(v4[0]), on(v4[1]), on(v4[2]), on(v4[3]));
+      }
+    } else {
+      for (int e = tid; e < n * DPD; e += nt) {
+        const int tk = e / DPD, d = e % DPD;
+        const T* row = (const T*)p.qkv + (size_t)(c0 + tk) * p.qkv_stride;
+        qs[e] = d < p.D ? on(ldf(row + p.q_off + hq * p.D + d)) * qsc : 0.f;
+        ks[e] = d < p.D ? on(ldf(row + p.k_off + hq * p.D + d)) : 0.f;
+      }
+      for (int e = tid; e < n * VP; e += nt) {
+        const int tk = e / VP, c = e % VP;
+        vs[e] = c < nv ? on(ldf((const T*)p.qkv + (size_t)(c0 + tk) * p.qkv_stride + p.v_off +
+                                h * p.V + c_lo + c))
+                       : 0.f;
+      }
+    }
+    if (tid < n) {
+      const T* row = (const T*)p.proj + (size_t)(c0 + tid) * p.proj_stride;
+      if (MODE == kDecay) {
+        g0[tid] = pa;
+      } else if (MODE == kMatrixMemory) {
+        const float f = p.cap * tanhf((ldf(row + p.a_off + h) + pa) / p.cap);
+        g0[tid] = -softplusf(-f);
+        g1[tid] = p.cap * tanhf((ldf(row + p.b_off + h) + pb) / p.cap);
+      } else {
+        g0[tid] = expf(-ea * softplusf(ldf(row + p.a_off + h) + pb));
+        g1[tid] = 1.0f / (1.0f + expf(-ldf(row + p.b_off + h)));
+      }
+    }
+    __syncthreads();
+    if (MODE == kMatrixMemory) {
+      if (tid == 0) {
+        float m = mrun[0];
+        for (int tk = 0; tk < n; ++tk) {
+          const float f = g0[tk], i = g1[tk], m2 = fmaxf(f + m, i);
+          g0[tk] = expf(f + m - m2);
+          g1[tk] = expf(i - m2);
+          g2[tk] = expf(-m2);
+          m = m2;
+        }
+        mrun[0] = m;
+      }
+      __syncthreads();
+    } else if (MODE == kDelta) {
+      for (int tk = tid / LPT; tk < n; tk += nt / LPT) {
+        const int ln = tid % LPT;
+        float sq = 0.f, sk = 0.f;
+        for (int d = ln; d < p.D; d += LPT) {
+          const float a = qs[tk * DPD + d], c = ks[tk * DPD + d];
+          sq += a * a;
+          sk += c * c;
+        }
+        for (int o = LPT >> 1; o > 0; o >>= 1) {
+          sq += __shfl_xor(sq, o, 64);
+          sk += __shfl_xor(sk, o, 64);
+        }
+        if (ln == 0) {
+          g2[tk] = p.q_scale / sqrtf(sq + 1e-6f);
+          g3[tk] = 1.0f / sqrtf(sk + 1e-6f);
+        }
+      }
+      __syncthreads();
+    }
+    // the recurrence
+    for (int tk = 0; tk < n; ++tk) {
+      float4 vv = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (v0 < VP) vv = *(const float4*)(vs + tk * VP + v0);
+      float vr[kVR] = {vv.x, vv.y, vv.z, vv.w};
+      const float* kq = ks + tk * DPD + 4 * part;
+      const float* qq = qs + tk * DPD + 4 * part;
+      const float dec = g0[tk];
+      float acc[kVR] = {0.f, 0.f, 0.f, 0.f};
+      float accn = 0.f;
+      if (MODE == kDelta) {
+        float kk[kDreg];
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          const float4 k4 = *(const float4*)(kq + 4 * j * DP);
+          kk[4 * j] = k4.x; kk[4 * j + 1] = k4.y; kk[4 * j + 2] = k4.z; kk[4 * j + 3] = k4.w;
+        }
+        float seen[kVR] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < kDreg; ++i)
+#pragma unroll
+          for (int r = 0; r < kVR; ++r) {
+            S[r][i] *= dec;
+            seen[r] = fmaf(S[r][i], kk[i], seen[r]);
+          }
+        for (int o = DP >> 1; o > 0; o >>= 1) {
+#pragma unroll
+          for (int r = 0; r < kVR; ++r) seen[r] += __shfl_xor(seen[r], o, 64);
+        }
+        const float beta = g1[tk], ik = g3[tk];
+#pragma unroll
+        for (int r = 0; r < kVR; ++r) vr[r] = beta * (vr[r] - ik * seen[r]) * ik;
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          const float4 q4 = *(const float4*)(qq + 4 * j * DP);
+          const float qv[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int r = 0; r < kVR; ++r) {
+              S[r][4 * j + i] = fmaf(kk[4 * j + i], vr[r], S[r][4 * j + i]);
+              acc[r] = fmaf(S[r][4 * j + i], qv[i], acc[r]);
+            }
+        }
+      } else {
+        if (MODE == kMatrixMemory) {
+          const float add = g1[tk];
+#pragma unroll
+          for (int r = 0; r < kVR; ++r) vr[r] *= add;
+        }
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          const float4 k4 = *(const float4*)(kq + 4 * j * DP);
+          const float4 q4 = *(const float4*)(qq + 4 * j * DP);
+          const float kv[4] = {k4.x, k4.y, k4.z, k4.w}, qv[4] = {q4.x, q4.y, q4.z, q4.w};
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+#pragma unroll
+            for (int r = 0; r < kVR; ++r) {
+              S[r][4 * j + i] = fmaf(dec, S[r][4 * j + i], kv[i] * vr[r]);
+              acc[r] = fmaf(S[r][4 * j + i], qv[i], acc[r]);
+            }
+            if (MODE == kMatrixMemory) {
+              N[4 * j + i] = fmaf(dec, N[4 * j + i], kv[i] * g1[tk]);
+              accn = fmaf(N[4 * j + i], qv[i], accn);
+            }
+          }
+        }
+      }
+      for (int o = DP >> 1; o > 0; o >>= 1) {
+#pragma unroll
+        for (int r = 0; r < kVR; ++r) acc[r] += __shfl_xor(acc[r], o, 64);
+        if (MODE == kMatrixMemory) accn += __shfl_xor(accn, o, 64);
+      }
+      float f = 1.0f;
+      if (MODE == kMatrixMemory) f = 1.0f / (fmaxf(fabsf(accn), g2[tk]) + 1e-6f);
+      if (MODE == kDelta) f = g2[tk];
+      if (v0 < VP && part == 0)
+        *(float4*)(os + tk * VP + v0) = make_float4(acc[0] * f, acc[1] * f, acc[2] * f, acc[3] * f);
+    }
+    __syncthreads();
+    if (p.raw) {
+      for (int e = tid; e < n * nv; e += nt) {
+        const int tk = e / nv, c = e - tk * nv;
+        p.raw[((size_t)(c0 + tk) * p.H + h) * p.V + c_lo + c] = os[tk * VP + c];
+      }
+    } else {
+      // the head norm over its V entries, the weights and the output gate: LPT lanes per token
+      for (int tk = tid / LPT; tk < n; tk += nt / LPT) {
+        const int ln = tid % LPT;
+        float ss = 0.f;
+        for (int c = ln; c < p.V; c += LPT) {
+          const float f = os[tk * VP + c];
+          ss += f * f;
+        }
+        for (int o = LPT >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+        const float inv = 1.0f / sqrtf(ss / (float)p.V + p.eps);
+        const T* g = (const T*)p.proj + (size_t)(c0 + tk) * p.proj_stride + p.g_off + h * p.V;
+        T* o = (T*)p.out + (size_t)(c0 + tk) * p.out_stride + h * p.V;
+        for (int c = ln; c < p.V; c += LPT)
+          stf(o + c, os[tk * VP + c] * inv * p.norm_w[h * p.V + c] * gatef(ldf(g + c), p.gate_act));
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int d = 4 * (j * DP + part);
+#pragma unroll
+    for (int r = 0; r < kVR; ++r)
+      if (v0 + r < nv)
+        store4(sbase + (size_t)(v0 + r) * p.D + d, d, S[r][4 * j], S[r][4 * j + 1],
+               S[r][4 * j + 2], S[r][4 * j + 3]);
+    if (MODE == kMatrixMemory && v0 == 0 && blockIdx.z == 0)
+      store4(nbase + d, d, N[4 * j], N[4 * j + 1], N[4 * j + 2], N[4 * j + 3]);
+  }
+  if (MODE == kMatrixMemory && tid == 0 && blockIdx.z == 0)
+    p.m_state[(size_t)slot * p.H + h] = mrun[0];
+}
+
+// ------------------------------------------------------------------ head norm + output gate
+// one workgroup of four waves per row: a part per wave when there are several, else all threads
+template <typename T>
+__global__ __launch_bounds__(256) void norm_gate_kernel(T* __restrict__ out, int out_stride,
+                                                        const float* __restrict__ y,
+                                                        const T* __restrict__ gate, int gate_stride,
+                                                        const float* __restrict__ w,
+                                                        const float* __restrict__ den,
+                                                        const float* __restrict__ floor, int silu,
+                                                        int n, int groups, float eps, int vec) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, part = n / groups;
+  const float* yr = y + (size_t)t * n;
+  const T* gr = gate + (size_t)t * gate_stride;
+  T* o = out + (size_t)t * out_stride;
+  const int wave = threadIdx.x >> 6;
+  const bool shared = groups == 1;
+  const int step = shared ? 256 : 64, ln = shared ? threadIdx.x : (threadIdx.x & 63);
+  for (int g = shared ? 0 : wave; g < groups; g += shared ? 1 : 4) {
+    const int c0 = g * part;
+    float scale = 1.0f;
+    if (den) {
+      const size_t i = (size_t)t * groups + g;
+      scale = 1.0f / (fmaxf(fabsf(den[i]), floor[i]) + 1e-6f);
+    }
+    float ss = 0.f;
+    if (vec) {
+      for (int c = ln * 4; c < part; c += step * 4) {
+        const float4 v = *(const float4*)(yr + c0 + c);
+        ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+      }
+    } else {
+      for (int c = ln; c < part; c += step) ss += yr[c0 + c] * yr[c0 + c];
+    }
+    ss = shared ? block_sum(ss, scratch) : akap::wave_sum(ss);
+    // eps inside the root of the divided values
+    const float inv = scale / sqrtf(ss * scale * scale / (float)part + eps);
+    if (vec) {
+      for (int c = ln * 4; c < part; c += step * 4) {
+        const float4 v = *(const float4*)(yr + c0 + c);
+        const float4 wv = *(const float4*)(w + c0 + c);
+        float gv[4];
+        ld4(gr + c0 + c, gv);
+        T r[4] = {(T)(v.x * inv * wv.x * gatef(gv[0], silu)), (T)(v.y * inv * wv.y * gatef(gv[1], silu)),
+                  (T)(v.z * inv * wv.z * gatef(gv[2], silu)), (T)(v.w * inv * wv.w * gatef(gv[3], silu))};
+        __builtin_memcpy(o + c0 + c, r, sizeof(r));
+      }
+    } else {
+      for (int c = ln; c < part; c += step)
+        stf(o + c0 + c, yr[c0 + c] * inv * w[c0 + c] * gatef(ldf(gr + c0 + c), silu));
+    }
+  }
+}
+
+// lanes per column group and columns per workgroup
+void scan_shape(int D, int V, int* dp, int* vb) {
+  int p = 1;
+  while (p * kDreg < D) p <<= 1;
+  *dp = p;
+  const int cols = kVR * (256 / p);
+  *vb = V <= cols ? V : cols;
+}
+
+}  // namespace
+
+// ================================================================== launchers
+bool recurrence_supported(int D, int V) { return D >= 1 && D <= 64 * kDreg && V >= 1; }
+
+bool recurrence_fused(int D, int V) {
+  int dp, vb;
+  scan_shape(D, V, &dp, &vb);
+  return vb == V;
+}
+
+void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s) {
+  if (p.num_seqs <= 0) return;
+  scan_shape(p.D, p.V, &p.DP, &p.VB);
+  const int groups = (p.VB + kVR - 1) / kVR;
+  const int nt = ((groups * p.DP + 63) / 64) * 64;
+  const int vp = (p.VB + 3) & ~3;
+  p.TC = p.q_start ? kTokens : 1;
+  auto need = [&](int tc) {
+    return (size_t)(tc * (2 * p.DP * kDreg + 2 * vp + 4) + 4) * sizeof(float);
+  };
+  while (p.TC > 1 && need(p.TC) > 65536) p.TC >>= 1;
+  const size_t lds = need(p.TC);
+  const dim3 grid(p.num_seqs, p.H, (p.V + p.VB - 1) / p.VB);
+#define AKAP_REC(TY)                                                                          \
+  do {                                                                                        \
+    if (mode == kDecay) recurrence_kernel<TY, kDecay><<<grid, nt, lds, s>>>(p);               \
+    else if (mode == kMatrixMemory)                                                           \
+      recurrence_kernel<TY, kMatrixMemory><<<grid, nt, lds, s>>>(p);                          \
+    else recurrence_kernel<TY, kDelta><<<grid, nt, lds, s>>>(p);                              \
+  } while (0)
+  if (f32) AKAP_REC(float);
+  else AKAP_REC(bf16);
+#undef AKAP_REC
+}
+
+void launch_norm_gate(void* out, int out_stride, const float* y, const void* gate, int gate_stride,
+                      const float* w, const float* den, const float* floor, bool f32, int act,
+                      int rows, int n, int groups, float eps, hipStream_t s) {
+  if (rows <= 0) return;
+  const int part = n / groups, es = f32 ? 4 : 2;
+  auto al = [](const void* p, int bytes) { return ((uintptr_t)p % bytes) == 0; };
+  const int vec = part % 4 == 0 && out_stride % 4 == 0 && gate_stride % 4 == 0 && al(y, 16) &&
+                  al(w, 16) && al(out, 4 * es) && al(gate, 4 * es);
+  if (f32)
+    norm_gate_kernel<float><<<rows, 256, 0, s>>>((float*)out, out_stride, y, (const float*)gate,
+                                                 gate_stride, w, den, floor, act, n, groups, eps,
+                                                 vec);
+  else
+    norm_gate_kernel<bf16><<<rows, 256, 0, s>>>((bf16*)out, out_stride, y, (const bf16*)gate,
+                                                gate_stride, w, den, floor, act, n, groups, eps,
+                                                vec);
+}
+
+}  // namespace akap_stream

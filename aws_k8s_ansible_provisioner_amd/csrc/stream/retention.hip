@@ -169,6 +169,18 @@ __global__ __launch_bounds__(256) void post_norm_add_norm_kernel(
       sx += f * f;
     }
   }
+  if (!next_w) {   // the next sublayer reads the stream itself
+    for (int c = c0; c < d; c += step) {
+      if (VEC) {
+        float f[8];
+        ld8(ra + c, f);
+        st8(o + c, f);
+      } else {
+        stf(o + c, ra[c]);
+      }
+    }
+    return;
+  }
   sx = block_sum(sx, scratch);
   const float ix = 1.0f / sqrtf(sx * inv_d + eps);
   for (int c = c0; c < d; c += step) {
@@ -201,7 +213,11 @@ __global__ __launch_bounds__(256) void head_norm_cache_kernel(HeadNormParams p) 
     T* dst;
     int n, vstep = 1;
     bool norm;
+    const float* w = nullptr;
+    bool rot = false;
     if (u < p.H) {
+      w = p.q_w;
+      rot = p.cos_sin != nullptr;
       src = row + p.q_off + u * p.D;
       dst = (T*)p.q_out + ((size_t)t * p.H + u) * p.D;
       n = p.D;
@@ -209,6 +225,8 @@ __global__ __launch_bounds__(256) void head_norm_cache_kernel(HeadNormParams p) 
     } else if (u < p.H + p.G) {
       if (!cached) continue;
       const int g = u - p.H;
+      w = p.k_w;
+      rot = p.cos_sin != nullptr;
       src = row + p.k_off + g * p.D;
       dst = (T*)p.k_cache + ((size_t)(blk * p.G + g) * p.BS + off) * p.D;
       n = p.D;
@@ -235,7 +253,24 @@ __global__ __launch_bounds__(256) void head_norm_cache_kernel(HeadNormParams p) 
       ss = wave_sum(ss);
       inv = 1.0f / sqrtf(ss / (float)n + p.eps);
     }
-    for (int c = lane; c < n; c += 64) stf(dst + c * vstep, ldf(src + c) * inv);
+    if (rot) {
+      // rotate-half pairs (i, i + half) of the normed and weighted head, a pair per lane
+      const int half = p.rot_dims >> 1;
+      const int64_t pos = p.positions[t];
+      const float* cs = p.cos_sin + (size_t)(pos < p.max_pos ? pos : p.max_pos - 1) * p.rot_dims;
+      for (int i = lane; i < half; i += 64) {
+        const float a = ldf(src + i) * inv * (w ? w[i] : 1.0f);
+        const float b = ldf(src + i + half) * inv * (w ? w[i + half] : 1.0f);
+        const float c = cs[i], s = cs[half + i];
+        stf(dst + i, a * c - b * s);
+        stf(dst + i + half, b * c + a * s);
+      }
+      for (int c = p.rot_dims + lane; c < n; c += 64)
+        stf(dst + c, ldf(src + c) * inv * (w ? w[c] : 1.0f));
+      continue;
+    }
+    for (int c = lane; c < n; c += 64)
+      stf(dst + c * vstep, ldf(src + c) * inv * (w ? w[c] : 1.0f));
   }
 }
 

@@ -17,8 +17,9 @@ void launch_embed_scaled(float* out, const int64_t* ids, const void* table, bool
 void launch_add_norm(void* out, bool out_f32, float* x, const void* y, bool y_f32, int y_stride,
                      const void* bias, float mult, const float* w, int rows, int d,
                      int out_stride, float eps, hipStream_t s);
-void launch_relu2(void* out, const void* x, bool f32, int rows, int F, int x_stride,
-                  int out_stride, hipStream_t s);
+// act 0: relu(x)^2, 1: gelu in its tanh form
+void launch_activation(void* out, const void* x, bool f32, int act, int rows, int F, int x_stride,
+                       int out_stride, hipStream_t s);
 
 struct ProjParams {
   const void* proj;   // [T, N] fused projection rows
@@ -162,7 +163,7 @@ void launch_moe_combine(float* out, const void* y, const int32_t* inv, const int
 
 // ---- sandwich norms, retention, head-mixed attention, logit-top-k routing (retention.hip) -------
 // m = ya, or (rms(ya) wa + rms(yb) wb) / 2 when yb is given; x (fp32 rows of d) <- x + rms(m)
-// post_w (fresh: x is not read); out = rms(x) next_w.  Every weight has a stride of 1 (d
+// post_w (fresh: x is not read); out = rms(x) next_w (next_w null: out = x).  Every weight has a stride of 1 (d
 // entries) or 0 (one number).  ya / yb are both fp32 or both of the activation type.
 void launch_post_norm_add_norm(void* out, bool out_f32, int out_stride, float* x, const void* ya,
                                int ya_stride, const void* yb, int yb_stride, bool y_f32,
@@ -181,6 +182,11 @@ struct HeadNormParams {
   int64_t num_slots;  // NB * BS
   float eps;
   bool norm_qk, norm_v;
+  const float* q_w;   // [D] norm weights shared by the heads, or null
+  const float* k_w;
+  const float* cos_sin;       // [max_pos, rot_dims] = [cos | sin], rotate-half pairs, or null
+  const int64_t* positions;   // [T] (with cos_sin)
+  int max_pos, rot_dims;
 };
 void launch_head_norm_cache(const HeadNormParams& p, bool f32, hipStream_t s);
 
@@ -272,10 +278,11 @@ void launch_gate_group_norm(void* out, int out_stride, const float* y, const voi
 void launch_route_sigmoid(int32_t* ids, float* w, const void* h, int h_stride, bool f32,
                           const float* router, int rows, int d, int E, int top, int groups,
                           int keep, int group_top, hipStream_t s);
-// causal per-channel convolution + silu of columns [off, off + C) of proj, then the sequences'
-// last taps - 1 inputs to their slots; B sequences (q_start null: B = T, one row each)
-void launch_conv_silu(float* out, const void* proj, int proj_stride, int off, bool f32,
-                      void* state, const float* w, const float* b, const int32_t* seq_slot,
+// causal per-channel convolution of columns [off, off + C) of proj (b null: no bias; silu on the
+// channels from silu_from on), then the sequences' last taps - 1 inputs to their slots; out fp32
+// or proj's type; B sequences (q_start null: B = T, one row each)
+void launch_conv_silu(void* out, bool out_f32, const void* proj, int proj_stride, int off, bool f32,
+                      int silu_from, void* state, const float* w, const float* b, const int32_t* seq_slot,
                       const int64_t* positions, const int32_t* q_start, int T, int B, int C,
                       int taps, hipStream_t s);
 // state rows a thread of the one-column scan keeps in registers (at most 64); can a head of V
@@ -287,6 +294,43 @@ void launch_selective_scan(float* y, const float* xbc, const void* proj, int pro
                            const float* d_skip, float* state, const int32_t* seq_slot,
                            const int64_t* positions, const int32_t* q_start, int T, int B, int H,
                            int V, int N, int G, hipStream_t s);
+
+// ---- matrix-state recurrences (recurrence.hip) ---------------------------------------------------
+enum RecurrenceMode { kDecay = 0, kMatrixMemory = 1, kDelta = 2 };
+
+struct RecurrenceParams {
+  void* out;             // normed and gated heads, rows of out_stride; or
+  int out_stride;
+  float* raw;            // [T, H V]: the heads as they leave the state (raw given: out unused)
+  const void* qkv;       // rows of qkv_stride: q, k (G heads of D) and v (H heads of V)
+  int qkv_stride, q_off, k_off, v_off;
+  int act;               // 1: silu on q, k and v
+  const void* proj;      // rows of proj_stride: output gate, gates of the recurrence
+  int proj_stride, g_off, a_off, b_off;
+  const float* pa;       // [H] decay | forget gate bias | A_log
+  const float* pb;       // [H] -     | input gate bias  | dt_bias
+  float cap, q_scale, eps;
+  float* state;          // [slots, H, V, D], transposed
+  float* n_state;        // [slots, H, D] (matrix memory)
+  float* m_state;        // [slots, H]
+  int num_slots;
+  const float* norm_w;   // [H V]
+  int gate_act;          // 0 sigmoid, 1 silu
+  const int32_t* seq_slot;
+  const int64_t* positions;
+  const int32_t* q_start;   // [num_seqs + 1] or null (row t is sequence t)
+  int num_seqs, H, G, D, V;
+  int VB, DP, TC;        // set by the launcher
+};
+// does a workgroup hold all state columns of a head (the head norm and gate can be fused)?
+bool recurrence_fused(int D, int V);
+bool recurrence_supported(int D, int V);
+void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s);
+// out = gnorm(y / (max(|den|, floor) + 1e-6)) * w * act(gate) over `groups` equal parts of the n
+// columns (den null: y itself; act 0 sigmoid, 1 silu)
+void launch_norm_gate(void* out, int out_stride, const float* y, const void* gate, int gate_stride,
+                      const float* w, const float* den, const float* floor, bool f32, int act,
+                      int rows, int n, int groups, float eps, hipStream_t s);
 
 // ---- window + pooled blocks attention (pooled_attention.hip) -----------------------------------
 struct RopeCacheParams {

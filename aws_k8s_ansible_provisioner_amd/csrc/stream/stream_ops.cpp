@@ -71,14 +71,16 @@ void add_norm(Tensor out, Tensor x, std::optional<Tensor> y, double mult, Tensor
                                (float)eps, cur_stream());
 }
 
-void relu2(Tensor out, Tensor x) {
+void activation(Tensor out, Tensor x, int act) {
   CHECK_GPU(out); CHECK_GPU(x); CHECK_LAST_CONTIG(out); CHECK_LAST_CONTIG(x);
-  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && out.sizes() == x.sizes(), "relu2: shapes");
-  TORCH_CHECK(out.scalar_type() == x.scalar_type(), "relu2: dtypes differ");
+  TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && out.sizes() == x.sizes(), "activation: shapes");
+  TORCH_CHECK(out.scalar_type() == x.scalar_type(), "activation: dtypes differ");
   const c10::DeviceGuard g(x.device());
-  akap_stream::launch_relu2(out.data_ptr(), x.data_ptr(), is_f32(x, "x"), (int)x.size(0),
+  akap_stream::launch_activation(out.data_ptr(), x.data_ptr(), is_f32(x, "x"), act, (int)x.size(0),
                             (int)x.size(1), (int)x.stride(0), (int)out.stride(0), cur_stream());
 }
+void relu2(Tensor out, Tensor x) { activation(out, x, 0); }
+void gelu_tanh(Tensor out, Tensor x) { activation(out, x, 1); }
 
 void check_cache(const Tensor& k_cache, const Tensor& v_cache, int64_t G, int64_t D) {
   CHECK_GPU(k_cache); CHECK_GPU(v_cache); CHECK_CONTIG(k_cache); CHECK_CONTIG(v_cache);
@@ -693,7 +695,7 @@ int weight_stride(const Tensor& w, int64_t d, const char* name) {
 
 void post_norm_add_norm(Tensor out, Tensor x, Tensor ya, std::optional<Tensor> yb,
                         std::optional<Tensor> wa, std::optional<Tensor> wb, Tensor post_w,
-                        Tensor next_w, double eps, bool fresh) {
+                        std::optional<Tensor> next_w, double eps, bool fresh) {
   CHECK_GPU(out); CHECK_GPU(x); CHECK_GPU(ya);
   CHECK_F32(x); CHECK_CONTIG(x); CHECK_LAST_CONTIG(out); CHECK_LAST_CONTIG(ya);
   TORCH_CHECK(x.dim() == 2 && out.dim() == 2 && out.sizes() == x.sizes() && ya.dim() == 2 &&
@@ -716,17 +718,19 @@ void post_norm_add_norm(Tensor out, Tensor x, Tensor ya, std::optional<Tensor> y
     wap = wa->data_ptr<float>();
     wbp = wb->data_ptr<float>();
   }
-  const int pws = weight_stride(post_w, d, "post_w"), nws = weight_stride(next_w, d, "next_w");
+  const int pws = weight_stride(post_w, d, "post_w"), nws = next_w.has_value() ? weight_stride(*next_w, d, "next_w") : 0;
   const c10::DeviceGuard g(x.device());
   akap_stream::launch_post_norm_add_norm(
       out.data_ptr(), is_f32(out, "out"), (int)out.stride(0), x.data_ptr<float>(), ya.data_ptr(),
       (int)ya.stride(0), ybp, ybs, yf, wap, was, wbp, wbs, post_w.data_ptr<float>(), pws,
-      next_w.data_ptr<float>(), nws, (int)rows, (int)d, (float)eps, fresh, cur_stream());
+      next_w.has_value() ? next_w->data_ptr<float>() : nullptr, nws, (int)rows, (int)d, (float)eps, fresh, cur_stream());
 }
 
 void head_norm_cache(Tensor proj, Tensor q_out, Tensor k_cache, Tensor v_cache, Tensor slots,
                      int64_t H, int64_t G, int64_t D, int64_t Dv, int64_t q_off, int64_t k_off,
-                     int64_t v_off, double eps, bool norm_qk, bool norm_v) {
+                     int64_t v_off, double eps, bool norm_qk, bool norm_v,
+                     std::optional<Tensor> q_w, std::optional<Tensor> k_w,
+                     std::optional<Tensor> cos_sin, std::optional<Tensor> positions) {
   CHECK_GPU(proj); CHECK_GPU(q_out); CHECK_GPU(k_cache); CHECK_GPU(v_cache); CHECK_GPU(slots);
   CHECK_LAST_CONTIG(proj); CHECK_CONTIG(q_out); CHECK_CONTIG(k_cache); CHECK_CONTIG(v_cache);
   CHECK_CONTIG(slots);
@@ -753,6 +757,27 @@ void head_norm_cache(Tensor proj, Tensor q_out, Tensor k_cache, Tensor v_cache, 
   p.q_off = q_off; p.k_off = k_off; p.v_off = v_off;
   p.num_slots = k_cache.size(0) * k_cache.size(2);
   p.eps = (float)eps; p.norm_qk = norm_qk; p.norm_v = norm_v;
+  p.q_w = p.k_w = p.cos_sin = nullptr;
+  p.positions = nullptr;
+  p.max_pos = p.rot_dims = 0;
+  for (const auto* w : {&q_w, &k_w})
+    if (w->has_value())
+      TORCH_CHECK((*w)->is_cuda() && (*w)->scalar_type() == at::kFloat && (*w)->is_contiguous() &&
+                      (*w)->numel() == D, "head_norm_cache: norm weights must be fp32 [D]");
+  if (q_w.has_value()) p.q_w = q_w->data_ptr<float>();
+  if (k_w.has_value()) p.k_w = k_w->data_ptr<float>();
+  if (cos_sin.has_value()) {
+    CHECK_GPU(*cos_sin); CHECK_F32(*cos_sin); CHECK_CONTIG(*cos_sin);
+    TORCH_CHECK(positions.has_value() && positions->is_cuda() &&
+                    positions->scalar_type() == at::kLong && positions->is_contiguous() &&
+                    positions->numel() >= T, "head_norm_cache: a rotation needs int64 positions");
+    TORCH_CHECK(cos_sin->dim() == 2 && cos_sin->size(0) >= 1 && cos_sin->size(1) % 2 == 0 &&
+                    cos_sin->size(1) <= D, "head_norm_cache: cos_sin must be [max_pos, dims <= D]");
+    p.cos_sin = cos_sin->data_ptr<float>();
+    p.positions = positions->data_ptr<int64_t>();
+    p.max_pos = cos_sin->size(0);
+    p.rot_dims = cos_sin->size(1);
+  }
   const c10::DeviceGuard g(proj.device());
   akap_stream::launch_head_norm_cache(p, f32, cur_stream());
 }
@@ -1005,6 +1030,7 @@ TORCH_LIBRARY(akap_stream, m) {
   m.def("add_norm(Tensor(a!) out, Tensor(b!) x, Tensor? y, float mult, Tensor w, float eps, "
         "Tensor? bias=None) -> ()");
   m.def("relu2(Tensor(a!) out, Tensor x) -> ()");
+  m.def("gelu_tanh(Tensor(a!) out, Tensor x) -> ()");
   m.def(
       "proj_norm_rope_cache(Tensor proj, Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, "
       "Tensor positions, Tensor slots, Tensor? cos_sin, Tensor q_w, Tensor k_w, int H, int G, "
@@ -1045,10 +1071,11 @@ TORCH_LIBRARY(akap_stream, m) {
   m.def("moe_combine(Tensor(a!) out, Tensor y, Tensor? inv, Tensor ids, Tensor w, Tensor h, "
         "int experts) -> ()");
   m.def("post_norm_add_norm(Tensor(a!) out, Tensor(b!) x, Tensor ya, Tensor? yb, Tensor? wa, "
-        "Tensor? wb, Tensor post_w, Tensor next_w, float eps, bool fresh) -> ()");
+        "Tensor? wb, Tensor post_w, Tensor? next_w, float eps, bool fresh) -> ()");
   m.def("head_norm_cache(Tensor proj, Tensor(a!) q_out, Tensor(b!) k_cache, Tensor(c!) v_cache, "
         "Tensor slots, int H, int G, int D, int Dv, int q_off, int k_off, int v_off, float eps, "
-        "bool norm_qk, bool norm_v) -> ()");
+        "bool norm_qk, bool norm_v, "
+        "Tensor? q_w=None, Tensor? k_w=None, Tensor? cos_sin=None, Tensor? positions=None) -> ()");
   m.def("retention(Tensor(a!) out, Tensor proj, int q_off, int k_off, int v_off, int g_off, "
         "Tensor(b!) state, Tensor seq_slot, Tensor positions, Tensor? q_start, Tensor? cos_sin, "
         "Tensor log2_decay, int H, int D, int V, float eps, Tensor(c!)? seg_buf=None, "
@@ -1095,6 +1122,7 @@ TORCH_LIBRARY_IMPL(akap_stream, CUDA, m) {
   m.impl("embed_scaled", &embed_scaled);
   m.impl("add_norm", &add_norm);
   m.impl("relu2", &relu2);
+  m.impl("gelu_tanh", &gelu_tanh);
   m.impl("proj_norm_rope_cache", &proj_norm_rope_cache);
   m.impl("sink_attention_prefill", &sink_attention_prefill);
   m.impl("sink_attention_decode", &sink_attention_decode);
