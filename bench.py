@@ -89,7 +89,8 @@ def parse():
                          "kernel table")
     ap.add_argument("--profile-steps", type=int, default=0,
                     help="extra untimed waves run after timing (for rocprofv3 captures)")
-    ap.add_argument("--compare-design", default=None, choices=["bidetar", "puputar", "sazepel", "mudepel"],
+    ap.add_argument("--compare-design", default=None, choices=["bidetar", "puputar", "sazepel", "mudepel",
+                                                               "papivik"],
                     help="instead of the serving wave: prefill and decode throughput of this "
                          "design at real layer sizes (random weights) beside the closest "
                          "existing model of equal size; prints one JSON line with the table")
@@ -117,6 +118,10 @@ COMPARE_SETS = {
     # and routed experts at the same width and depth, and the dense fp32-stream design
     "mudepel": [("mudepel-w2048", "sazepel-w2048"), ("mudepel-w4096", "sazepel-w4096"),
                 ("bidetar-w2048", None)],
+    # matrix-memory, linear-attention and attention + delta-rule layers beside the framework's
+    # two other hybrids of a recurrent state and an attention at the same width and depth
+    "papivik": [("papivik-w2048", "sazepel-w2048"), ("papivik-w4096", "sazepel-w4096"),
+                ("mudepel-w2048", None)],
 }
 
 

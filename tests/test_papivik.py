@@ -405,13 +405,15 @@ def test_bf16_stays_near(model, reference):
 
 
 def test_far_key_stands_out(tmp_path):
-    """One attention layer whose query at the last position matches the key of ONE distinctive
-    token far back, in a page of its own: leaving it out would move the logits."""
+    """One attention layer whose query at the last position matches its own key and that of ONE
+    equal token far back; the values' convolution takes the token before, so the two bring
+    different values: leaving the far key out moves the logits."""
     cfg = oracle.make_config(24, 40, [oracle.parallel_layer((2, 1, 8, 8), (1, 1, 4, 4), 4.0, 0,
-                                                            conv=(1, 1), scales=(1.0, 0.05))])
+                                                            conv=(2, 1), scales=(1.0, 0.05))])
     W = oracle.random_weights(cfg, seed=4)
-    for n in ("q", "k", "v"):
-        W[f"l0.mix.left.{n}.conv"] = torch.ones_like(W[f"l0.mix.left.{n}.conv"])
+    for n, taps in (("q", [0.0, 1.0]), ("k", [0.0, 1.0]), ("v", [1.0, 0.0])):
+        rows = W[f"l0.mix.left.{n}.conv"].shape[0]
+        W[f"l0.mix.left.{n}.conv"] = torch.tensor([taps] * rows, dtype=torch.bfloat16)
     W["l0.mix.left.q"][8:] = W["l0.mix.left.q"][:8]
     W["l0.mix.left.k"] = W["l0.mix.left.q"][:8].clone()
     for n in ("q.norm", "k.norm"):
@@ -477,7 +479,7 @@ def test_greedy_generation(model):
                        prompt_ids=prompts)
     W64 = oracle.as_f64(W)
     for p, o in zip(prompts, out):
-        assert list(o.token_ids) == greedy_reference(cfg, W64, p, 7)
+        assert list(o.output_ids) == greedy_reference(cfg, W64, p, 7)
 
 
 def test_trace_runner_command(model, reference, tmp_path):
