@@ -1,0 +1,548 @@
+// The recurrences of recurrence.hip for prompt chunks on the matrix cores (bf16 storage): a
+// sequence's rows are cut into chunks of 64 tokens, a first launch prepares every chunk of every
+// head side by side, a second one walks the chunks of a (sequence, head) with the fp32 state in
+// accumulator registers.
+//
+// With L_t the sum of the log decays from the chunk's start through token t, S0 the state before
+// the chunk, and c_s / d_t the scalars of a key and a query (input scale or 1 / |k|; q's scale
+// or that over |q|):
+//   o_t   = d_t e^(L_t) q_t S0 + sum_{s <= t} P_ts x_s,   P_ts = d_t e^(L_t - L_s) c_s (q_t . k_s)
+//   S_end = e^(L_end) S0 + sum_s k_s (e^(L_end - L_s) c_s x_s)^T
+// with x_s = v_s for the plain recurrences; for the delta rule x = u solves
+//   (I + A) u = beta v - beta e^L c (K S0),   A_ts = beta_t e^(L_t - L_s) c_t c_s (k_t . k_s), s < t
+// (the unit-vector recurrence with the lengths pulled out of the products), whose unit lower
+// triangular inverse depends on the keys and gates alone and is prepared per chunk.
+//
+// bf16 operands are the stored q, k, v (exact); every fp32 quantity that has to be an operand
+// (S0, P, u, the inverse) is split into a bf16 pair hi + lo, so products keep about 16 bits of
+// it; sums are fp32.
+//
+// Operand layouts (v_mfma_f32_32x32x16_bf16): an accumulator lane holds column l & 31 and rows
+// 8 i + 4 (l >> 5) + j in registers 4 i + j.  Read as the B operand of the next product, registers
+// 8 kb .. 8 kb + 7 are 8 of the 16 contraction indices of block kb, in the order
+// slot 8 hl + e <-> index 8 (e >> 2) + 4 hl + (e & 3).  A operands are stored in that order (a
+// fragment = 64 lanes x 8 elements, 1 KB, one 16-byte load per lane), so the state, the solved
+// rows and the outputs of one product feed the next without leaving the registers.
+#include "../kernels/common.h"
+#include "stream.h"
+
+namespace akap_stream {
+
+using akap::bf16;
+using akap::bf16x4;
+using akap::bf16x8;
+using akap::f32x16;
+
+namespace {
+
+constexpr int kC = 64;          // tokens of a chunk
+constexpr int kFrag = 512;      // elements of a fragment
+constexpr int kPT = 12;         // fragments of P (and of the inverse): 6 of hi, 6 of lo
+constexpr int kSc = 5 * kC;     // floats of scalars per (chunk, head)
+
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __expf(-z)); }
+__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+__device__ __forceinline__ f32x16 mfma(bf16x8 a, bf16x8 b, f32x16 c) {
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
+}
+
+__device__ __forceinline__ void split8(const float (&v)[8], bf16x8& hi, bf16x8& lo) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    hi[i] = (bf16)v[i];
+    lo[i] = (bf16)(v[i] - (float)hi[i]);
+  }
+}
+
+// entries of a chunk buffer: sequence b (counted from the first chunked one) owns those from
+// (first row - row0) / 64 + b on
+__device__ __forceinline__ int chunk_base(const int32_t* q_start, int b, int row0) {
+  return (q_start[b] - row0) / kC + b;
+}
+
+// ------------------------------------------------------------------ chunk preparation
+// One workgroup of four waves per (chunk, head).
+template <int MODE, int DT>
+__global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
+  constexpr int D = DT * 32, LS = D + 8, NKB = D / 16;
+  constexpr int AS = 68;
+  __shared__ __align__(16) bf16 qs[kC * LS];
+  __shared__ __align__(16) bf16 ks[kC * LS];
+  __shared__ __align__(16) float am[MODE == kDelta ? kC * AS : 4];
+  __shared__ float Ls[kC], ct[kC], cs[kC], bt[kC];
+  const RecurrenceParams& r = p.r;
+  const int h = blockIdx.y, entry = blockIdx.x;
+  int lo = 0, hi = r.num_seqs - 1;
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (chunk_base(r.q_start, mid, p.row0) <= entry) lo = mid; else hi = mid - 1;
+  }
+  const int b = lo;
+  const int first = r.q_start[b], end = r.q_start[b + 1];
+  const int r0 = first + (entry - chunk_base(r.q_start, b, p.row0)) * kC;
+  if (r0 < first || r0 >= end) return;
+  const int slot = r.seq_slot[first];
+  if (slot < 0 || slot >= r.num_slots) return;
+  const int n = min(kC, end - r0);
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, hl = lane >> 5, ln = lane & 31;
+  const int rep = r.H / r.G, hq = h / rep;
+  const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
+
+  // q and k of the chunk, activated, rows past its end zero
+  for (int e = tid; e < kC * (D / 8); e += 256) {
+    const int row = e / (D / 8), c = (e - row * (D / 8)) * 8;
+    bf16x8 q8, k8;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) q8[i] = k8[i] = (bf16)0.f;
+    if (row < n) {
+      const bf16* src = (const bf16*)r.qkv + (size_t)(r0 + row) * r.qkv_stride + hq * D + c;
+      q8 = *(const bf16x8*)(src + r.q_off);
+      k8 = *(const bf16x8*)(src + r.k_off);
+      if (MODE == kDecay && r.act) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const float a = (float)q8[i], c2 = (float)k8[i];
+          q8[i] = (bf16)(a * sigmoidf(a));
+          k8[i] = (bf16)(c2 * sigmoidf(c2));
+        }
+      }
+    }
+    *(bf16x8*)(qs + row * LS + c) = q8;
+    *(bf16x8*)(ks + row * LS + c) = k8;
+  }
+  __syncthreads();
+  if (MODE == kDelta) {
+    // lengths: four lanes per token
+    const int row = tid >> 2;
+    float sq = 0.f, sk = 0.f;
+    for (int c = (tid & 3) * 8; c < D; c += 32) {
+      const bf16x8 q8 = *(const bf16x8*)(qs + row * LS + c), k8 = *(const bf16x8*)(ks + row * LS + c);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        sq += (float)q8[i] * (float)q8[i];
+        sk += (float)k8[i] * (float)k8[i];
+      }
+    }
+    sq += __shfl_xor(sq, 1, 64);
+    sk += __shfl_xor(sk, 1, 64);
+    sq += __shfl_xor(sq, 2, 64);
+    sk += __shfl_xor(sk, 2, 64);
+    if ((tid & 3) == 0) {
+      ct[row] = r.q_scale / sqrtf(sq + 1e-6f);
+      cs[row] = 1.0f / sqrtf(sk + 1e-6f);
+    }
+    __syncthreads();
+  }
+  if (wave == 0) {
+    const int row = r0 + min(lane, n - 1);
+    const bool live = lane < n;
+    float la = 0.f, beta = 0.f, c_s = 1.f, d_t = r.q_scale;
+    if (MODE == kDecay) {
+      la = fmaxf(logf(r.pa[h]), -1e4f);
+    } else if (MODE == kMatrixMemory) {
+      la = p.la[(size_t)row * r.H + h];
+      c_s = p.lb[(size_t)row * r.H + h];
+    } else {
+      const bf16* pr = (const bf16*)r.proj + (size_t)row * r.proj_stride;
+      la = -expf(r.pa[h]) * softplusf((float)pr[r.a_off + h] + r.pb[h]);
+      beta = 1.0f / (1.0f + expf(-(float)pr[r.b_off + h]));
+      c_s = cs[lane];
+      d_t = ct[lane];
+    }
+    if (!live) { la = 0.f; beta = 0.f; c_s = 0.f; }
+    float L = la;
+    for (int o = 1; o < 64; o <<= 1) {
+      const float t = __shfl_up(L, o, 64);
+      if (lane >= o) L += t;
+    }
+    const float Lend = __shfl(L, 63, 64), eL = expf(L);
+    Ls[lane] = L;
+    ct[lane] = d_t;
+    cs[lane] = c_s;
+    bt[lane] = beta;
+    float* sc = p.sc + ch * kSc;
+    sc[lane] = eL * d_t;
+    sc[kC + lane] = expf(Lend - L) * c_s;
+    sc[2 * kC + lane] = beta;
+    sc[3 * kC + lane] = beta * eL * c_s;
+    sc[4 * kC + lane] = expf(Lend);
+  }
+  __syncthreads();
+  // P (and A): the transposed product, key tile x query tile, so that a lane holds a query's row
+  if (wave < 3) {
+    const int ts = wave == 2, tt = wave > 0;
+    f32x16 qk, kk;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) qk[i] = kk[i] = 0.f;
+#pragma unroll
+    for (int kb = 0; kb < NKB; ++kb) {
+      const bf16x8 a = *(const bf16x8*)(ks + (ts * 32 + ln) * LS + kb * 16 + hl * 8);
+      const bf16x8 q = *(const bf16x8*)(qs + (tt * 32 + ln) * LS + kb * 16 + hl * 8);
+      qk = mfma(a, q, qk);
+      if (MODE == kDelta) {
+        const bf16x8 k = *(const bf16x8*)(ks + (tt * 32 + ln) * LS + kb * 16 + hl * 8);
+        kk = mfma(a, k, kk);
+      }
+    }
+    const int t = tt * 32 + ln;
+    const float Lt = Ls[t], dt = ct[t], at = MODE == kDelta ? bt[t] * cs[t] : 0.f;
+    bf16* pf = (bf16*)p.pf + ch * kPT * kFrag;
+#pragma unroll
+    for (int kbl = 0; kbl < 2; ++kbl) {
+      float v[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int s = ts * 32 + kbl * 16 + 8 * (e >> 2) + 4 * hl + (e & 3);
+        const float w = expf(fminf(Lt - Ls[s], 0.f)) * cs[s];
+        v[e] = s <= t ? qk[kbl * 8 + e] * w * dt : 0.f;
+        if (MODE == kDelta) am[t * AS + s] = s < t ? kk[kbl * 8 + e] * w * at : 0.f;
+      }
+      bf16x8 vh, vl;
+      split8(v, vh, vl);
+      const int idx = tt == 0 ? kbl : 2 + ts * 2 + kbl;
+      *(bf16x8*)(pf + idx * kFrag + lane * 8) = vh;
+      *(bf16x8*)(pf + (6 + idx) * kFrag + lane * 8) = vl;
+    }
+  }
+  // fragments of q, k (rows = tokens) and of k transposed (rows = dimensions), once per key head
+  if (h % rep == 0) {
+    bf16* qf = (bf16*)p.qf + cg * 2 * NKB * kFrag;
+    bf16* kf = (bf16*)p.kf + cg * 2 * NKB * kFrag;
+    bf16* kt = (bf16*)p.ktf + cg * DT * 4 * kFrag;
+    constexpr int kQ = 2 * NKB, kAll = kQ + (MODE == kDelta ? kQ : 0);
+    for (int f = wave; f < kAll; f += 4) {
+      const int g = f < kQ ? f : f - kQ;
+      const bf16* src = (f < kQ ? qs : ks) + ((g / NKB) * 32 + ln) * LS + (g % NKB) * 16 + 4 * hl;
+      const bf16x4 x = *(const bf16x4*)src, y = *(const bf16x4*)(src + 8);
+      bf16x8 o;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) { o[i] = x[i]; o[4 + i] = y[i]; }
+      *(bf16x8*)((f < kQ ? qf : kf) + g * kFrag + lane * 8) = o;
+    }
+    for (int f = wave; f < DT * 4; f += 4) {
+      const int d = (f >> 2) * 32 + ln, kb = f & 3;
+      bf16x8 o;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] = ks[(kb * 16 + 8 * (e >> 2) + 4 * hl + (e & 3)) * LS + d];
+      *(bf16x8*)(kt + f * kFrag + lane * 8) = o;
+    }
+  }
+  if (MODE != kDelta) return;
+  __syncthreads();
+  // the inverse of I + A by forward substitution, a column per lane of one wave
+  if (wave == 0) {
+    float x[kC];
+#pragma unroll
+    for (int i = 0; i < kC; ++i) {
+      float a0 = lane == i ? 1.f : 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
+#pragma unroll
+      for (int j = 0; j < i; j += 4) {
+        const float4 a = *(const float4*)(am + i * AS + j);
+        a0 = fmaf(-a.x, x[j], a0);
+        if (j + 1 < i) a1 = fmaf(-a.y, x[j + 1], a1);
+        if (j + 2 < i) a2 = fmaf(-a.z, x[j + 2], a2);
+        if (j + 3 < i) a3 = fmaf(-a.w, x[j + 3], a3);
+      }
+      x[i] = (a0 + a1) + (a2 + a3);
+    }
+#pragma unroll
+    for (int i = 0; i < kC; ++i) am[i * AS + lane] = x[i];
+  }
+  __syncthreads();
+  bf16* tf = (bf16*)p.tf + ch * kPT * kFrag;
+  for (int f = wave; f < 6; f += 4) {
+    const int row = (f < 2 ? 0 : 32) + ln, kb = f < 2 ? f : f - 2;
+    const float* src = am + row * AS + kb * 16 + 4 * hl;
+    const float4 x = *(const float4*)src, y = *(const float4*)(src + 8);
+    const float v[8] = {x.x, x.y, x.z, x.w, y.x, y.y, y.z, y.w};
+    bf16x8 vh, vl;
+    split8(v, vh, vl);
+    *(bf16x8*)(tf + f * kFrag + lane * 8) = vh;
+    *(bf16x8*)(tf + (6 + f) * kFrag + lane * 8) = vl;
+  }
+}
+
+// ------------------------------------------------------------------ walk over the chunks
+// a wave per (sequence, head, 32 state columns); no barriers, the four waves of a workgroup only
+// share their operand loads through the caches
+__device__ __forceinline__ bf16x8 frag(const bf16* base, int i, int lane) {
+  return *(const bf16x8*)(base + i * kFrag + lane * 8);
+}
+
+template <int MODE, int DT>
+__global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
+  constexpr int D = DT * 32, NKB = D / 16;
+  const RecurrenceParams& r = p.r;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, hl = lane >> 5, ln = lane & 31;
+  const int h = blockIdx.y, b = blockIdx.z;
+  const int cols = r.V + (MODE == kMatrixMemory ? 1 : 0);   // column V: the normaliser
+  const int c0 = (blockIdx.x * 4 + wave) * 32;
+  const int first = r.q_start[b], end = r.q_start[b + 1];
+  if (c0 >= cols || end <= first) return;
+  const int slot = r.seq_slot[first];
+  if (slot < 0 || slot >= r.num_slots) return;
+  const int rep = r.H / r.G, hq = h / rep;
+  const int c = c0 + ln;
+  const bool isv = c < r.V, isn = MODE == kMatrixMemory && c == r.V;
+  float* sp = isn ? r.n_state + ((size_t)slot * r.H + h) * D
+                  : r.state + (((size_t)slot * r.H + h) * r.V + (isv ? c : 0)) * D;
+  f32x16 S[DT];
+  const bool carry = r.positions[first] != 0 && (isv || isn);
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (carry) x = *(const float4*)(sp + dt * 32 + 8 * i + 4 * hl);
+      S[dt][4 * i] = x.x; S[dt][4 * i + 1] = x.y; S[dt][4 * i + 2] = x.z; S[dt][4 * i + 3] = x.w;
+    }
+  int entry = chunk_base(r.q_start, b, p.row0);
+  for (int r0 = first; r0 < end; r0 += kC, ++entry) {
+    const int n = min(kC, end - r0);
+    const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
+    const bf16* qf = (bf16*)p.qf + cg * 2 * NKB * kFrag;
+    const bf16* kf = (bf16*)p.kf + cg * 2 * NKB * kFrag;
+    const bf16* kt = (bf16*)p.ktf + cg * DT * 4 * kFrag;
+    const bf16* pf = (bf16*)p.pf + ch * kPT * kFrag;
+    const bf16* tf = (bf16*)p.tf + ch * kPT * kFrag;
+    const float* sc = p.sc + ch * kSc;
+    // values of this lane's column, rows as in an accumulator
+    bf16 vv[32];
+#pragma unroll
+    for (int i = 0; i < 32; ++i) {
+      const int row = min((i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3), n - 1);
+      bf16 v = (bf16)(isn ? 1.f : 0.f);
+      if (isv) v = ((const bf16*)r.qkv)[(size_t)(r0 + row) * r.qkv_stride + r.v_off + h * r.V + c];
+      vv[i] = v;
+    }
+    // products with the state before the chunk
+    f32x16 O[2], X[2];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) O[0][i] = O[1][i] = X[0][i] = X[1][i] = 0.f;
+#pragma unroll
+    for (int kb = 0; kb < NKB; ++kb) {
+      float s[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s[e] = S[kb >> 1][(kb & 1) * 8 + e];
+      bf16x8 sh, sl;
+      split8(s, sh, sl);
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        if (MODE == kDelta) {
+          const bf16x8 a = frag(kf, t * NKB + kb, lane);
+          X[t] = mfma(a, sh, X[t]);
+          X[t] = mfma(a, sl, X[t]);
+        }
+        const bf16x8 a = frag(qf, t * NKB + kb, lane);
+        O[t] = mfma(a, sh, O[t]);
+        O[t] = mfma(a, sl, O[t]);
+      }
+    }
+    if (MODE == kDecay && r.act) {
+#pragma unroll
+      for (int i = 0; i < 32; ++i) {
+        const float z = (float)vv[i];
+        vv[i] = (bf16)(z * sigmoidf(z));
+      }
+    }
+    if (MODE == kDelta) {
+      // u = (I + A)^-1 (beta v - beta e^L c (K S0))
+      bf16x8 xh[4], xl[4];
+#pragma unroll
+      for (int kb = 0; kb < 4; ++kb) {
+        float x[8];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+          const int row = kb * 16 + 8 * i + 4 * hl;
+          const float4 be = *(const float4*)(sc + 2 * kC + row);
+          const float4 bk = *(const float4*)(sc + 3 * kC + row);
+          const float b4[4] = {be.x, be.y, be.z, be.w}, k4[4] = {bk.x, bk.y, bk.z, bk.w};
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            x[4 * i + j] = b4[j] * (float)vv[kb * 8 + 4 * i + j] -
+                           k4[j] * X[kb >> 1][(kb & 1) * 8 + 4 * i + j];
+        }
+        split8(x, xh[kb], xl[kb]);
+      }
+#pragma unroll
+      for (int i = 0; i < 16; ++i) X[0][i] = X[1][i] = 0.f;
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int kb = 0; kb < 2 + 2 * t; ++kb) {
+          const int idx = t == 0 ? kb : 2 + kb;
+          const bf16x8 ah = frag(tf, idx, lane), al = frag(tf, 6 + idx, lane);
+          X[t] = mfma(ah, xh[kb], X[t]);
+          X[t] = mfma(ah, xl[kb], X[t]);
+          X[t] = mfma(al, xh[kb], X[t]);
+        }
+    }
+    // outputs: the part through S0 scaled by row, the part inside the chunk
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float4 w = *(const float4*)(sc + t * 32 + 8 * i + 4 * hl);
+        O[t][4 * i] *= w.x; O[t][4 * i + 1] *= w.y; O[t][4 * i + 2] *= w.z; O[t][4 * i + 3] *= w.w;
+      }
+    bf16x8 wh[4], wl[4];        // what enters the state: hi + lo of e^(L_end - L) c x
+#pragma unroll
+    for (int kb = 0; kb < 4; ++kb) {
+      bf16x8 uh, ul;
+      float w[8];
+      if (MODE == kDelta) {
+        float u[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) w[e] = u[e] = X[kb >> 1][(kb & 1) * 8 + e];
+        split8(u, uh, ul);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          uh[e] = vv[kb * 8 + e];
+          w[e] = (float)vv[kb * 8 + e];
+        }
+      }
+#pragma unroll
+      for (int t = kb >> 1; t < 2; ++t) {
+        const int idx = t == 0 ? kb : 2 + kb;
+        const bf16x8 ah = frag(pf, idx, lane), al = frag(pf, 6 + idx, lane);
+        O[t] = mfma(ah, uh, O[t]);
+        O[t] = mfma(al, uh, O[t]);
+        if (MODE == kDelta) O[t] = mfma(ah, ul, O[t]);
+      }
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const float4 z = *(const float4*)(sc + kC + kb * 16 + 8 * i + 4 * hl);
+        w[4 * i] *= z.x; w[4 * i + 1] *= z.y; w[4 * i + 2] *= z.z; w[4 * i + 3] *= z.w;
+      }
+      split8(w, wh[kb], wl[kb]);
+    }
+    // the state after the chunk
+    const float eend = sc[4 * kC];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) S[dt][i] *= eend;
+#pragma unroll
+      for (int kb = 0; kb < 4; ++kb) {
+        const bf16x8 a = frag(kt, dt * 4 + kb, lane);
+        S[dt] = mfma(a, wh[kb], S[dt]);
+        S[dt] = mfma(a, wl[kb], S[dt]);
+      }
+    }
+    if (isv || isn) {
+      float* o = isn ? p.den + (size_t)r0 * r.H + h : r.raw + ((size_t)r0 * r.H + h) * r.V + c;
+      const size_t os = isn ? (size_t)r.H : (size_t)r.H * r.V;
+#pragma unroll
+      for (int i = 0; i < 32; ++i) {
+        const int row = (i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3);
+        if (row < n) o[row * os] = O[i >> 4][i & 15];
+      }
+    }
+  }
+  if (isv || isn) {
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        *(float4*)(sp + dt * 32 + 8 * i + 4 * hl) =
+            make_float4(S[dt][4 * i], S[dt][4 * i + 1], S[dt][4 * i + 2], S[dt][4 * i + 3]);
+  }
+}
+
+// ------------------------------------------------------------------ gates of the matrix memory
+// a wave per (sequence, head), 64 tokens a turn: the running maximum m_t = max(f_t + m_(t-1), i_t)
+// is a scan over the maps m -> max(F + m, I), composed by lane exchange
+__global__ __launch_bounds__(64) void memory_gates_kernel(ChunkParams p) {
+  const RecurrenceParams& r = p.r;
+  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  const int first = r.q_start[b], end = r.q_start[b + 1];
+  if (end <= first) return;
+  const int slot = r.seq_slot[first];
+  if (slot < 0 || slot >= r.num_slots) return;
+  float* ms = r.m_state + (size_t)slot * r.H + h;
+  float m = r.positions[first] == 0 ? 0.f : *ms;
+  const float fb = r.pa[h], ib = r.pb[h], icap = 1.0f / r.cap;
+  for (int r0 = first; r0 < end; r0 += 64) {
+    const int row = r0 + lane;
+    const bool live = row < end;
+    float f = 0.f, i = -INFINITY;      // past the end: the identity
+    if (live) {
+      const bf16* pr = (const bf16*)r.proj + (size_t)row * r.proj_stride;
+      f = -softplusf(-r.cap * tanhf(((float)pr[r.a_off + h] + fb) * icap));
+      i = r.cap * tanhf(((float)pr[r.b_off + h] + ib) * icap);
+    }
+    float F = f, I = i;
+    for (int o = 1; o < 64; o <<= 1) {
+      const float Fp = __shfl_up(F, o, 64), Ip = __shfl_up(I, o, 64);
+      if (lane >= o) {
+        I = fmaxf(F + Ip, I);
+        F += Fp;
+      }
+    }
+    const float mt = fmaxf(F + m, I);
+    float mp = __shfl_up(mt, 1, 64);
+    if (lane == 0) mp = m;
+    if (live) {
+      const size_t at = (size_t)row * r.H + h;
+      p.la[at] = f + mp - mt;
+      p.lb[at] = expf(i - mt);
+      p.floor[at] = expf(-mt);
+    }
+    m = __shfl(mt, 63, 64);
+  }
+  if (lane == 0) *ms = m;
+}
+
+}  // namespace
+
+// ================================================================== launchers
+bool chunk_supported(int D) { return D == 32 || D == 64 || D == 96 || D == 128 || D == 256; }
+
+// bf16 elements / floats of a workspace of `chunks` chunk entries
+void chunk_workspace(int mode, int chunks, int H, int G, int D, int64_t* halves, int64_t* floats) {
+  const int64_t g = (int64_t)chunks * G, hh = (int64_t)chunks * H;
+  *halves = g * (int64_t)(D / 16) * 2 * kFrag * (mode == kDelta ? 2 : 1) +
+            g * (D / 32) * 4 * kFrag + hh * kPT * kFrag * (mode == kDelta ? 2 : 1);
+  *floats = hh * kSc;
+}
+
+void launch_chunk_recurrence(ChunkParams p, int mode, uint16_t* halves, float* floats,
+                             hipStream_t s) {
+  const RecurrenceParams& r = p.r;
+  if (r.num_seqs <= 0 || p.num_chunks <= 0) return;
+  const int64_t g = (int64_t)p.num_chunks * r.G, hh = (int64_t)p.num_chunks * r.H;
+  const int64_t rows = g * (r.D / 16) * 2 * kFrag;
+  uint16_t* w = halves;
+  p.qf = w; w += rows;
+  p.kf = w;
+  if (mode == kDelta) w += rows;
+  p.ktf = w; w += g * (r.D / 32) * 4 * kFrag;
+  p.pf = w; w += hh * kPT * kFrag;
+  p.tf = w;
+  p.sc = floats;
+  const int cols = r.V + (mode == kMatrixMemory ? 1 : 0);
+  const dim3 pg(p.num_chunks, r.H), wg((cols + 127) / 128, r.H, r.num_seqs);
+  if (mode == kMatrixMemory) memory_gates_kernel<<<dim3(r.num_seqs, r.H), 64, 0, s>>>(p);
+#define AKAP_CH(M, T)                                \
+  do {                                               \
+    chunk_prep_kernel<M, T><<<pg, 256, 0, s>>>(p);   \
+    chunk_walk_kernel<M, T><<<wg, 256, 0, s>>>(p);   \
+  } while (0)
+#define AKAP_CHD(M)                    \
+  switch (r.D / 32) {                  \
+    case 1: AKAP_CH(M, 1); break;      \
+    case 2: AKAP_CH(M, 2); break;      \
+    case 3: AKAP_CH(M, 3); break;      \
+    case 4: AKAP_CH(M, 4); break;      \
+    default: AKAP_CH(M, 8); break;     \
+  }
+  if (mode == kDecay) AKAP_CHD(kDecay)
+  else if (mode == kMatrixMemory) AKAP_CHD(kMatrixMemory)
+  else AKAP_CHD(kDelta)
+#undef AKAP_CHD
+#undef AKAP_CH
+}
+
+}  // namespace akap_stream

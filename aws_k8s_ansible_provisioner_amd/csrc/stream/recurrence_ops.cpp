@@ -1,5 +1,5 @@
 // torch custom-op registrations (namespace `akap_stream`, a fragment beside stream_ops.cpp) of
-// the kernels in recurrence.hip.
+// the kernels in recurrence.hip and recurrence_mfma.hip.
 //
 // Like the other ops: every op launches on the caller's current HIP stream, allocates nothing
 // and never synchronises (hipGraph-capturable).  Operand shapes are checked here, on the host,
@@ -145,6 +145,58 @@ void recurrence(int64_t mode, Tensor out, std::optional<Tensor> raw, Tensor qkv,
   akap_stream::launch_recurrence(p, (int)mode, is_f32(qkv, "qkv"), cur_stream());
 }
 
+// the chunked form over the sequences from first_seq on (their first row is row0, on the host)
+void chunk_recurrence(int64_t mode, Tensor raw, Tensor qkv, int64_t q_off, int64_t k_off,
+                      int64_t v_off, int64_t act, Tensor proj, int64_t a_off, int64_t b_off,
+                      Tensor pa, std::optional<Tensor> pb, double cap, double q_scale,
+                      Tensor state, std::optional<Tensor> n_state, std::optional<Tensor> m_state,
+                      Tensor seq_slot, Tensor positions, Tensor q_start, int64_t first_seq,
+                      int64_t row0, int64_t H, int64_t G, int64_t D, int64_t V,
+                      std::optional<Tensor> memory, Tensor halves, Tensor floats) {
+  auto p = recurrence_params(mode, qkv, q_off, k_off, v_off, act, proj, a_off, b_off, pa, pb, cap,
+                             q_scale, state, n_state, m_state, seq_slot, positions, q_start, H, G,
+                             D, V);
+  const int64_t T = qkv.size(0);
+  TORCH_CHECK(qkv.scalar_type() == at::kBFloat16 && akap_stream::chunk_supported((int)D),
+              "chunk_recurrence: bf16 heads of 32 / 64 / 96 / 128 / 256");
+  TORCH_CHECK(((q_off | k_off | qkv.stride(0)) & 7) == 0 &&
+                  ((uintptr_t)qkv.data_ptr() & 15) == 0, "chunk_recurrence: 16-byte aligned rows");
+  TORCH_CHECK(first_seq >= 0 && first_seq < q_start.numel() && row0 >= 0 && row0 <= T,
+              "chunk_recurrence: first_seq / row0");
+  p.q_start += first_seq;
+  p.num_seqs -= (int)first_seq;
+  TORCH_CHECK(p.num_seqs <= 65535, "chunk_recurrence: at most 65535 sequences");
+  akap_stream::ChunkParams c{};
+  p.raw = f32_ptr(raw, T * H * V, "raw");
+  c.r = p;
+  c.row0 = (int)row0;
+  c.num_chunks = (int)((T - row0) / 64 + p.num_seqs);
+  if (mode == akap_stream::kMatrixMemory) {
+    TORCH_CHECK(memory.has_value(), "chunk_recurrence: the matrix memory needs [4, T, H] floats");
+    float* m = f32_ptr(*memory, 4 * T * H, "memory");
+    c.la = m; c.lb = m + T * H; c.den = m + 2 * T * H; c.floor = m + 3 * T * H;
+  }
+  int64_t nh = 0, nf = 0;
+  akap_stream::chunk_workspace((int)mode, c.num_chunks, (int)H, (int)G, (int)D, &nh, &nf);
+  TORCH_CHECK(halves.is_cuda() && halves.is_contiguous() &&
+                  halves.scalar_type() == at::kBFloat16 && halves.numel() >= nh &&
+                  ((uintptr_t)halves.data_ptr() & 15) == 0 && floats.is_cuda() &&
+                  floats.is_contiguous() && floats.scalar_type() == at::kFloat &&
+                  floats.numel() >= nf && ((uintptr_t)floats.data_ptr() & 15) == 0,
+              "chunk_recurrence: workspace");
+  const c10::DeviceGuard g(qkv.device());
+  akap_stream::launch_chunk_recurrence(c, (int)mode, (uint16_t*)halves.data_ptr(),
+                                       floats.data_ptr<float>(), cur_stream());
+}
+
+bool chunk_supported(int64_t D) { return akap_stream::chunk_supported((int)D); }
+
+std::vector<int64_t> chunk_workspace(int64_t mode, int64_t chunks, int64_t H, int64_t G, int64_t D) {
+  int64_t nh = 0, nf = 0;
+  akap_stream::chunk_workspace((int)mode, (int)chunks, (int)H, (int)G, (int)D, &nh, &nf);
+  return {nh, nf};
+}
+
 bool recurrence_fused(int64_t D, int64_t V) {
   return akap_stream::recurrence_fused((int)D, (int)V);
 }
@@ -159,10 +211,18 @@ TORCH_LIBRARY_FRAGMENT(akap_stream, m) {
         "float q_scale, Tensor(c!) state, Tensor(d!)? n_state, Tensor(e!)? m_state, Tensor norm_w, "
         "int g_off, int gate_act, float eps, Tensor seq_slot, Tensor positions, Tensor? q_start, "
         "int H, int G, int D, int V) -> ()");
+  m.def("chunk_recurrence(int mode, Tensor(a!) raw, Tensor qkv, int q_off, int k_off, int v_off, "
+        "int act, Tensor proj, int a_off, int b_off, Tensor pa, Tensor? pb, float cap, "
+        "float q_scale, Tensor(b!) state, Tensor(c!)? n_state, Tensor(d!)? m_state, "
+        "Tensor seq_slot, Tensor positions, Tensor q_start, int first_seq, int row0, int H, int G, "
+        "int D, int V, Tensor(e!)? memory, Tensor(f!) halves, Tensor(g!) floats) -> ()");
+  m.def("chunk_supported(int D) -> bool", &chunk_supported);
+  m.def("chunk_workspace(int mode, int chunks, int H, int G, int D) -> int[]", &chunk_workspace);
   m.def("recurrence_fused(int D, int V) -> bool", &recurrence_fused);
 }
 
 TORCH_LIBRARY_IMPL(akap_stream, CUDA, m) {
   m.impl("norm_gate", &norm_gate);
   m.impl("recurrence", &recurrence);
+  m.impl("chunk_recurrence", &chunk_recurrence);
 }

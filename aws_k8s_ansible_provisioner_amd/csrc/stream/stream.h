@@ -326,6 +326,29 @@ struct RecurrenceParams {
 bool recurrence_fused(int D, int V);
 bool recurrence_supported(int D, int V);
 void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s);
+// chunked matrix-core form for prompt portions (recurrence_mfma.hip, bf16): the sequences of r
+// (q_start given, pointing at the first chunked sequence, whose first row is row0); r.raw takes
+// the heads as they leave the state (the matrix memory's still undivided, with den = n . q and
+// floor = e^-m per row and head)
+struct ChunkParams {
+  RecurrenceParams r;
+  int row0, num_chunks;   // chunk entries: rows / 64 + sequences
+  float* la;              // [T, H] log decay / input scale (matrix memory only)
+  float* lb;
+  float* den;
+  float* floor;
+  // workspace, set by the launcher: operand fragments per (chunk, key head) and (chunk, head),
+  // scalars per (chunk, head, token)
+  uint16_t* qf;
+  uint16_t* kf;
+  uint16_t* ktf;
+  uint16_t* pf;
+  uint16_t* tf;
+  float* sc;
+};
+bool chunk_supported(int D);
+void chunk_workspace(int mode, int chunks, int H, int G, int D, int64_t* halves, int64_t* floats);
+void launch_chunk_recurrence(ChunkParams p, int mode, uint16_t* halves, float* floats, hipStream_t s);
 // out = gnorm(y / (max(|den|, floor) + 1e-6)) * w * act(gate) over `groups` equal parts of the n
 // columns (den null: y itself; act 0 sigmoid, 1 silu)
 void launch_norm_gate(void* out, int out_stride, const float* y, const void* gate, int gate_stride,

@@ -943,23 +943,52 @@ def norm_gate(out: torch.Tensor, y: torch.Tensor, gate: torch.Tensor, w: torch.T
 _REC_MODE = {"decay": 0, "mlstm": 1, "delta": 2}
 
 
+# steps whose sequences (past the leading single rows) hold at least this many rows on average take
+# the chunked form
+CHUNK_MIN_ROWS = 16
+
+
 def _recurrence(mode: str, out, qkv, q_off, k_off, v_off, act, proj, gates: tuple, pa, pb, cap,
                 q_scale, state, n_state, m_state, norm_w, g_off, gate_act, norm_all, eps,
-                seq_slot, positions, q_start, H, G, D, V) -> None:
-    """GPU form of the recurrences below: the scan kernel (one workgroup per sequence, head and
-    block of state columns, state in registers) with the head norm and the gate fused where a
-    workgroup holds a whole head, else followed by norm_gate."""
-    T = qkv.shape[0]
-    fuse = not norm_all and torch.ops.akap_stream.recurrence_fused(D, V)
+                seq_slot, positions, q_start, H, G, D, V, first_seq) -> None:
+    """GPU form of the recurrences below.  Prompt portions in bf16, at head sizes the matrix-core
+    kernels take: chunks of 64 tokens prepared side by side, then walked with the state in
+    accumulators, followed by norm_gate.  Everything else (single rows, fp32, other sizes): the
+    scan kernel (one workgroup per sequence, head and block of state columns, state in
+    registers) with the head norm and the gate fused where a workgroup holds a whole head, else
+    followed by norm_gate."""
+    ns = torch.ops.akap_stream
+    T, m = qkv.shape[0], _REC_MODE[mode]
+    args = (qkv, q_off, k_off, v_off, act, proj, gates[0], gates[1], pa, pb, float(cap),
+            float(q_scale), state, n_state, m_state)
+    groups = 1 if norm_all else H
+    if q_start is not None and qkv.dtype == torch.bfloat16 and ns.chunk_supported(D) \
+            and q_off % 8 == 0 and k_off % 8 == 0 and qkv.stride(0) % 8 == 0 \
+            and qkv.data_ptr() % 16 == 0:
+        seqs = q_start.numel() - 1 - first_seq
+        if seqs > 0 and T - first_seq >= CHUNK_MIN_ROWS * seqs:
+            nd = first_seq
+            if nd:      # the leading single rows of a mixed step
+                _recurrence(mode, out[:nd], qkv[:nd], q_off, k_off, v_off, act, proj[:nd], gates,
+                            pa, pb, cap, q_scale, state, n_state, m_state, norm_w, g_off, gate_act,
+                            norm_all, eps, seq_slot[:nd], positions[:nd], None, H, G, D, V, 0)
+            dev = qkv.device
+            nh, nf = ns.chunk_workspace(m, (T - nd) // 64 + seqs, H, G, D)
+            raw = torch.empty(T, H * V, dtype=torch.float32, device=dev)
+            mem = torch.empty(4, T, H, dtype=torch.float32, device=dev) if mode == "mlstm" else None
+            ns.chunk_recurrence(m, raw, *args, seq_slot, positions, q_start, nd, nd, H, G, D, V,
+                                mem, torch.empty(nh, dtype=torch.bfloat16, device=dev),
+                                torch.empty(nf, dtype=torch.float32, device=dev))
+            norm_gate(out[nd:], raw[nd:], proj[nd:, g_off:g_off + H * V], norm_w, groups, eps,
+                      gate_act, mem[2, nd:] if mem is not None else None,
+                      mem[3, nd:] if mem is not None else None)
+            return
+    fuse = not norm_all and ns.recurrence_fused(D, V)
     raw = None if fuse else torch.empty(T, H * V, dtype=torch.float32, device=qkv.device)
-    torch.ops.akap_stream.recurrence(_REC_MODE[mode], out, raw, qkv, q_off, k_off, v_off, act,
-                                     proj, gates[0], gates[1], pa, pb, float(cap), float(q_scale),
-                                     state, n_state, m_state, norm_w, g_off,
-                                     1 if gate_act == "silu" else 0, float(eps), seq_slot,
-                                     positions, q_start, H, G, D, V)
+    ns.recurrence(m, out, raw, *args, norm_w, g_off, 1 if gate_act == "silu" else 0, float(eps),
+                  seq_slot, positions, q_start, H, G, D, V)
     if raw is not None:
-        norm_gate(out, raw, proj[:, g_off:g_off + H * V], norm_w, 1 if norm_all else H, eps,
-                  gate_act)
+        norm_gate(out, raw, proj[:, g_off:g_off + H * V], norm_w, groups, eps, gate_act)
 
 
 def _heads(x: torch.Tensor, off: int, n: int, size: int) -> torch.Tensor:
@@ -989,7 +1018,7 @@ def linear_attention(out: torch.Tensor, proj: torch.Tensor, q_off: int, k_off: i
     if _native(proj):
         _recurrence("decay", out, proj, q_off, k_off, v_off, 1 if act == "silu" else 0, proj,
                     (0, 0), decay, None, 0.0, 1.0, state, None, None, norm_w, g_off, gate,
-                    norm == "all", eps, seq_slot, positions, q_start, H, H, D, V)
+                    norm == "all", eps, seq_slot, positions, q_start, H, H, D, V, first_seq)
         return
     T = proj.shape[0]
     q, k, v = _heads(proj, q_off, H, D), _heads(proj, k_off, H, D), _heads(proj, v_off, H, V)
@@ -1022,7 +1051,7 @@ def matrix_memory(out: torch.Tensor, proj: torch.Tensor, q_off: int, k_off: int,
     if _native(proj):
         _recurrence("mlstm", out, proj, q_off, k_off, v_off, 0, proj, (f_off, i_off), f_b, i_b,
                     cap, D ** -0.5, S_st, n_st, m_st, norm_w, g_off, "sigmoid", False, eps,
-                    seq_slot, positions, q_start, H, H, D, V)
+                    seq_slot, positions, q_start, H, H, D, V, first_seq)
         return
     T = proj.shape[0]
     q, k, v = _heads(proj, q_off, H, D), _heads(proj, k_off, H, D), _heads(proj, v_off, H, V)
@@ -1064,7 +1093,7 @@ def gated_delta(out: torch.Tensor, qkv: torch.Tensor, q_off: int, k_off: int, v_
     if _native(qkv):
         _recurrence("delta", out, qkv, q_off, k_off, v_off, 0, proj, (a_off, b_off), a_log,
                     dt_bias, 0.0, D ** -0.5, state, None, None, norm_w, g_off, "silu", False, eps,
-                    seq_slot, positions, q_start, H, G, D, V)
+                    seq_slot, positions, q_start, H, G, D, V, first_seq)
         return
     T = qkv.shape[0]
     q, k, v = _heads(qkv, q_off, G, D), _heads(qkv, k_off, G, D), _heads(qkv, v_off, H, V)
