@@ -23,6 +23,8 @@
 // slot 8 hl + e <-> index 8 (e >> 2) + 4 hl + (e & 3).  A operands are stored in that order (a
 // fragment = 64 lanes x 8 elements, 1 KB, one 16-byte load per lane), so the state, the solved
 // rows and the outputs of one product feed the next without leaving the registers.
+#include <type_traits>
+
 #include "../kernels/common.h"
 #include "stream.h"
 
@@ -38,7 +40,7 @@ namespace {
 constexpr int kC = 64;          // tokens of a chunk
 constexpr int kFrag = 512;      // elements of a fragment
 constexpr int kPT = 12;         // fragments of P (and of the inverse): 6 of hi, 6 of lo
-constexpr int kSc = 5 * kC;     // floats of scalars per (chunk, head)
+constexpr int kSc = 4 * kC;     // floats of scalars per (chunk, head)
 
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __expf(-z)); }
 __device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
@@ -47,12 +49,22 @@ __device__ __forceinline__ f32x16 mfma(bf16x8 a, bf16x8 b, f32x16 c) {
   return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
 }
 
+// two floats rounded to a pair of bf16
+__device__ __forceinline__ uint32_t pack2(float a, float b) {
+  const akap::f32x2 f = {a, b};
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f, akap::bf16x2));
+}
+
 __device__ __forceinline__ void split8(const float (&v)[8], bf16x8& hi, bf16x8& lo) {
+  uint32_t h[4], l[4];
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    hi[i] = (bf16)v[i];
-    lo[i] = (bf16)(v[i] - (float)hi[i]);
+  for (int i = 0; i < 4; ++i) {
+    h[i] = pack2(v[2 * i], v[2 * i + 1]);
+    l[i] = pack2(v[2 * i] - __uint_as_float(h[i] << 16),
+                 v[2 * i + 1] - __uint_as_float(h[i] & 0xffff0000u));
   }
+  hi = __builtin_bit_cast(bf16x8, h);
+  lo = __builtin_bit_cast(bf16x8, l);
 }
 
 // entries of a chunk buffer: sequence b (counted from the first chunked one) owns those from
@@ -166,7 +178,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
     sc[kC + lane] = expf(Lend - L) * c_s;
     sc[2 * kC + lane] = beta;
     sc[3 * kC + lane] = beta * eL * c_s;
-    sc[4 * kC + lane] = expf(Lend);
+    if (lane == 0) p.eend[ch] = expf(Lend);
   }
   __syncthreads();
   // P (and A): the transposed product, key tile x query tile, so that a lane holds a query's row
@@ -264,29 +276,80 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
 }
 
 // ------------------------------------------------------------------ walk over the chunks
-// a wave per (sequence, head, 32 state columns); no barriers, the four waves of a workgroup only
-// share their operand loads through the caches
-__device__ __forceinline__ bf16x8 frag(const bf16* base, int i, int lane) {
-  return *(const bf16x8*)(base + i * kFrag + lane * 8);
+// A workgroup of NW waves per (sequence, head, NW x 32 state columns); a wave owns 32 columns.
+// The operand fragments and scalars of a chunk go to LDS by LDS-DMA, one chunk ahead of the
+// products where two chunks fit; the values of the next chunk are fetched into registers.
+__device__ __forceinline__ void dma16(const void* g, void* lds_wave_base) {
+  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g,
+                                   (__attribute__((address_space(3))) void*)lds_wave_base, 16, 0, 0);
 }
 
 template <int MODE, int DT>
-__global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
-  constexpr int D = DT * 32, NKB = D / 16;
+struct Walk {
+  static constexpr int NKB = DT * 2;
+  static constexpr int Q = 0;                                    // fragment indices in a buffer
+  static constexpr int K = Q + 2 * NKB;
+  static constexpr int P = K + (MODE == kDelta ? 2 * NKB : 0);
+  static constexpr int T = P + kPT;
+  static constexpr int KT = T + (MODE == kDelta ? kPT : 0);
+  static constexpr int SC = KT + 4 * DT;
+  static constexpr int N = SC + 1;                               // 1 KB each
+  static constexpr int NB = N <= 80 ? 2 : 1;                     // buffers (160 KB of LDS)
+};
+
+template <int MODE, int DT, int NW>
+__global__ __launch_bounds__(NW * 64) void chunk_walk_kernel(ChunkParams p) {
+  using W = Walk<MODE, DT>;
+  constexpr int D = DT * 32, NKB = W::NKB;
+  __shared__ __align__(16) bf16 lds[W::NB * W::N * kFrag];
   const RecurrenceParams& r = p.r;
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, hl = lane >> 5, ln = lane & 31;
-  const int h = blockIdx.y, b = blockIdx.z;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int lane = threadIdx.x & 63, hl = lane >> 5, ln = lane & 31;
   const int cols = r.V + (MODE == kMatrixMemory ? 1 : 0);   // column V: the normaliser
-  const int c0 = (blockIdx.x * 4 + wave) * 32;
+  const int nct = (cols + NW * 32 - 1) / (NW * 32);
+  // the workgroups of a sequence's heads share an XCD
+  const int id = akap::xcd_remap(blockIdx.x, gridDim.x);
+  const int h = (id / nct) % r.H, b = id / (nct * r.H);
+  const int c0 = ((id % nct) * NW + wave) * 32;
   const int first = r.q_start[b], end = r.q_start[b + 1];
-  if (c0 >= cols || end <= first) return;
+  if (end <= first) return;
   const int slot = r.seq_slot[first];
   if (slot < 0 || slot >= r.num_slots) return;
   const int rep = r.H / r.G, hq = h / rep;
   const int c = c0 + ln;
   const bool isv = c < r.V, isn = MODE == kMatrixMemory && c == r.V;
+  const bool active = c0 < cols;          // wave-uniform: a wave past the columns only stages
   float* sp = isn ? r.n_state + ((size_t)slot * r.H + h) * D
                   : r.state + (((size_t)slot * r.H + h) * r.V + (isv ? c : 0)) * D;
+
+  auto stage = [&](int entry, int buf) {
+    const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
+    bf16* dst = lds + buf * W::N * kFrag;
+    auto seg = [&](const uint16_t* src, int at, auto n) {
+      static_assert(decltype(n)::value % NW == 0, "whole rounds of the waves");
+#pragma unroll
+      for (int f = 0; f < decltype(n)::value; f += NW)
+        dma16(src + (f + wave) * kFrag + lane * 8, dst + (at + f + wave) * kFrag);
+    };
+    if (MODE == kDelta) seg(p.kf + cg * 2 * NKB * kFrag, W::K, std::integral_constant<int, 2 * NKB>());
+    seg(p.qf + cg * 2 * NKB * kFrag, W::Q, std::integral_constant<int, 2 * NKB>());
+    if (MODE == kDelta) seg(p.tf + ch * kPT * kFrag, W::T, std::integral_constant<int, kPT>());
+    seg(p.pf + ch * kPT * kFrag, W::P, std::integral_constant<int, kPT>());
+    seg(p.ktf + cg * DT * 4 * kFrag, W::KT, std::integral_constant<int, DT * 4>());
+    if (wave == 0) dma16(p.sc + ch * kSc + lane * 4, dst + W::SC * kFrag);
+  };
+  // values of this lane's column, rows as in an accumulator, a register each: packing two would
+  // wait for the loads (columns past V load column 0 and are masked at their use)
+  const uint16_t* vsrc = (const uint16_t*)r.qkv + r.v_off + h * r.V + (isv ? c : 0);
+  auto values = [&](int r0, uint32_t (&v)[32]) {
+    const int n = min(kC, end - r0);
+#pragma unroll
+    for (int i = 0; i < 32; ++i) {
+      const int row = min((i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3), n - 1);
+      v[i] = vsrc[(size_t)(r0 + row) * r.qkv_stride];
+    }
+  };
+
   f32x16 S[DT];
   const bool carry = r.positions[first] != 0 && (isv || isn);
 #pragma unroll
@@ -298,24 +361,40 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
       S[dt][4 * i] = x.x; S[dt][4 * i + 1] = x.y; S[dt][4 * i + 2] = x.z; S[dt][4 * i + 3] = x.w;
     }
   int entry = chunk_base(r.q_start, b, p.row0);
+  int buf = 0;
+  const uint32_t vmask = isv ? 0xffffu : 0u, vone = isn ? 0x3f80u : 0u;   // bf16 1.0
+  uint32_t nv[32];
+  values(first, nv);
+  if (W::NB == 2) stage(entry, 0);
   for (int r0 = first; r0 < end; r0 += kC, ++entry) {
     const int n = min(kC, end - r0);
-    const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
-    const bf16* qf = (bf16*)p.qf + cg * 2 * NKB * kFrag;
-    const bf16* kf = (bf16*)p.kf + cg * 2 * NKB * kFrag;
-    const bf16* kt = (bf16*)p.ktf + cg * DT * 4 * kFrag;
-    const bf16* pf = (bf16*)p.pf + ch * kPT * kFrag;
-    const bf16* tf = (bf16*)p.tf + ch * kPT * kFrag;
-    const float* sc = p.sc + ch * kSc;
-    // values of this lane's column, rows as in an accumulator
+    if (W::NB == 1) {
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      __builtin_amdgcn_s_barrier();       // every wave has read the previous chunk
+      asm volatile("" ::: "memory");
+      stage(entry, 0);
+    }
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();         // this chunk has landed; the other buffer is free
+    asm volatile("" ::: "memory");
+    const float eend = p.eend[(size_t)entry * r.H + h];
     bf16 vv[32];
 #pragma unroll
-    for (int i = 0; i < 32; ++i) {
-      const int row = min((i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3), n - 1);
-      bf16 v = (bf16)(isn ? 1.f : 0.f);
-      if (isv) v = ((const bf16*)r.qkv)[(size_t)(r0 + row) * r.qkv_stride + r.v_off + h * r.V + c];
-      vv[i] = v;
+    for (int i = 0; i < 32; ++i)
+      vv[i] = __builtin_bit_cast(bf16, (uint16_t)((nv[i] & vmask) | vone));
+    if (r0 + kC < end) {
+      if (W::NB == 2) stage(entry + 1, buf ^ 1);
+      values(r0 + kC, nv);
     }
+    const bf16* cur = lds + buf * W::N * kFrag;
+    if (W::NB == 2) buf ^= 1;
+    if (!active) continue;
+    auto frag = [&](int i) { return *(const bf16x8*)(cur + i * kFrag + lane * 8); };
+    // four neighbouring scalars, read like a fragment (a read of another type would wait for the
+    // chunk in flight)
+    auto sc4 = [&](int i) {
+      return __builtin_bit_cast(float4, *(const bf16x8*)(cur + W::SC * kFrag + i * 2));
+    };
     // products with the state before the chunk
     f32x16 O[2], X[2];
 #pragma unroll
@@ -330,11 +409,11 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
         if (MODE == kDelta) {
-          const bf16x8 a = frag(kf, t * NKB + kb, lane);
+          const bf16x8 a = frag(W::K + t * NKB + kb);
           X[t] = mfma(a, sh, X[t]);
           X[t] = mfma(a, sl, X[t]);
         }
-        const bf16x8 a = frag(qf, t * NKB + kb, lane);
+        const bf16x8 a = frag(W::Q + t * NKB + kb);
         O[t] = mfma(a, sh, O[t]);
         O[t] = mfma(a, sl, O[t]);
       }
@@ -355,8 +434,8 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
           const int row = kb * 16 + 8 * i + 4 * hl;
-          const float4 be = *(const float4*)(sc + 2 * kC + row);
-          const float4 bk = *(const float4*)(sc + 3 * kC + row);
+          const float4 be = sc4(2 * kC + row);
+          const float4 bk = sc4(3 * kC + row);
           const float b4[4] = {be.x, be.y, be.z, be.w}, k4[4] = {bk.x, bk.y, bk.z, bk.w};
 #pragma unroll
           for (int j = 0; j < 4; ++j)
@@ -372,7 +451,7 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
 #pragma unroll
         for (int kb = 0; kb < 2 + 2 * t; ++kb) {
           const int idx = t == 0 ? kb : 2 + kb;
-          const bf16x8 ah = frag(tf, idx, lane), al = frag(tf, 6 + idx, lane);
+          const bf16x8 ah = frag(W::T + idx), al = frag(W::T + 6 + idx);
           X[t] = mfma(ah, xh[kb], X[t]);
           X[t] = mfma(ah, xl[kb], X[t]);
           X[t] = mfma(al, xh[kb], X[t]);
@@ -383,7 +462,7 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float4 w = *(const float4*)(sc + t * 32 + 8 * i + 4 * hl);
+        const float4 w = sc4(t * 32 + 8 * i + 4 * hl);
         O[t][4 * i] *= w.x; O[t][4 * i + 1] *= w.y; O[t][4 * i + 2] *= w.z; O[t][4 * i + 3] *= w.w;
       }
     bf16x8 wh[4], wl[4];        // what enters the state: hi + lo of e^(L_end - L) c x
@@ -406,38 +485,44 @@ __global__ __launch_bounds__(256) void chunk_walk_kernel(ChunkParams p) {
 #pragma unroll
       for (int t = kb >> 1; t < 2; ++t) {
         const int idx = t == 0 ? kb : 2 + kb;
-        const bf16x8 ah = frag(pf, idx, lane), al = frag(pf, 6 + idx, lane);
+        const bf16x8 ah = frag(W::P + idx), al = frag(W::P + 6 + idx);
         O[t] = mfma(ah, uh, O[t]);
         O[t] = mfma(al, uh, O[t]);
         if (MODE == kDelta) O[t] = mfma(ah, ul, O[t]);
       }
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        const float4 z = *(const float4*)(sc + kC + kb * 16 + 8 * i + 4 * hl);
+        const float4 z = sc4(kC + kb * 16 + 8 * i + 4 * hl);
         w[4 * i] *= z.x; w[4 * i + 1] *= z.y; w[4 * i + 2] *= z.z; w[4 * i + 3] *= z.w;
       }
       split8(w, wh[kb], wl[kb]);
     }
+    if (isv || isn) {
+      float* o = isn ? p.den + (size_t)r0 * r.H + h : r.raw + ((size_t)r0 * r.H + h) * r.V + c;
+      const size_t os = isn ? (size_t)r.H : (size_t)r.H * r.V;
+      o += 4 * hl * os;
+      if (n == kC) {
+#pragma unroll
+        for (int i = 0; i < 32; ++i)
+          o[((i >> 4) * 32 + 8 * ((i >> 2) & 3) + (i & 3)) * os] = O[i >> 4][i & 15];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 32; ++i) {
+          const int row = (i >> 4) * 32 + 8 * ((i >> 2) & 3) + (i & 3);
+          if (row + 4 * hl < n) o[row * os] = O[i >> 4][i & 15];
+        }
+      }
+    }
     // the state after the chunk
-    const float eend = sc[4 * kC];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
 #pragma unroll
       for (int i = 0; i < 16; ++i) S[dt][i] *= eend;
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) {
-        const bf16x8 a = frag(kt, dt * 4 + kb, lane);
+        const bf16x8 a = frag(W::KT + dt * 4 + kb);
         S[dt] = mfma(a, wh[kb], S[dt]);
         S[dt] = mfma(a, wl[kb], S[dt]);
-      }
-    }
-    if (isv || isn) {
-      float* o = isn ? p.den + (size_t)r0 * r.H + h : r.raw + ((size_t)r0 * r.H + h) * r.V + c;
-      const size_t os = isn ? (size_t)r.H : (size_t)r.H * r.V;
-#pragma unroll
-      for (int i = 0; i < 32; ++i) {
-        const int row = (i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3);
-        if (row < n) o[row * os] = O[i >> 4][i & 15];
       }
     }
   }
@@ -505,7 +590,7 @@ void chunk_workspace(int mode, int chunks, int H, int G, int D, int64_t* halves,
   const int64_t g = (int64_t)chunks * G, hh = (int64_t)chunks * H;
   *halves = g * (int64_t)(D / 16) * 2 * kFrag * (mode == kDelta ? 2 : 1) +
             g * (D / 32) * 4 * kFrag + hh * kPT * kFrag * (mode == kDelta ? 2 : 1);
-  *floats = hh * kSc;
+  *floats = hh * (kSc + 1);
 }
 
 void launch_chunk_recurrence(ChunkParams p, int mode, uint16_t* halves, float* floats,
@@ -522,13 +607,19 @@ void launch_chunk_recurrence(ChunkParams p, int mode, uint16_t* halves, float* f
   p.pf = w; w += hh * kPT * kFrag;
   p.tf = w;
   p.sc = floats;
+  p.eend = floats + hh * kSc;
   const int cols = r.V + (mode == kMatrixMemory ? 1 : 0);
-  const dim3 pg(p.num_chunks, r.H), wg((cols + 127) / 128, r.H, r.num_seqs);
+  const dim3 pg(p.num_chunks, r.H);
+  // workgroups of four waves share a staged chunk among 128 columns; of two when those would
+  // leave CUs idle
+  const int wg4 = (cols + 127) / 128 * r.H * r.num_seqs, wg2 = (cols + 63) / 64 * r.H * r.num_seqs;
+  const bool four = wg4 >= 256;
   if (mode == kMatrixMemory) memory_gates_kernel<<<dim3(r.num_seqs, r.H), 64, 0, s>>>(p);
 #define AKAP_CH(M, T)                                \
   do {                                               \
     chunk_prep_kernel<M, T><<<pg, 256, 0, s>>>(p);   \
-    chunk_walk_kernel<M, T><<<wg, 256, 0, s>>>(p);   \
+    if (four) chunk_walk_kernel<M, T, 4><<<wg4, 256, 0, s>>>(p);  \
+    else chunk_walk_kernel<M, T, 2><<<wg2, 128, 0, s>>>(p);       \
   } while (0)
 #define AKAP_CHD(M)                    \
   switch (r.D / 32) {                  \

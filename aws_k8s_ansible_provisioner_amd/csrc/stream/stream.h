@@ -345,6 +345,7 @@ struct ChunkParams {
   uint16_t* pf;
   uint16_t* tf;
   float* sc;
+  float* eend;            // e^(L_end) per (chunk, head)
 };
 bool chunk_supported(int D);
 void chunk_workspace(int mode, int chunks, int H, int G, int D, int64_t* halves, int64_t* floats);
