@@ -17,10 +17,10 @@
 // (S0, P, u, the inverse) is split into a bf16 pair hi + lo, so products keep about 16 bits of
 // it; sums are fp32.
 //
-// Operand layouts (v_mfma_f32_32x32x16_bf16): an accumulator lane holds column l & 31 and rows
-// 8 i + 4 (l >> 5) + j in registers 4 i + j.  Read as the B operand of the next product, registers
-// 8 kb .. 8 kb + 7 are 8 of the 16 contraction indices of block kb, in the order
-// slot 8 hl + e <-> index 8 (e >> 2) + 4 hl + (e & 3).  A operands are stored in that order (a
+// Operand layouts (v_mfma_f32_16x16x32_bf16, g = lane >> 4): an accumulator lane holds column
+// l & 15 and rows 4 g + j in registers j.  Two neighbouring tiles read as the B operand of the
+// next product are 8 of the 32 contraction indices of a block, in the order
+// slot 8 g + e <-> index 16 (e >> 2) + 4 g + (e & 3).  A operands are stored in that order (a
 // fragment = 64 lanes x 8 elements, 1 KB, one 16-byte load per lane), so the state, the solved
 // rows and the outputs of one product feed the next without leaving the registers.
 #include <type_traits>
@@ -33,7 +33,7 @@ namespace akap_stream {
 using akap::bf16;
 using akap::bf16x4;
 using akap::bf16x8;
-using akap::f32x16;
+using akap::f32x4;
 
 namespace {
 
@@ -45,8 +45,13 @@ constexpr int kSc = 4 * kC;     // floats of scalars per (chunk, head)
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __expf(-z)); }
 __device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
-__device__ __forceinline__ f32x16 mfma(bf16x8 a, bf16x8 b, f32x16 c) {
-  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
+__device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+// fragment of P and of the inverse: tile of 16 rows tt, block of 32 columns kb (kb <= tt / 2)
+__device__ __forceinline__ constexpr int tri(int tt, int kb) {
+  return tt < 2 ? tt : 2 + (tt - 2) * 2 + kb;
 }
 
 // two floats rounded to a pair of bf16
@@ -77,7 +82,7 @@ __device__ __forceinline__ int chunk_base(const int32_t* q_start, int b, int row
 // One workgroup of four waves per (chunk, head).
 template <int MODE, int DT>
 __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
-  constexpr int D = DT * 32, LS = D + 8, NKB = D / 16;
+  constexpr int D = DT * 32, LS = D + 8;
   constexpr int AS = 68;
   __shared__ __align__(16) bf16 qs[kC * LS];
   __shared__ __align__(16) bf16 ks[kC * LS];
@@ -97,7 +102,7 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
   const int slot = r.seq_slot[first];
   if (slot < 0 || slot >= r.num_slots) return;
   const int n = min(kC, end - r0);
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, hl = lane >> 5, ln = lane & 31;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = (lane >> 4) * 4, ln = lane & 15;
   const int rep = r.H / r.G, hq = h / rep;
   const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
 
@@ -181,62 +186,68 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
     if (lane == 0) p.eend[ch] = expf(Lend);
   }
   __syncthreads();
-  // P (and A): the transposed product, key tile x query tile, so that a lane holds a query's row
-  if (wave < 3) {
-    const int ts = wave == 2, tt = wave > 0;
-    f32x16 qk, kk;
-#pragma unroll
-    for (int i = 0; i < 16; ++i) qk[i] = kk[i] = 0.f;
-#pragma unroll
-    for (int kb = 0; kb < NKB; ++kb) {
-      const bf16x8 a = *(const bf16x8*)(ks + (ts * 32 + ln) * LS + kb * 16 + hl * 8);
-      const bf16x8 q = *(const bf16x8*)(qs + (tt * 32 + ln) * LS + kb * 16 + hl * 8);
-      qk = mfma(a, q, qk);
-      if (MODE == kDelta) {
-        const bf16x8 k = *(const bf16x8*)(ks + (tt * 32 + ln) * LS + kb * 16 + hl * 8);
-        kk = mfma(a, k, kk);
-      }
-    }
-    const int t = tt * 32 + ln;
+  // P (and A): the transposed product, key tiles x a query tile, so that a lane holds a query's
+  // row; a wave takes the 16 queries of its number
+  {
+    const int tt = wave, t = tt * 16 + ln;
     const float Lt = Ls[t], dt = ct[t], at = MODE == kDelta ? bt[t] * cs[t] : 0.f;
     bf16* pf = (bf16*)p.pf + ch * kPT * kFrag;
-#pragma unroll
-    for (int kbl = 0; kbl < 2; ++kbl) {
+    for (int kb = 0; kb <= tt >> 1; ++kb) {
       float v[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int s = ts * 32 + kbl * 16 + 8 * (e >> 2) + 4 * hl + (e & 3);
-        const float w = expf(fminf(Lt - Ls[s], 0.f)) * cs[s];
-        v[e] = s <= t ? qk[kbl * 8 + e] * w * dt : 0.f;
-        if (MODE == kDelta) am[t * AS + s] = s < t ? kk[kbl * 8 + e] * w * at : 0.f;
+      for (int half = 0; half < 2; ++half) {
+        const int st = 2 * kb + half;
+        f32x4 qk = {0.f, 0.f, 0.f, 0.f}, kk = {0.f, 0.f, 0.f, 0.f};
+        if (st <= tt) {
+#pragma unroll
+          for (int k = 0; k < DT; ++k) {
+            const bf16x8 a = *(const bf16x8*)(ks + (st * 16 + ln) * LS + k * 32 + g4 * 2);
+            const bf16x8 q = *(const bf16x8*)(qs + t * LS + k * 32 + g4 * 2);
+            qk = mfma(a, q, qk);
+            if (MODE == kDelta) {
+              const bf16x8 k8 = *(const bf16x8*)(ks + t * LS + k * 32 + g4 * 2);
+              kk = mfma(a, k8, kk);
+            }
+          }
+        }
+        float av[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int s = st * 16 + g4 + e;
+          const float w = __expf(fminf(Lt - Ls[s], 0.f)) * cs[s];
+          v[half * 4 + e] = s <= t ? qk[e] * w * dt : 0.f;
+          av[e] = s < t ? kk[e] * w * at : 0.f;
+        }
+        if (MODE == kDelta)
+          *(float4*)(am + t * AS + st * 16 + g4) = make_float4(av[0], av[1], av[2], av[3]);
       }
       bf16x8 vh, vl;
       split8(v, vh, vl);
-      const int idx = tt == 0 ? kbl : 2 + ts * 2 + kbl;
+      const int idx = tri(tt, kb);
       *(bf16x8*)(pf + idx * kFrag + lane * 8) = vh;
       *(bf16x8*)(pf + (6 + idx) * kFrag + lane * 8) = vl;
     }
   }
   // fragments of q, k (rows = tokens) and of k transposed (rows = dimensions), once per key head
   if (h % rep == 0) {
-    bf16* qf = (bf16*)p.qf + cg * 2 * NKB * kFrag;
-    bf16* kf = (bf16*)p.kf + cg * 2 * NKB * kFrag;
-    bf16* kt = (bf16*)p.ktf + cg * DT * 4 * kFrag;
-    constexpr int kQ = 2 * NKB, kAll = kQ + (MODE == kDelta ? kQ : 0);
+    bf16* qf = (bf16*)p.qf + cg * 4 * DT * kFrag;
+    bf16* kf = (bf16*)p.kf + cg * 4 * DT * kFrag;
+    bf16* kt = (bf16*)p.ktf + cg * 4 * DT * kFrag;
+    constexpr int kQ = 4 * DT, kAll = kQ + (MODE == kDelta ? kQ : 0);
     for (int f = wave; f < kAll; f += 4) {
-      const int g = f < kQ ? f : f - kQ;
-      const bf16* src = (f < kQ ? qs : ks) + ((g / NKB) * 32 + ln) * LS + (g % NKB) * 16 + 4 * hl;
-      const bf16x4 x = *(const bf16x4*)src, y = *(const bf16x4*)(src + 8);
+      const int fr = f < kQ ? f : f - kQ;
+      const bf16* src = (f < kQ ? qs : ks) + ((fr / DT) * 16 + ln) * LS + (fr % DT) * 32 + g4;
+      const bf16x4 x = *(const bf16x4*)src, y = *(const bf16x4*)(src + 16);
       bf16x8 o;
 #pragma unroll
       for (int i = 0; i < 4; ++i) { o[i] = x[i]; o[4 + i] = y[i]; }
-      *(bf16x8*)((f < kQ ? qf : kf) + g * kFrag + lane * 8) = o;
+      *(bf16x8*)((f < kQ ? qf : kf) + fr * kFrag + lane * 8) = o;
     }
-    for (int f = wave; f < DT * 4; f += 4) {
-      const int d = (f >> 2) * 32 + ln, kb = f & 3;
+    for (int f = wave; f < kQ; f += 4) {
+      const int d = (f >> 1) * 16 + ln, kb = f & 1;
       bf16x8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = ks[(kb * 16 + 8 * (e >> 2) + 4 * hl + (e & 3)) * LS + d];
+      for (int e = 0; e < 8; ++e) o[e] = ks[(kb * 32 + 16 * (e >> 2) + g4 + (e & 3)) * LS + d];
       *(bf16x8*)(kt + f * kFrag + lane * 8) = o;
     }
   }
@@ -264,9 +275,9 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
   __syncthreads();
   bf16* tf = (bf16*)p.tf + ch * kPT * kFrag;
   for (int f = wave; f < 6; f += 4) {
-    const int row = (f < 2 ? 0 : 32) + ln, kb = f < 2 ? f : f - 2;
-    const float* src = am + row * AS + kb * 16 + 4 * hl;
-    const float4 x = *(const float4*)src, y = *(const float4*)(src + 8);
+    const int tt = f < 2 ? f : 2 + ((f - 2) >> 1), kb = f < 2 ? 0 : (f - 2) & 1;
+    const float* src = am + (tt * 16 + ln) * AS + kb * 32 + g4;
+    const float4 x = *(const float4*)src, y = *(const float4*)(src + 16);
     const float v[8] = {x.x, x.y, x.z, x.w, y.x, y.y, y.z, y.w};
     bf16x8 vh, vl;
     split8(v, vh, vl);
@@ -276,9 +287,11 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
 }
 
 // ------------------------------------------------------------------ walk over the chunks
-// A workgroup of NW waves per (sequence, head, NW x 32 state columns); a wave owns 32 columns.
-// The operand fragments and scalars of a chunk go to LDS by LDS-DMA, one chunk ahead of the
-// products where two chunks fit; the values of the next chunk are fetched into registers.
+// A workgroup per (sequence, head, NW x 16 state columns); a wave owns 16 columns.  The
+// normaliser of the matrix memory is one more wave (of the head's first workgroup) whose single
+// column has ones for values.  The operand fragments and scalars of a chunk go to LDS by
+// LDS-DMA, one chunk ahead of the products where two chunks fit; the values of the next chunk are
+// fetched into registers.
 __device__ __forceinline__ void dma16(const void* g, void* lds_wave_base) {
   __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g,
                                    (__attribute__((address_space(3))) void*)lds_wave_base, 16, 0, 0);
@@ -286,84 +299,96 @@ __device__ __forceinline__ void dma16(const void* g, void* lds_wave_base) {
 
 template <int MODE, int DT>
 struct Walk {
-  static constexpr int NKB = DT * 2;
+  static constexpr int F = 4 * DT;                               // fragments of q, k, k transposed
   static constexpr int Q = 0;                                    // fragment indices in a buffer
-  static constexpr int K = Q + 2 * NKB;
-  static constexpr int P = K + (MODE == kDelta ? 2 * NKB : 0);
+  static constexpr int K = Q + F;
+  static constexpr int P = K + (MODE == kDelta ? F : 0);
   static constexpr int T = P + kPT;
   static constexpr int KT = T + (MODE == kDelta ? kPT : 0);
-  static constexpr int SC = KT + 4 * DT;
+  static constexpr int SC = KT + F;
   static constexpr int N = SC + 1;                               // 1 KB each
   static constexpr int NB = N <= 80 ? 2 : 1;                     // buffers (160 KB of LDS)
 };
 
 template <int MODE, int DT, int NW>
-__global__ __launch_bounds__(NW * 64) void chunk_walk_kernel(ChunkParams p) {
+__global__ __launch_bounds__(NW * 64 + (MODE == kMatrixMemory ? 64 : 0)) void chunk_walk_kernel(
+    ChunkParams p) {
   using W = Walk<MODE, DT>;
-  constexpr int D = DT * 32, NKB = W::NKB;
+  constexpr int D = DT * 32;
   __shared__ __align__(16) bf16 lds[W::NB * W::N * kFrag];
   const RecurrenceParams& r = p.r;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int lane = threadIdx.x & 63, hl = lane >> 5, ln = lane & 31;
-  const int cols = r.V + (MODE == kMatrixMemory ? 1 : 0);   // column V: the normaliser
-  const int nct = (cols + NW * 32 - 1) / (NW * 32);
+  const int lane = threadIdx.x & 63, g4 = (lane >> 4) * 4, ln = lane & 15;
+  const int nct = (r.V + NW * 16 - 1) / (NW * 16);
   // the workgroups of a sequence's heads share an XCD
   const int id = akap::xcd_remap(blockIdx.x, gridDim.x);
-  const int h = (id / nct) % r.H, b = id / (nct * r.H);
-  const int c0 = ((id % nct) * NW + wave) * 32;
+  const int h = (id / nct) % r.H, b = id / (nct * r.H), ct = id % nct;
   const int first = r.q_start[b], end = r.q_start[b + 1];
   if (end <= first) return;
   const int slot = r.seq_slot[first];
   if (slot < 0 || slot >= r.num_slots) return;
   const int rep = r.H / r.G, hq = h / rep;
-  const int c = c0 + ln;
-  const bool isv = c < r.V, isn = MODE == kMatrixMemory && c == r.V;
-  const bool active = c0 < cols;          // wave-uniform: a wave past the columns only stages
-  float* sp = isn ? r.n_state + ((size_t)slot * r.H + h) * D
-                  : r.state + (((size_t)slot * r.H + h) * r.V + (isv ? c : 0)) * D;
+  const bool nwave = MODE == kMatrixMemory && wave == NW;        // the normaliser's wave
+  const int c0 = (ct * NW + wave) * 16, c = c0 + ln;
+  const bool isv = !nwave && c < r.V, isn = nwave && ct == 0 && ln == 0;
+  // wave-uniform: a wave past the columns only stages
+  const bool active = nwave ? ct == 0 : c0 < r.V;
+  float* sp = nwave ? r.n_state + ((size_t)slot * r.H + h) * D
+                    : r.state + (((size_t)slot * r.H + h) * r.V + (isv ? c : 0)) * D;
 
   auto stage = [&](int entry, int buf) {
+    if (MODE == kMatrixMemory && wave >= NW) return;
     const size_t ch = (size_t)entry * r.H + h, cg = (size_t)entry * r.G + hq;
     bf16* dst = lds + buf * W::N * kFrag;
     auto seg = [&](const uint16_t* src, int at, auto n) {
-      static_assert(decltype(n)::value % NW == 0, "whole rounds of the waves");
+      static_assert(decltype(n)::value % 4 == 0, "whole rounds of four waves");
 #pragma unroll
       for (int f = 0; f < decltype(n)::value; f += NW)
-        dma16(src + (f + wave) * kFrag + lane * 8, dst + (at + f + wave) * kFrag);
+        if (decltype(n)::value % NW == 0 || f + wave < decltype(n)::value)
+          dma16(src + (f + wave) * kFrag + lane * 8, dst + (at + f + wave) * kFrag);
     };
-    if (MODE == kDelta) seg(p.kf + cg * 2 * NKB * kFrag, W::K, std::integral_constant<int, 2 * NKB>());
-    seg(p.qf + cg * 2 * NKB * kFrag, W::Q, std::integral_constant<int, 2 * NKB>());
-    if (MODE == kDelta) seg(p.tf + ch * kPT * kFrag, W::T, std::integral_constant<int, kPT>());
-    seg(p.pf + ch * kPT * kFrag, W::P, std::integral_constant<int, kPT>());
-    seg(p.ktf + cg * DT * 4 * kFrag, W::KT, std::integral_constant<int, DT * 4>());
+    using NF = std::integral_constant<int, W::F>;
+    using NP = std::integral_constant<int, kPT>;
+    if (MODE == kDelta) seg(p.kf + cg * W::F * kFrag, W::K, NF());
+    seg(p.qf + cg * W::F * kFrag, W::Q, NF());
+    if (MODE == kDelta) seg(p.tf + ch * kPT * kFrag, W::T, NP());
+    seg(p.pf + ch * kPT * kFrag, W::P, NP());
+    seg(p.ktf + cg * W::F * kFrag, W::KT, NF());
     if (wave == 0) dma16(p.sc + ch * kSc + lane * 4, dst + W::SC * kFrag);
   };
   // values of this lane's column, rows as in an accumulator, a register each: packing two would
   // wait for the loads (columns past V load column 0 and are masked at their use)
-  const uint16_t* vsrc = (const uint16_t*)r.qkv + r.v_off + h * r.V + (isv ? c : 0);
-  auto values = [&](int r0, uint32_t (&v)[32]) {
+  const uint32_t vbytes = (uint32_t)(isv ? c : 0) * 2u;
+  auto values = [&](int r0, uint32_t (&v)[16]) {
     const int n = min(kC, end - r0);
+    const char* row0 = (const char*)((const uint16_t*)r.qkv + (size_t)r0 * r.qkv_stride + r.v_off +
+                                     h * r.V);
+    const uint32_t rb = (uint32_t)r.qkv_stride * 2u;
+    if (n == kC) {
+      const uint32_t lo = vbytes + (uint32_t)g4 * rb;
 #pragma unroll
-    for (int i = 0; i < 32; ++i) {
-      const int row = min((i >> 4) * 32 + 8 * ((i >> 2) & 3) + 4 * hl + (i & 3), n - 1);
-      v[i] = vsrc[(size_t)(r0 + row) * r.qkv_stride];
+      for (int i = 0; i < 16; ++i)
+        v[i] = *(const uint16_t*)(row0 + (size_t)((i >> 2) * 16 + (i & 3)) * rb + lo);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 16; ++i)
+        v[i] = *(const uint16_t*)(row0 + (uint32_t)min((i >> 2) * 16 + g4 + (i & 3), n - 1) * rb +
+                                  vbytes);
     }
   };
 
-  f32x16 S[DT];
+  f32x4 S[2 * DT];
   const bool carry = r.positions[first] != 0 && (isv || isn);
 #pragma unroll
-  for (int dt = 0; dt < DT; ++dt)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (carry) x = *(const float4*)(sp + dt * 32 + 8 * i + 4 * hl);
-      S[dt][4 * i] = x.x; S[dt][4 * i + 1] = x.y; S[dt][4 * i + 2] = x.z; S[dt][4 * i + 3] = x.w;
-    }
+  for (int d = 0; d < 2 * DT; ++d) {
+    float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (carry) x = *(const float4*)(sp + d * 16 + g4);
+    S[d] = f32x4{x.x, x.y, x.z, x.w};
+  }
   int entry = chunk_base(r.q_start, b, p.row0);
   int buf = 0;
   const uint32_t vmask = isv ? 0xffffu : 0u, vone = isn ? 0x3f80u : 0u;   // bf16 1.0
-  uint32_t nv[32];
+  uint32_t nv[16];
   values(first, nv);
   if (W::NB == 2) stage(entry, 0);
   for (int r0 = first; r0 < end; r0 += kC, ++entry) {
@@ -374,14 +399,16 @@ __global__ __launch_bounds__(NW * 64) void chunk_walk_kernel(ChunkParams p) {
       asm volatile("" ::: "memory");
       stage(entry, 0);
     }
-    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+    // a builtin wait (vmcnt 0, lgkmcnt 0): the compiler then knows that the values fetched during
+    // the previous chunk have arrived, and adds no wait of its own after the next ones are issued
+    __builtin_amdgcn_s_waitcnt(0x0070);
+    asm volatile("" ::: "memory");
     __builtin_amdgcn_s_barrier();         // this chunk has landed; the other buffer is free
     asm volatile("" ::: "memory");
     const float eend = p.eend[(size_t)entry * r.H + h];
-    bf16 vv[32];
+    float vv[16];
 #pragma unroll
-    for (int i = 0; i < 32; ++i)
-      vv[i] = __builtin_bit_cast(bf16, (uint16_t)((nv[i] & vmask) | vone));
+    for (int i = 0; i < 16; ++i) vv[i] = __uint_as_float(((nv[i] & vmask) | vone) << 16);
     if (r0 + kC < end) {
       if (W::NB == 2) stage(entry + 1, buf ^ 1);
       values(r0 + kC, nv);
@@ -389,150 +416,128 @@ __global__ __launch_bounds__(NW * 64) void chunk_walk_kernel(ChunkParams p) {
     const bf16* cur = lds + buf * W::N * kFrag;
     if (W::NB == 2) buf ^= 1;
     if (!active) continue;
-    auto frag = [&](int i) { return *(const bf16x8*)(cur + i * kFrag + lane * 8); };
-    // four neighbouring scalars, read like a fragment (a read of another type would wait for the
-    // chunk in flight)
-    auto sc4 = [&](int i) {
-      return __builtin_bit_cast(float4, *(const bf16x8*)(cur + W::SC * kFrag + i * 2));
+    const bf16* fl = cur + lane * 8;
+    auto frag = [&](int i) { return *(const bf16x8*)(fl + i * kFrag); };
+    // scalars of the four rows 16 t + 4 g .. +3 of array a
+    const bf16* sl = cur + W::SC * kFrag + g4 * 2;
+    auto sc4 = [&](int a, int t) {
+      return __builtin_bit_cast(f32x4, *(const bf16x8*)(sl + (a * kC + t * 16) * 2));
     };
-    // products with the state before the chunk
-    f32x16 O[2], X[2];
-#pragma unroll
-    for (int i = 0; i < 16; ++i) O[0][i] = O[1][i] = X[0][i] = X[1][i] = 0.f;
-#pragma unroll
-    for (int kb = 0; kb < NKB; ++kb) {
-      float s[8];
-#pragma unroll
-      for (int e = 0; e < 8; ++e) s[e] = S[kb >> 1][(kb & 1) * 8 + e];
-      bf16x8 sh, sl;
-      split8(s, sh, sl);
-#pragma unroll
-      for (int t = 0; t < 2; ++t) {
-        if (MODE == kDelta) {
-          const bf16x8 a = frag(W::K + t * NKB + kb);
-          X[t] = mfma(a, sh, X[t]);
-          X[t] = mfma(a, sl, X[t]);
-        }
-        const bf16x8 a = frag(W::Q + t * NKB + kb);
-        O[t] = mfma(a, sh, O[t]);
-        O[t] = mfma(a, sl, O[t]);
-      }
-    }
     if (MODE == kDecay && r.act) {
 #pragma unroll
-      for (int i = 0; i < 32; ++i) {
-        const float z = (float)vv[i];
-        vv[i] = (bf16)(z * sigmoidf(z));
+      for (int i = 0; i < 16; ++i) vv[i] *= sigmoidf(vv[i]);
+    }
+    // products with the state before the chunk
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    f32x4 O[4] = {zero, zero, zero, zero}, X[4] = {zero, zero, zero, zero};
+#pragma unroll
+    for (int k = 0; k < DT; ++k) {
+      float s[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s[e] = S[2 * k + (e >> 2)][e & 3];
+      bf16x8 sh, sl2;
+      split8(s, sh, sl2);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        if (MODE == kDelta) {
+          const bf16x8 a = frag(W::K + t * DT + k);
+          X[t] = mfma(a, sh, X[t]);
+          X[t] = mfma(a, sl2, X[t]);
+        }
+        const bf16x8 a = frag(W::Q + t * DT + k);
+        O[t] = mfma(a, sh, O[t]);
+        O[t] = mfma(a, sl2, O[t]);
       }
     }
     if (MODE == kDelta) {
       // u = (I + A)^-1 (beta v - beta e^L c (K S0))
-      bf16x8 xh[4], xl[4];
+      bf16x8 xh[2], xl[2];
 #pragma unroll
-      for (int kb = 0; kb < 4; ++kb) {
+      for (int kb = 0; kb < 2; ++kb) {
         float x[8];
 #pragma unroll
         for (int i = 0; i < 2; ++i) {
-          const int row = kb * 16 + 8 * i + 4 * hl;
-          const float4 be = sc4(2 * kC + row);
-          const float4 bk = sc4(3 * kC + row);
-          const float b4[4] = {be.x, be.y, be.z, be.w}, k4[4] = {bk.x, bk.y, bk.z, bk.w};
+          const f32x4 be = sc4(2, 2 * kb + i), bk = sc4(3, 2 * kb + i);
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            x[4 * i + j] = b4[j] * (float)vv[kb * 8 + 4 * i + j] -
-                           k4[j] * X[kb >> 1][(kb & 1) * 8 + 4 * i + j];
+            x[4 * i + j] = be[j] * vv[kb * 8 + 4 * i + j] - bk[j] * X[2 * kb + i][j];
         }
         split8(x, xh[kb], xl[kb]);
       }
 #pragma unroll
-      for (int i = 0; i < 16; ++i) X[0][i] = X[1][i] = 0.f;
+      for (int t = 0; t < 4; ++t) {
+        X[t] = zero;
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
-#pragma unroll
-        for (int kb = 0; kb < 2 + 2 * t; ++kb) {
-          const int idx = t == 0 ? kb : 2 + kb;
-          const bf16x8 ah = frag(W::T + idx), al = frag(W::T + 6 + idx);
+        for (int kb = 0; kb <= t >> 1; ++kb) {
+          const bf16x8 ah = frag(W::T + tri(t, kb)), al = frag(W::T + 6 + tri(t, kb));
           X[t] = mfma(ah, xh[kb], X[t]);
           X[t] = mfma(ah, xl[kb], X[t]);
           X[t] = mfma(al, xh[kb], X[t]);
         }
+      }
     }
     // outputs: the part through S0 scaled by row, the part inside the chunk
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
+    for (int t = 0; t < 4; ++t) O[t] *= sc4(0, t);
+    bf16x8 wh[2], wl[2];        // what enters the state: hi + lo of e^(L_end - L) c x
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float4 w = sc4(t * 32 + 8 * i + 4 * hl);
-        O[t][4 * i] *= w.x; O[t][4 * i + 1] *= w.y; O[t][4 * i + 2] *= w.z; O[t][4 * i + 3] *= w.w;
-      }
-    bf16x8 wh[4], wl[4];        // what enters the state: hi + lo of e^(L_end - L) c x
-#pragma unroll
-    for (int kb = 0; kb < 4; ++kb) {
+    for (int kb = 0; kb < 2; ++kb) {
       bf16x8 uh, ul;
-      float w[8];
-      if (MODE == kDelta) {
-        float u[8];
+      float u[8], w[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) w[e] = u[e] = X[kb >> 1][(kb & 1) * 8 + e];
-        split8(u, uh, ul);
-      } else {
+      for (int e = 0; e < 8; ++e)
+        u[e] = MODE == kDelta ? X[2 * kb + (e >> 2)][e & 3] : vv[kb * 8 + e];
+      // (plain recurrences: v is a bf16 number or, activated, rounded to one by its lo part)
+      split8(u, uh, ul);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          uh[e] = vv[kb * 8 + e];
-          w[e] = (float)vv[kb * 8 + e];
-        }
-      }
-#pragma unroll
-      for (int t = kb >> 1; t < 2; ++t) {
-        const int idx = t == 0 ? kb : 2 + kb;
-        const bf16x8 ah = frag(W::P + idx), al = frag(W::P + 6 + idx);
+      for (int t = 2 * kb; t < 4; ++t) {
+        const bf16x8 ah = frag(W::P + tri(t, kb)), al = frag(W::P + 6 + tri(t, kb));
         O[t] = mfma(ah, uh, O[t]);
         O[t] = mfma(al, uh, O[t]);
-        if (MODE == kDelta) O[t] = mfma(ah, ul, O[t]);
+        if (MODE != kMatrixMemory) O[t] = mfma(ah, ul, O[t]);
       }
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        const float4 z = sc4(kC + kb * 16 + 8 * i + 4 * hl);
-        w[4 * i] *= z.x; w[4 * i + 1] *= z.y; w[4 * i + 2] *= z.z; w[4 * i + 3] *= z.w;
+        const f32x4 z = sc4(1, 2 * kb + i);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) w[4 * i + j] = u[4 * i + j] * z[j];
       }
       split8(w, wh[kb], wl[kb]);
     }
-    if (isv || isn) {
-      float* o = isn ? p.den + (size_t)r0 * r.H + h : r.raw + ((size_t)r0 * r.H + h) * r.V + c;
-      const size_t os = isn ? (size_t)r.H : (size_t)r.H * r.V;
-      o += 4 * hl * os;
-      if (n == kC) {
+    {
+      const size_t os = (nwave ? (size_t)r.H : (size_t)r.H * r.V) * sizeof(float);   // row pitch
+      char* o = nwave ? (char*)(p.den + (size_t)r0 * r.H + h)
+                      : (char*)(r.raw + ((size_t)r0 * r.H + h) * r.V);
+      const uint32_t lo = (uint32_t)(nwave ? 0 : c) * 4u + (uint32_t)g4 * (uint32_t)os;
+      if (isv || isn) {
+        if (n == kC) {
 #pragma unroll
-        for (int i = 0; i < 32; ++i)
-          o[((i >> 4) * 32 + 8 * ((i >> 2) & 3) + (i & 3)) * os] = O[i >> 4][i & 15];
-      } else {
+          for (int i = 0; i < 16; ++i)
+            *(float*)(o + ((i >> 2) * 16 + (i & 3)) * os + lo) = O[i >> 2][i & 3];
+        } else {
 #pragma unroll
-        for (int i = 0; i < 32; ++i) {
-          const int row = (i >> 4) * 32 + 8 * ((i >> 2) & 3) + (i & 3);
-          if (row + 4 * hl < n) o[row * os] = O[i >> 4][i & 15];
+          for (int i = 0; i < 16; ++i)
+            if ((i >> 2) * 16 + g4 + (i & 3) < n)
+              *(float*)(o + ((i >> 2) * 16 + (i & 3)) * os + lo) = O[i >> 2][i & 3];
         }
       }
     }
     // the state after the chunk
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
+    for (int d = 0; d < 2 * DT; ++d) {
+      S[d] *= eend;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) S[dt][i] *= eend;
-#pragma unroll
-      for (int kb = 0; kb < 4; ++kb) {
-        const bf16x8 a = frag(W::KT + dt * 4 + kb);
-        S[dt] = mfma(a, wh[kb], S[dt]);
-        S[dt] = mfma(a, wl[kb], S[dt]);
+      for (int kb = 0; kb < 2; ++kb) {
+        const bf16x8 a = frag(W::KT + d * 2 + kb);
+        S[d] = mfma(a, wh[kb], S[d]);
+        S[d] = mfma(a, wl[kb], S[d]);
       }
     }
   }
   if (isv || isn) {
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        *(float4*)(sp + dt * 32 + 8 * i + 4 * hl) =
-            make_float4(S[dt][4 * i], S[dt][4 * i + 1], S[dt][4 * i + 2], S[dt][4 * i + 3]);
+    for (int d = 0; d < 2 * DT; ++d)
+      *(float4*)(sp + d * 16 + g4) = make_float4(S[d][0], S[d][1], S[d][2], S[d][3]);
   }
 }
 
@@ -608,18 +613,18 @@ void launch_chunk_recurrence(ChunkParams p, int mode, uint16_t* halves, float* f
   p.tf = w;
   p.sc = floats;
   p.eend = floats + hh * kSc;
-  const int cols = r.V + (mode == kMatrixMemory ? 1 : 0);
   const dim3 pg(p.num_chunks, r.H);
-  // workgroups of four waves share a staged chunk among 128 columns; of two when those would
+  // workgroups of eight waves share a staged chunk among 128 columns; of four when those would
   // leave CUs idle
-  const int wg4 = (cols + 127) / 128 * r.H * r.num_seqs, wg2 = (cols + 63) / 64 * r.H * r.num_seqs;
-  const bool four = wg4 >= 256;
+  const int wg8 = (r.V + 127) / 128 * r.H * r.num_seqs, wg4 = (r.V + 63) / 64 * r.H * r.num_seqs;
+  const bool eight = wg8 >= 256;
+  const int extra = mode == kMatrixMemory ? 64 : 0;
   if (mode == kMatrixMemory) memory_gates_kernel<<<dim3(r.num_seqs, r.H), 64, 0, s>>>(p);
 #define AKAP_CH(M, T)                                \
   do {                                               \
     chunk_prep_kernel<M, T><<<pg, 256, 0, s>>>(p);   \
-    if (four) chunk_walk_kernel<M, T, 4><<<wg4, 256, 0, s>>>(p);  \
-    else chunk_walk_kernel<M, T, 2><<<wg2, 128, 0, s>>>(p);       \
+    if (eight) chunk_walk_kernel<M, T, 8><<<wg8, 512 + extra, 0, s>>>(p);   \
+    else chunk_walk_kernel<M, T, 4><<<wg4, 256 + extra, 0, s>>>(p);         \
   } while (0)
 #define AKAP_CHD(M)                    \
   switch (r.D / 32) {                  \
