@@ -44,6 +44,17 @@ __device__ __forceinline__ void st4(bf16* p, const float (&v)[4]) {
   *(akap::bf16x4*)p = o;
 }
 
+__device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
+  *(float4*)p = make_float4(v[0], v[1], v[2], v[3]);
+  *(float4*)(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
+}
+__device__ __forceinline__ void st8(bf16* p, const float (&v)[8]) {
+  akap::bf16x8 o;
+#pragma unroll
+  for (int k = 0; k < 8; ++k) o[k] = (bf16)v[k];
+  *(akap::bf16x8*)p = o;
+}
+
 __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __expf(-z)); }
 __device__ __forceinline__ float siluf(float z) { return z * sigmoidf(z); }
 
@@ -442,6 +453,130 @@ __global__ __launch_bounds__(256) void conv_silu_vec_kernel(const ConvArgs a, co
         for (int k = 0; k < 4; ++k) hist[j][k] = cur[k];
       }
   }
+}
+
+// eight channels per thread (16-byte accesses of bf16), TAPS at compile time: a tile of RB rows
+// inside one sequence is fetched four rows at a time ahead of its products; tiles with a
+// sequence's start or end go row by row with the history from the tile or the slot
+constexpr int kConvRows8 = 32;
+
+template <typename TO, int TAPS>
+__global__ __launch_bounds__(128) void conv_silu_vec8_kernel(const ConvArgs a) {
+  const int c = (blockIdx.y * 128 + threadIdx.x) * 8;
+  if (c >= a.C) return;
+  const int tb = blockIdx.x * kConvRows8, te = min(a.T, tb + kConvRows8);
+  const bf16* in = (const bf16*)a.proj + a.off + c;
+  TO* out = (TO*)a.out + c;
+  float w[TAPS][8], hist[TAPS][8], bias[8];          // hist[j]: the input TAPS - 1 - j rows back
+#pragma unroll
+  for (int k = 0; k < 8; ++k) {
+    bias[k] = a.b ? a.b[c + k] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j][k] = a.w[(size_t)(c + k) * TAPS + j];
+  }
+  auto load = [&](int t, float (&v)[8]) {
+    const akap::bf16x8 x = *(const akap::bf16x8*)(in + (size_t)t * a.proj_stride);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[k] = (float)x[k];
+  };
+  auto emit = [&](int t, const float (&cur)[8]) {
+    float o[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      float z = bias[k];
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) z += w[j][k] * hist[j][k];
+      z += w[TAPS - 1][k] * cur[k];
+      o[k] = c + k >= a.silu_from ? siluf(z) : z;
+    }
+    TO* op = out + (size_t)t * a.C;
+    st8(op, o);
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j)
+#pragma unroll
+      for (int k = 0; k < 8; ++k) hist[j][k] = j == TAPS - 2 ? cur[k] : hist[j + 1][k];
+  };
+  int b = seq_of_row(a.q_start, a.B, tb);
+  for (int t = tb; t < te;) {
+    while (b + 1 < a.B && a.q_start[b + 1] <= t) ++b;   // empty sequences
+    const int r0 = a.q_start[b], r1 = min(a.q_start[b + 1], te);
+    if (t >= r1) break;                              // rows past the last sequence
+    const int slot = a.seq_slot[r0];
+    if (slot < 0) {
+      t = r1;
+      continue;
+    }
+    const int pos0 = (int)a.positions[r0];
+    const bf16* st = (const bf16*)a.state + (size_t)slot * (TAPS - 1) * a.C + c;
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) {
+      const int src = t - (TAPS - 1 - j), kk = src - r0;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) hist[j][k] = 0.f;
+      if (kk >= 0) {
+        load(src, hist[j]);
+      } else if (pos0 + kk >= 0) {                   // -1: the input just before the step
+        const akap::bf16x8 x = *(const akap::bf16x8*)(st + (size_t)(TAPS - 1 + kk) * a.C);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) hist[j][k] = (float)x[k];
+      }
+    }
+    for (; t + 4 <= r1; t += 4) {
+      float cur[4][8];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) load(t + i, cur[i]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) emit(t + i, cur[i]);
+    }
+    for (; t < r1; ++t) {
+      float cur[8];
+      load(t, cur);
+      emit(t, cur);
+    }
+  }
+}
+
+// steps of single rows: a thread per (row, four channels) convolves and shifts its slot's inputs
+template <typename TY, typename TO>
+__global__ __launch_bounds__(256) void conv_step_kernel(const ConvArgs a) {
+  const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (c >= a.C) return;
+  const int slot = a.seq_slot[t];
+  if (slot < 0) return;
+  constexpr bool F32 = sizeof(TY) == 4;
+  const int64_t pos = a.positions[t];
+  const int keep = a.taps - 1;
+  TY* st = (TY*)a.state + (size_t)slot * keep * a.C + c;
+  float cur[4], h[kMaxTaps - 1][4], acc[4] = {0.f, 0.f, 0.f, 0.f};
+  ld4v(a.proj, F32, (size_t)t * a.proj_stride + a.off + c, cur);
+#pragma unroll
+  for (int j = 0; j < kMaxTaps - 1; ++j)
+    if (j < keep) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) h[j][k] = 0.f;
+      if (pos - (keep - j) >= 0) ld4v(st, F32, (size_t)j * a.C, h[j]);
+    }
+  if (a.b) ld4v(a.b, true, c, acc);
+#pragma unroll
+  for (int j = 0; j < kMaxTaps - 1; ++j)
+    if (j < keep) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) acc[k] += a.w[(size_t)(c + k) * a.taps + j] * h[j][k];
+    }
+  float o[4];
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float z = acc[k] + a.w[(size_t)(c + k) * a.taps + keep] * cur[k];
+    o[k] = c + k >= a.silu_from ? siluf(z) : z;
+  }
+  st4((TO*)a.out + (size_t)t * a.C + c, o);
+#pragma unroll
+  for (int j = 0; j < kMaxTaps - 1; ++j)
+    if (j < keep) {
+      // (the index stays inside h where the compiler cannot see that keep bounds it)
+      if (j + 1 < keep) st4(st + (size_t)j * a.C, h[j + 1 < kMaxTaps - 1 ? j + 1 : j]);
+      else st4(st + (size_t)j * a.C, cur);
+    }
 }
 
 // a thread per (sequence, channel): the last taps - 1 inputs of the sequence go to its slot
@@ -856,6 +991,30 @@ void launch_conv_silu(void* out, bool out_f32, const void* proj, int proj_stride
   const bool vec = C % 4 == 0 && off % 4 == 0 && proj_stride % 4 == 0 &&
                    (uintptr_t)proj % (4 * es) == 0 && (uintptr_t)state % (4 * es) == 0 &&
                    (uintptr_t)out % 16 == 0 && (uintptr_t)b % 16 == 0;
+  if (vec && !q_start) {
+    const dim3 gs(T, (C / 4 + 255) / 256);
+    if (f32) conv_step_kernel<float, float><<<gs, 256, 0, s>>>(a);
+    else if (out_f32) conv_step_kernel<bf16, float><<<gs, 256, 0, s>>>(a);
+    else conv_step_kernel<bf16, bf16><<<gs, 256, 0, s>>>(a);
+    return;
+  }
+  const bool vec8 = vec && !f32 && C % 8 == 0 && off % 8 == 0 && proj_stride % 8 == 0 &&
+                    (uintptr_t)proj % 16 == 0 && (uintptr_t)state % 16 == 0 && taps >= 2 &&
+                    taps <= 4;
+  if (vec8) {
+    const dim3 g8((T + kConvRows8 - 1) / kConvRows8, (C / 8 + 127) / 128);
+#define AKAP_CONV8(TO)                                                           \
+  do {                                                                           \
+    if (taps == 2) conv_silu_vec8_kernel<TO, 2><<<g8, 128, 0, s>>>(a);           \
+    else if (taps == 3) conv_silu_vec8_kernel<TO, 3><<<g8, 128, 0, s>>>(a);      \
+    else conv_silu_vec8_kernel<TO, 4><<<g8, 128, 0, s>>>(a);                     \
+  } while (0)
+    if (out_f32) AKAP_CONV8(float);
+    else AKAP_CONV8(bf16);
+#undef AKAP_CONV8
+    conv_state_kernel<bf16><<<g2, 256, 0, s>>>(a);
+    return;
+  }
 #define AKAP_CONV(TY, TO)                                              \
   do {                                                                 \
     if (vec) conv_silu_vec_kernel<TY, TO><<<g4, 256, 0, s>>>(a, RB);   \

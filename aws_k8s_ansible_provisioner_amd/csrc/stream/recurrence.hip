@@ -382,6 +382,63 @@ __global__ __launch_bounds__(256) void norm_gate_kernel(T* __restrict__ out, int
   }
 }
 
+// the same with the row's values, gates and weights held in registers (sizes in fours, aligned):
+// LG lanes per part (a power of two up to a wave, or all 256 threads for one part), NV groups of
+// four per lane
+template <typename T, int NV, bool ALL>
+__global__ __launch_bounds__(256) void norm_gate_vec_kernel(
+    T* __restrict__ out, int out_stride, const float* __restrict__ y, const T* __restrict__ gate,
+    int gate_stride, const float* __restrict__ w, const float* __restrict__ den,
+    const float* __restrict__ floor, int silu, int n, int groups, int LG, float eps) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, part = n / groups;
+  const float* yr = y + (size_t)t * n;
+  const T* gr = gate + (size_t)t * gate_stride;
+  T* o = out + (size_t)t * out_stride;
+  const int lanes = ALL ? 256 : LG, ln = ALL ? threadIdx.x : threadIdx.x & (LG - 1);
+  for (int g = ALL ? 0 : threadIdx.x / LG; g < groups; g += ALL ? 1 : 256 / LG) {
+    const int c0 = g * part;
+    float4 v[NV], wv[NV];
+    float gv[NV][4];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+      const int c = (k * lanes + ln) * 4;
+      if (c < part) {
+        v[k] = *(const float4*)(yr + c0 + c);
+        ld4(gr + c0 + c, gv[k]);
+        wv[k] = *(const float4*)(w + c0 + c);
+      } else {
+        v[k] = wv[k] = make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+      ss += v[k].x * v[k].x + v[k].y * v[k].y + v[k].z * v[k].z + v[k].w * v[k].w;
+    float scale = 1.0f;
+    if (den) {
+      const size_t i = (size_t)t * groups + g;
+      scale = 1.0f / (fmaxf(fabsf(den[i]), floor[i]) + 1e-6f);
+    }
+    if (ALL) {
+      ss = block_sum(ss, scratch);
+    } else {
+      for (int x = LG >> 1; x > 0; x >>= 1) ss += __shfl_xor(ss, x, 64);
+    }
+    const float inv = scale / sqrtf(ss * scale * scale / (float)part + eps);
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+      const int c = (k * lanes + ln) * 4;
+      if (c >= part) continue;
+      T r[4] = {(T)(v[k].x * inv * wv[k].x * gatef(gv[k][0], silu)),
+                (T)(v[k].y * inv * wv[k].y * gatef(gv[k][1], silu)),
+                (T)(v[k].z * inv * wv[k].z * gatef(gv[k][2], silu)),
+                (T)(v[k].w * inv * wv[k].w * gatef(gv[k][3], silu))};
+      __builtin_memcpy(o + c0 + c, r, sizeof(r));
+    }
+  }
+}
+
 // lanes per column group and columns per workgroup
 void scan_shape(int D, int V, int* dp, int* vb) {
   int p = 1;
@@ -435,6 +492,33 @@ void launch_norm_gate(void* out, int out_stride, const float* y, const void* gat
   auto al = [](const void* p, int bytes) { return ((uintptr_t)p % bytes) == 0; };
   const int vec = part % 4 == 0 && out_stride % 4 == 0 && gate_stride % 4 == 0 && al(y, 16) &&
                   al(w, 16) && al(out, 4 * es) && al(gate, 4 * es);
+  int lg = 1;
+  while (lg < 64 && lg * 4 < part) lg <<= 1;
+  const bool all = groups == 1 && part > 256;
+  const int nv = (part + (all ? 1023 : lg * 4 - 1)) / (all ? 1024 : lg * 4);
+  if (vec && nv <= 4) {
+#define AKAP_NG1(TY, N, A)                                                                        \
+  norm_gate_vec_kernel<TY, N, A><<<rows, 256, 0, s>>>((TY*)out, out_stride, y, (const TY*)gate,   \
+                                                      gate_stride, w, den, floor, act, n, groups, \
+                                                      lg, eps)
+#define AKAP_NG(TY)                                                               \
+  do {                                                                            \
+    if (all) {                                                                    \
+      if (nv == 1) AKAP_NG1(TY, 1, true);                                         \
+      else if (nv == 2) AKAP_NG1(TY, 2, true);                                    \
+      else AKAP_NG1(TY, 4, true);                                                 \
+    } else {                                                                      \
+      if (nv == 1) AKAP_NG1(TY, 1, false);                                        \
+      else if (nv == 2) AKAP_NG1(TY, 2, false);                                   \
+      else AKAP_NG1(TY, 4, false);                                                \
+    }                                                                             \
+  } while (0)
+    if (f32) AKAP_NG(float);
+    else AKAP_NG(bf16);
+#undef AKAP_NG
+#undef AKAP_NG1
+    return;
+  }
   if (f32)
     norm_gate_kernel<float><<<rows, 256, 0, s>>>((float*)out, out_stride, y, (const float*)gate,
                                                  gate_stride, w, den, floor, act, n, groups, eps,

@@ -554,14 +554,22 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(ChunkParams p) {
   float* ms = r.m_state + (size_t)slot * r.H + h;
   float m = r.positions[first] == 0 ? 0.f : *ms;
   const float fb = r.pa[h], ib = r.pb[h], icap = 1.0f / r.cap;
+  auto fetch = [&](int row, bf16& f, bf16& i) {
+    const bf16* pr = (const bf16*)r.proj + (size_t)min(row, end - 1) * r.proj_stride;
+    f = pr[r.a_off + h];
+    i = pr[r.b_off + h];
+  };
+  bf16 nf, ni;                         // the next 64 tokens' inputs, in flight
+  fetch(first + lane, nf, ni);
   for (int r0 = first; r0 < end; r0 += 64) {
     const int row = r0 + lane;
     const bool live = row < end;
     float f = 0.f, i = -INFINITY;      // past the end: the identity
+    const float zf = (float)nf, zi = (float)ni;
+    fetch(row + 64, nf, ni);
     if (live) {
-      const bf16* pr = (const bf16*)r.proj + (size_t)row * r.proj_stride;
-      f = -softplusf(-r.cap * tanhf(((float)pr[r.a_off + h] + fb) * icap));
-      i = r.cap * tanhf(((float)pr[r.b_off + h] + ib) * icap);
+      f = -softplusf(-r.cap * tanhf((zf + fb) * icap));
+      i = r.cap * tanhf((zi + ib) * icap);
     }
     float F = f, I = i;
     for (int o = 1; o < 64; o <<= 1) {

@@ -274,6 +274,108 @@ __global__ __launch_bounds__(256) void head_norm_cache_kernel(HeadNormParams p) 
   }
 }
 
+// The same in 16-byte pieces (D a multiple of 8 with D / 8 a power of two up to 64, Dv a multiple
+// of 8, values not normed): 8 dimensions per thread, D / 8 lanes per query / key head.  The
+// first nqk workgroups take the (row, head) pairs of q and k; the others the values, 8
+// dimensions of 8 neighbouring rows per thread: rows that fill one 8-token group of the cache
+// are transposed in registers and leave as whole 16-byte entries.
+template <typename T>
+__global__ __launch_bounds__(256) void head_norm_cache_vec_kernel(HeadNormParams p, int nqk) {
+  const int lph = p.D >> 3;
+  if ((int)blockIdx.x < nqk) {
+    const int item = (blockIdx.x * 256 + threadIdx.x) / lph, j = threadIdx.x & (lph - 1);
+    const int heads = p.H + p.G;
+    const int t = min(item / heads, p.T - 1), u = item % heads;   // the shuffles need every lane
+    const bool live = item < p.T * heads;
+    const bool isq = u < p.H;
+    const T* src = (const T*)p.proj + (size_t)t * p.proj_stride +
+                   (isq ? p.q_off + u * p.D : p.k_off + (u - p.H) * p.D);
+    const float* w = isq ? p.q_w : p.k_w;
+    const int d = j * 8;
+    float v[8];
+    ld8(src + d, v);
+    float inv = 1.0f;
+    if (p.norm_qk) {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
+      for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      inv = 1.0f / sqrtf(ss / (float)p.D + p.eps);
+    }
+    float wv[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) wv[i] = inv;
+    if (w) {
+      ld8(w + d, wv);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) wv[i] *= inv;
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= wv[i];
+    if (p.cos_sin && d < p.rot_dims) {
+      const int half = p.rot_dims >> 1;
+      const bool low = d < half;
+      const int d2 = low ? d + half : d - half, i0 = low ? d : d - half;
+      const int64_t pos = p.positions[t];
+      const float* cs = p.cos_sin + (size_t)(pos < p.max_pos ? pos : p.max_pos - 1) * p.rot_dims;
+      float v2[8], w2[8], c8[8], s8[8];
+      ld8(src + d2, v2);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) w2[i] = 1.0f;
+      if (w) ld8(w + d2, w2);
+      ld8(cs + i0, c8);
+      ld8(cs + half + i0, s8);
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        v[i] = v[i] * c8[i] + v2[i] * inv * w2[i] * (low ? -s8[i] : s8[i]);
+    }
+    if (!live) return;
+    if (isq) {
+      st8((T*)p.q_out + ((size_t)t * p.H + u) * p.D + d, v);
+      return;
+    }
+    const int64_t slot = p.slots[t];
+    if (slot < 0 || slot >= p.num_slots) return;
+    st8((T*)p.k_cache + ((size_t)(slot / p.BS * p.G + u - p.H) * p.BS + slot % p.BS) * p.D + d, v);
+    return;
+  }
+  const int per = p.G * (p.Dv >> 3);                  // threads of a group of 8 rows
+  const int item = (blockIdx.x - nqk) * 256 + threadIdx.x;
+  const int t0 = item / per * 8;
+  if (t0 >= p.T) return;
+  const int e = item % per, g = e / (p.Dv >> 3), c = (e % (p.Dv >> 3)) * 8;
+  const int n = min(8, p.T - t0);
+  const int64_t s0 = p.slots[t0];
+  bool whole = n == 8 && s0 >= 0 && (s0 & 7) == 0;
+  for (int i = 1; i < 8 && whole; ++i) whole = p.slots[t0 + i] == s0 + i;
+  const T* src = (const T*)p.proj + (size_t)t0 * p.proj_stride + p.v_off + g * p.Dv + c;
+  auto dst = [&](int64_t slot) {
+    return (T*)p.v_cache + (((size_t)(slot / p.BS * p.G + g) * (p.BS >> 3) +
+                             (slot % p.BS >> 3)) * p.Dv + c) * 8 + (slot & 7);
+  };
+  if (whole && s0 + 7 < p.num_slots) {
+    float v[8][8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ld8(src + (size_t)i * p.proj_stride, v[i]);
+    T* o = dst(s0);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const float r[8] = {v[0][k], v[1][k], v[2][k], v[3][k], v[4][k], v[5][k], v[6][k], v[7][k]};
+      st8(o + k * 8, r);
+    }
+    return;
+  }
+  for (int i = 0; i < n; ++i) {
+    const int64_t slot = p.slots[t0 + i];
+    if (slot < 0 || slot >= p.num_slots) continue;
+    float v[8];
+    ld8(src + (size_t)i * p.proj_stride, v);
+    T* o = dst(slot);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) stf(o + k * 8, v[k]);
+  }
+}
+
 // ------------------------------------------------------------------ retention
 // One workgroup per (sequence, head).  The state S[d][v] stays in registers over the sequence's
 // rows of this step: a thread owns RET_VR neighbouring state columns v and, of their rows d,
@@ -905,6 +1007,18 @@ void launch_post_norm_add_norm(void* out, bool out_f32, int out_stride, float* x
 
 void launch_head_norm_cache(const HeadNormParams& p, bool f32, hipStream_t s) {
   if (p.T <= 0) return;
+  const int lph = p.D >> 3, half = p.rot_dims >> 1;
+  if (!p.norm_v && p.D % 8 == 0 && lph <= 64 && (lph & (lph - 1)) == 0 && p.Dv % 8 == 0 &&
+      half % 8 == 0 && ((p.proj_stride | p.q_off | p.k_off | p.v_off) & 7) == 0 && p.BS % 8 == 0 &&
+      (((uintptr_t)p.proj | (uintptr_t)p.q_out | (uintptr_t)p.k_cache | (uintptr_t)p.v_cache |
+        (uintptr_t)p.q_w | (uintptr_t)p.k_w | (uintptr_t)p.cos_sin) & 15) == 0) {
+    const int64_t qk = (int64_t)p.T * (p.H + p.G) * lph;
+    const int64_t vt = (int64_t)((p.T + 7) / 8) * p.G * (p.Dv >> 3);
+    const int nqk = (int)((qk + 255) / 256), nvb = (int)((vt + 255) / 256);
+    if (f32) head_norm_cache_vec_kernel<float><<<nqk + nvb, 256, 0, s>>>(p, nqk);
+    else head_norm_cache_vec_kernel<bf16><<<nqk + nvb, 256, 0, s>>>(p, nqk);
+    return;
+  }
   if (f32) head_norm_cache_kernel<float><<<p.T, 256, 0, s>>>(p);
   else head_norm_cache_kernel<bf16><<<p.T, 256, 0, s>>>(p);
 }
