@@ -162,6 +162,8 @@ def run_steps(kind, dtype, H, G, D, V, dev, seed):
         slot, pos, qs = step_rows(st, dev)
         qkv = torch.randn(T, 2 * G * D + HV + 8, generator=g)
         gates = torch.randn(T, HV + 2 * H, generator=g)
+        # rows of a multiple of 8 elements, like the model's projections: the chunked form takes them
+        gates = torch.nn.functional.pad(gates, (0, -(2 * G * D + 2 * HV + 2 * H) % 8))
         out = torch.zeros(T, HV + 8, dtype=dt, device=dev)
         if kind == "delta":
             qkv, proj = qkv.to(dt).to(dev), gates.to(dt).to(dev)
@@ -201,7 +203,8 @@ def test_recurrence_kernels(kind, H, G, D, V, dtype):
         if i < len(a) - ns:
             close(n, c, dtype, scale=4.0)
         else:
-            tol = 2e-4 if dtype == "float32" else 1e-2
+            # (bf16: the chunked form rounds activated q, k, v of the plain recurrence once more)
+            tol = 2e-4 if dtype == "float32" else 1e-2 if kind in ("all", "head") else 3e-4
             err = (n.cpu() - c).abs().max() / c.abs().max()
             assert err < tol, (i, err.item())
 
