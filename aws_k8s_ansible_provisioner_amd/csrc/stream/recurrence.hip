@@ -33,10 +33,22 @@ __device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + __exp
 __device__ __forceinline__ float gatef(float z, int silu) { return silu ? z * sigmoidf(z) : sigmoidf(z); }
 __device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
+// sum over the DP neighbouring lanes of a group (a power of two; every lane of the wave takes
+// part): lane swaps inside a row of 16 on DPP, wider ones by exchange
+__device__ __forceinline__ float group_sum(float v, int DP) {
+  if (DP > 1) v += akap::dpp_mov<0xB1>(v);
+  if (DP > 2) v += akap::dpp_mov<0x4E>(v);
+  if (DP > 4) v += akap::dpp_mov<0x141>(v);
+  if (DP > 8) v += akap::dpp_mov<0x140>(v);
+  if (DP > 16) v += __shfl_xor(v, 16, 64);
+  if (DP > 32) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
 // ------------------------------------------------------------------ scan
 // One workgroup per (sequence, head, VB state columns), at most 256 threads.  A thread keeps
-// VR = 4 neighbouring state columns and, of their D rows, DREG / 4 groups of four (group j of lane
-// part `part` covers d = 4 (j DP + part) ..+4, so the DP lanes of a column group read and write
+// VR = 4 neighbouring state columns and, of their D rows, 4 groups of four (group j of lane part
+// `part` covers d = 4 (j DP + part) ..+4, so the DP lanes of a column group read and write
 // consecutive 16-byte pieces of the stored state and of the staged rows).  Rows are staged TC at
 // a time; the recurrence then runs over them without a barrier: the DP lanes of a column group
 // add their partial sums by lane exchange.  The normaliser of the matrix memory is one more
@@ -47,7 +59,10 @@ constexpr int kVR = 4;
 constexpr int kDreg = 16;
 constexpr int kTokens = 16;
 
-template <typename T, int MODE>
+// VEC: D a multiple of 4 (16-byte pieces of the stored state; lanes past D or the columns load a
+// valid piece that is masked once the first rows are staged, so that the loads of state and rows
+// are in flight together)
+template <typename T, int MODE, bool VEC>
 __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
   extern __shared__ __align__(16) float lds[];
   constexpr int NJ = kDreg / 4;
@@ -74,27 +89,26 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
   const bool fresh = p.positions[r0] == 0;
   float* sbase = p.state + (((size_t)slot * p.H + h) * p.V + c_lo) * p.D;
   float* nbase = MODE == kMatrixMemory ? p.n_state + ((size_t)slot * p.H + h) * p.D : nullptr;
-  const bool vec = (p.D & 3) == 0;
-  auto load4 = [&](const float* sp, int d) {
+  auto load4 = [&](const float* col, int d, bool live) {
     float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (vec) {
-      if (d < p.D) t = *(const float4*)sp;
-    } else {
-      if (d < p.D) t.x = sp[0];
-      if (d + 1 < p.D) t.y = sp[1];
-      if (d + 2 < p.D) t.z = sp[2];
-      if (d + 3 < p.D) t.w = sp[3];
+    if (VEC) {
+      t = *(const float4*)(col + min(d, p.D - 4));
+    } else if (live) {
+      if (d < p.D) t.x = col[d];
+      if (d + 1 < p.D) t.y = col[d + 1];
+      if (d + 2 < p.D) t.z = col[d + 2];
+      if (d + 3 < p.D) t.w = col[d + 3];
     }
     return t;
   };
-  auto store4 = [&](float* sp, int d, float x, float y, float z, float w) {
-    if (vec) {
-      if (d < p.D) *(float4*)sp = make_float4(x, y, z, w);
+  auto store4 = [&](float* col, int d, float x, float y, float z, float w) {
+    if (VEC) {
+      if (d < p.D) *(float4*)(col + d) = make_float4(x, y, z, w);
     } else {
-      if (d < p.D) sp[0] = x;
-      if (d + 1 < p.D) sp[1] = y;
-      if (d + 2 < p.D) sp[2] = z;
-      if (d + 3 < p.D) sp[3] = w;
+      if (d < p.D) col[d] = x;
+      if (d + 1 < p.D) col[d + 1] = y;
+      if (d + 2 < p.D) col[d + 2] = z;
+      if (d + 3 < p.D) col[d + 3] = w;
     }
   };
   float S[kVR][kDreg], N[kDreg];
@@ -103,12 +117,11 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
     const int d = 4 * (j * DP + part);
 #pragma unroll
     for (int r = 0; r < kVR; ++r) {
-      float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (!fresh && v0 + r < nv) t = load4(sbase + (size_t)(v0 + r) * p.D + d, d);
+      const float4 t = load4(sbase + (size_t)min(v0 + r, nv - 1) * p.D, d, !fresh && v0 + r < nv);
       S[r][4 * j] = t.x; S[r][4 * j + 1] = t.y; S[r][4 * j + 2] = t.z; S[r][4 * j + 3] = t.w;
     }
     float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (MODE == kMatrixMemory && !fresh) t = load4(nbase + d, d);
+    if (MODE == kMatrixMemory) t = load4(nbase, d, !fresh);
     N[4 * j] = t.x; N[4 * j + 1] = t.y; N[4 * j + 2] = t.z; N[4 * j + 3] = t.w;
   }
   if (MODE == kMatrixMemory && tid == 0)
@@ -208,6 +221,15 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
       }
       __syncthreads();
     }
+    if (VEC && c0 == r0) {
+#pragma unroll
+      for (int i = 0; i < kDreg; ++i) {
+        const bool in = !fresh && 4 * ((i >> 2) * DP + part) < p.D;
+#pragma unroll
+        for (int r = 0; r < kVR; ++r) S[r][i] = in && v0 + r < nv ? S[r][i] : 0.f;
+        if (MODE == kMatrixMemory) N[i] = in ? N[i] : 0.f;
+      }
+    }
     // the recurrence
     for (int tk = 0; tk < n; ++tk) {
       float4 vv = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -233,10 +255,8 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
             S[r][i] *= dec;
             seen[r] = fmaf(S[r][i], kk[i], seen[r]);
           }
-        for (int o = DP >> 1; o > 0; o >>= 1) {
 #pragma unroll
-          for (int r = 0; r < kVR; ++r) seen[r] += __shfl_xor(seen[r], o, 64);
-        }
+        for (int r = 0; r < kVR; ++r) seen[r] = group_sum(seen[r], DP);
         const float beta = g1[tk], ik = g3[tk];
 #pragma unroll
         for (int r = 0; r < kVR; ++r) vr[r] = beta * (vr[r] - ik * seen[r]) * ik;
@@ -277,11 +297,9 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
           }
         }
       }
-      for (int o = DP >> 1; o > 0; o >>= 1) {
 #pragma unroll
-        for (int r = 0; r < kVR; ++r) acc[r] += __shfl_xor(acc[r], o, 64);
-        if (MODE == kMatrixMemory) accn += __shfl_xor(accn, o, 64);
-      }
+      for (int r = 0; r < kVR; ++r) acc[r] = group_sum(acc[r], DP);
+      if (MODE == kMatrixMemory) accn = group_sum(accn, DP);
       float f = 1.0f;
       if (MODE == kMatrixMemory) f = 1.0f / (fmaxf(fabsf(accn), g2[tk]) + 1e-6f);
       if (MODE == kDelta) f = g2[tk];
@@ -319,13 +337,184 @@ __global__ __launch_bounds__(256) void recurrence_kernel(RecurrenceParams p) {
 #pragma unroll
     for (int r = 0; r < kVR; ++r)
       if (v0 + r < nv)
-        store4(sbase + (size_t)(v0 + r) * p.D + d, d, S[r][4 * j], S[r][4 * j + 1],
+        store4(sbase + (size_t)(v0 + r) * p.D, d, S[r][4 * j], S[r][4 * j + 1],
                S[r][4 * j + 2], S[r][4 * j + 3]);
     if (MODE == kMatrixMemory && v0 == 0 && blockIdx.z == 0)
-      store4(nbase + d, d, N[4 * j], N[4 * j + 1], N[4 * j + 2], N[4 * j + 3]);
+      store4(nbase, d, N[4 * j], N[4 * j + 1], N[4 * j + 2], N[4 * j + 3]);
   }
   if (MODE == kMatrixMemory && tid == 0 && blockIdx.z == 0)
     p.m_state[(size_t)slot * p.H + h] = mrun[0];
+}
+
+// ------------------------------------------------------------------ one token per sequence
+// The same for steps of single rows, which only stream the state in and out: a workgroup per
+// (row, head), up to 1024 threads.  Nothing is staged: a lane loads the pieces of q and k that
+// meet its state rows, everything before the head norm happens inside the lanes of a column
+// group, and all loads are issued together.  Sizes in fours, aligned.
+template <typename T, int MODE, int DREG>
+__global__ __launch_bounds__(1024) void recurrence_step_kernel(RecurrenceParams p) {
+  __shared__ float scratch[16];
+  constexpr int NJ = DREG / 4;
+  const int DP = p.DP;
+  const int t = blockIdx.x, h = blockIdx.y;
+  const int slot = p.seq_slot[t];
+  if (slot < 0 || slot >= p.num_slots) return;
+  const int tid = threadIdx.x, hq = h / (p.H / p.G);
+  const int v0 = (tid / DP) * kVR, part = tid % DP;
+  const bool col = v0 < p.V;
+  const int vc = col ? v0 : p.V - kVR;
+  const T* row = (const T*)p.qkv + (size_t)t * p.qkv_stride;
+  const T* pr = (const T*)p.proj + (size_t)t * p.proj_stride;
+  float* sp = p.state + (((size_t)slot * p.H + h) * p.V + vc) * p.D;
+  float* np = MODE == kMatrixMemory ? p.n_state + ((size_t)slot * p.H + h) * p.D : nullptr;
+  float q[DREG], k[DREG], v[kVR];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int d = min(4 * (j * DP + part), p.D - 4);
+    float q4[4], k4[4];
+    ld4(row + p.q_off + hq * p.D + d, q4);
+    ld4(row + p.k_off + hq * p.D + d, k4);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      q[4 * j + i] = q4[i];
+      k[4 * j + i] = k4[i];
+    }
+  }
+  ld4(row + p.v_off + h * p.V + vc, v);
+  akap::f32x4 S[kVR][NJ], N[NJ];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int d = min(4 * (j * DP + part), p.D - 4);
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) S[r][j] = *(const akap::f32x4*)(sp + r * p.D + d);
+    if (MODE == kMatrixMemory) N[j] = *(const akap::f32x4*)(np + d);
+  }
+  const bool fresh = p.positions[t] == 0;
+  float dec, add = 1.f, floor_m = 0.f, m2 = 0.f;
+  if (MODE == kDecay) {
+    dec = p.pa[h];
+  } else if (MODE == kMatrixMemory) {
+    const float f = -softplusf(-p.cap * tanhf((ldf(pr + p.a_off + h) + p.pa[h]) / p.cap));
+    const float i = p.cap * tanhf((ldf(pr + p.b_off + h) + p.pb[h]) / p.cap);
+    const float m = fresh ? 0.f : p.m_state[(size_t)slot * p.H + h];
+    m2 = fmaxf(f + m, i);
+    dec = expf(f + m - m2);
+    add = expf(i - m2);
+    floor_m = expf(-m2);
+  } else {
+    dec = expf(-expf(p.pa[h]) * softplusf(ldf(pr + p.a_off + h) + p.pb[h]));
+    add = 1.0f / (1.0f + expf(-ldf(pr + p.b_off + h)));   // the step size
+  }
+  if (fresh) dec = 0.f;
+  const float qs = MODE == kDelta ? 1.0f : p.q_scale;
+#pragma unroll
+  for (int i = 0; i < DREG; ++i) {
+    const bool in = 4 * ((i >> 2) * DP + part) < p.D;
+    if (p.act) {
+      q[i] *= sigmoidf(q[i]);
+      k[i] *= sigmoidf(k[i]);
+    }
+    q[i] = in ? q[i] * qs : 0.f;
+    k[i] = in ? k[i] : 0.f;
+  }
+  if (p.act) {
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) v[r] *= sigmoidf(v[r]);
+  }
+  // a fresh row: the slot's stale contents (which may be anything) do not enter
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+#pragma unroll
+      for (int r = 0; r < kVR; ++r) S[r][j][i] = fresh ? 0.f : S[r][j][i];
+      if (MODE == kMatrixMemory) N[j][i] = fresh ? 0.f : N[j][i];
+    }
+  }
+  float acc[kVR] = {0.f, 0.f, 0.f, 0.f}, f = 1.0f;
+  if (MODE == kDelta) {
+    float seen[kVR] = {0.f, 0.f, 0.f, 0.f}, sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+#pragma unroll
+      for (int r = 0; r < kVR; ++r) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          S[r][j][i] *= dec;
+          seen[r] = fmaf(S[r][j][i], k[4 * j + i], seen[r]);
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        sq = fmaf(q[4 * j + i], q[4 * j + i], sq);
+        sk = fmaf(k[4 * j + i], k[4 * j + i], sk);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) seen[r] = group_sum(seen[r], DP);
+    const float ik = 1.0f / sqrtf(group_sum(sk, DP) + 1e-6f);
+    f = p.q_scale / sqrtf(group_sum(sq, DP) + 1e-6f);
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) v[r] = add * (v[r] - ik * seen[r]) * ik;
+    dec = 1.f;
+  } else {
+#pragma unroll
+    for (int r = 0; r < kVR; ++r) v[r] *= add;
+  }
+  float accn = 0.f;
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+#pragma unroll
+      for (int r = 0; r < kVR; ++r) {
+        S[r][j][i] = fmaf(dec, S[r][j][i], k[4 * j + i] * v[r]);
+        acc[r] = fmaf(S[r][j][i], q[4 * j + i], acc[r]);
+      }
+      if (MODE == kMatrixMemory) {
+        N[j][i] = fmaf(dec, N[j][i], k[4 * j + i] * add);
+        accn = fmaf(N[j][i], q[4 * j + i], accn);
+      }
+    }
+  }
+  // the state leaves before the sums are finished (the normaliser: every column group has read it
+  // by the barrier below)
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) {
+    const int d = 4 * (j * DP + part);
+    if (col && d < p.D)
+#pragma unroll
+      for (int r = 0; r < kVR; ++r) *(akap::f32x4*)(sp + r * p.D + d) = S[r][j];
+  }
+#pragma unroll
+  for (int r = 0; r < kVR; ++r) acc[r] = group_sum(acc[r], DP);
+  if (MODE == kMatrixMemory) f = 1.0f / (fmaxf(fabsf(group_sum(accn, DP)), floor_m) + 1e-6f);
+  float ss = 0.f;
+#pragma unroll
+  for (int r = 0; r < kVR; ++r) {
+    acc[r] = col ? acc[r] * f : 0.f;
+    ss += acc[r] * acc[r];
+  }
+  ss = block_sum(part == 0 ? ss : 0.f, scratch);
+  if (MODE == kMatrixMemory && v0 == 0) {
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const int d = 4 * (j * DP + part);
+      if (d < p.D) *(akap::f32x4*)(np + d) = N[j];
+    }
+    if (part == 0) p.m_state[(size_t)slot * p.H + h] = m2;
+  }
+  if (!col || part != 0) return;
+  if (p.raw) {
+    *(float4*)(p.raw + ((size_t)t * p.H + h) * p.V + v0) = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    return;
+  }
+  const float inv = 1.0f / sqrtf(ss / (float)p.V + p.eps);
+  const T* g = pr + p.g_off + h * p.V + v0;
+  T* o = (T*)p.out + (size_t)t * p.out_stride + h * p.V + v0;
+#pragma unroll
+  for (int r = 0; r < kVR; ++r)
+    stf(o + r, acc[r] * inv * p.norm_w[h * p.V + v0 + r] * gatef(ldf(g + r), p.gate_act));
 }
 
 // ------------------------------------------------------------------ head norm + output gate
@@ -439,7 +628,7 @@ __global__ __launch_bounds__(256) void norm_gate_vec_kernel(
   }
 }
 
-// lanes per column group and columns per workgroup
+// lanes per column group and columns per workgroup of the scan
 void scan_shape(int D, int V, int* dp, int* vb) {
   int p = 1;
   while (p * kDreg < D) p <<= 1;
@@ -448,15 +637,55 @@ void scan_shape(int D, int V, int* dp, int* vb) {
   *vb = V <= cols ? V : cols;
 }
 
+// state rows per thread of the single-row form (0: too large for a workgroup) and its lanes per
+// column group
+int step_shape(int D, int V, int* dp) {
+  for (int dreg : {8, 16}) {
+    int p = 1;
+    while (p * dreg < D) p <<= 1;
+    *dp = p;
+    if (p <= 64 && (V / kVR) * p <= (dreg == 8 ? 512 : 1024)) return dreg;
+  }
+  return 0;
+}
+
 }  // namespace
 
 // ================================================================== launchers
-bool recurrence_supported(int D, int V) { return D >= 1 && D <= 64 * kDreg && V >= 1; }
+bool recurrence_supported(int D, int V) { return D >= 1 && D <= 64 * 16 && V >= 1; }
 
 bool recurrence_fused(int D, int V) {
   int dp, vb;
   scan_shape(D, V, &dp, &vb);
   return vb == V;
+}
+
+bool recurrence_step_supported(int D, int V) {
+  int dp;
+  return D >= 4 && V >= 4 && D % 4 == 0 && V % 4 == 0 && step_shape(D, V, &dp) > 0;
+}
+
+void launch_recurrence_step(RecurrenceParams p, int mode, bool f32, hipStream_t s) {
+  if (p.num_seqs <= 0) return;
+  const int dreg = step_shape(p.D, p.V, &p.DP);
+  const int nt = ((p.V / kVR * p.DP + 63) / 64) * 64;
+  const dim3 grid(p.num_seqs, p.H);
+#define AKAP_ST1(TY, R)                                                                       \
+  do {                                                                                        \
+    if (mode == kDecay) recurrence_step_kernel<TY, kDecay, R><<<grid, nt, 0, s>>>(p);         \
+    else if (mode == kMatrixMemory)                                                           \
+      recurrence_step_kernel<TY, kMatrixMemory, R><<<grid, nt, 0, s>>>(p);                    \
+    else recurrence_step_kernel<TY, kDelta, R><<<grid, nt, 0, s>>>(p);                        \
+  } while (0)
+#define AKAP_ST(TY)                     \
+  do {                                  \
+    if (dreg == 8) AKAP_ST1(TY, 8);     \
+    else AKAP_ST1(TY, 16);              \
+  } while (0)
+  if (f32) AKAP_ST(float);
+  else AKAP_ST(bf16);
+#undef AKAP_ST
+#undef AKAP_ST1
 }
 
 void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s) {
@@ -472,16 +701,22 @@ void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s) {
   while (p.TC > 1 && need(p.TC) > 65536) p.TC >>= 1;
   const size_t lds = need(p.TC);
   const dim3 grid(p.num_seqs, p.H, (p.V + p.VB - 1) / p.VB);
-#define AKAP_REC(TY)                                                                          \
+#define AKAP_REC1(TY, VC)                                                                      \
   do {                                                                                        \
-    if (mode == kDecay) recurrence_kernel<TY, kDecay><<<grid, nt, lds, s>>>(p);               \
+    if (mode == kDecay) recurrence_kernel<TY, kDecay, VC><<<grid, nt, lds, s>>>(p);           \
     else if (mode == kMatrixMemory)                                                           \
-      recurrence_kernel<TY, kMatrixMemory><<<grid, nt, lds, s>>>(p);                          \
-    else recurrence_kernel<TY, kDelta><<<grid, nt, lds, s>>>(p);                              \
+      recurrence_kernel<TY, kMatrixMemory, VC><<<grid, nt, lds, s>>>(p);                      \
+    else recurrence_kernel<TY, kDelta, VC><<<grid, nt, lds, s>>>(p);                          \
+  } while (0)
+#define AKAP_REC(TY)                       \
+  do {                                     \
+    if (p.D % 4 == 0) AKAP_REC1(TY, true); \
+    else AKAP_REC1(TY, false);             \
   } while (0)
   if (f32) AKAP_REC(float);
   else AKAP_REC(bf16);
 #undef AKAP_REC
+#undef AKAP_REC1
 }
 
 void launch_norm_gate(void* out, int out_stride, const float* y, const void* gate, int gate_stride,

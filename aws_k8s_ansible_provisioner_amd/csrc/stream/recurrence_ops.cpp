@@ -125,7 +125,7 @@ void recurrence(int64_t mode, Tensor out, std::optional<Tensor> raw, Tensor qkv,
                 Tensor state, std::optional<Tensor> n_state, std::optional<Tensor> m_state,
                 Tensor norm_w, int64_t g_off, int64_t gate_act, double eps, Tensor seq_slot,
                 Tensor positions, std::optional<Tensor> q_start, int64_t H, int64_t G, int64_t D,
-                int64_t V) {
+                int64_t V, bool step) {
   auto p = recurrence_params(mode, qkv, q_off, k_off, v_off, act, proj, a_off, b_off, pa, pb, cap,
                              q_scale, state, n_state, m_state, seq_slot, positions, q_start, H, G,
                              D, V);
@@ -134,7 +134,7 @@ void recurrence(int64_t mode, Tensor out, std::optional<Tensor> raw, Tensor qkv,
   TORCH_CHECK(out.size(1) == H * V && out.scalar_type() == qkv.scalar_type(),
               "recurrence: out [T, H V] of qkv's type");
   TORCH_CHECK(g_off >= 0 && g_off + H * V <= proj.size(1), "recurrence: gate outside the projection");
-  TORCH_CHECK(raw.has_value() || akap_stream::recurrence_fused((int)D, (int)V),
+  TORCH_CHECK(raw.has_value() || step || akap_stream::recurrence_fused((int)D, (int)V),
               "recurrence: this head size needs raw");
   p.out = out.data_ptr(); p.out_stride = (int)out.stride(0);
   p.raw = raw ? f32_ptr(*raw, T * H * V, "raw") : nullptr;
@@ -142,6 +142,14 @@ void recurrence(int64_t mode, Tensor out, std::optional<Tensor> raw, Tensor qkv,
   p.norm_w = f32_ptr(norm_w, H * V, "norm_w");
   p.eps = (float)eps;
   const c10::DeviceGuard g(qkv.device());
+  if (step) {
+    TORCH_CHECK(!q_start.has_value() && akap_stream::recurrence_step_supported((int)D, (int)V) &&
+                    ((q_off | k_off | v_off | qkv.stride(0)) & 3) == 0 &&
+                    ((uintptr_t)qkv.data_ptr() & 15) == 0,
+                "recurrence: the single-row form needs sizes, offsets and strides in fours");
+    akap_stream::launch_recurrence_step(p, (int)mode, is_f32(qkv, "qkv"), cur_stream());
+    return;
+  }
   akap_stream::launch_recurrence(p, (int)mode, is_f32(qkv, "qkv"), cur_stream());
 }
 
@@ -197,6 +205,10 @@ std::vector<int64_t> chunk_workspace(int64_t mode, int64_t chunks, int64_t H, in
   return {nh, nf};
 }
 
+bool recurrence_step_supported(int64_t D, int64_t V) {
+  return akap_stream::recurrence_step_supported((int)D, (int)V);
+}
+
 bool recurrence_fused(int64_t D, int64_t V) {
   return akap_stream::recurrence_fused((int)D, (int)V);
 }
@@ -210,7 +222,7 @@ TORCH_LIBRARY_FRAGMENT(akap_stream, m) {
         "int v_off, int act, Tensor proj, int a_off, int b_off, Tensor pa, Tensor? pb, float cap, "
         "float q_scale, Tensor(c!) state, Tensor(d!)? n_state, Tensor(e!)? m_state, Tensor norm_w, "
         "int g_off, int gate_act, float eps, Tensor seq_slot, Tensor positions, Tensor? q_start, "
-        "int H, int G, int D, int V) -> ()");
+        "int H, int G, int D, int V, bool step) -> ()");
   m.def("chunk_recurrence(int mode, Tensor(a!) raw, Tensor qkv, int q_off, int k_off, int v_off, "
         "int act, Tensor proj, int a_off, int b_off, Tensor pa, Tensor? pb, float cap, "
         "float q_scale, Tensor(b!) state, Tensor(c!)? n_state, Tensor(d!)? m_state, "
@@ -218,6 +230,7 @@ TORCH_LIBRARY_FRAGMENT(akap_stream, m) {
         "int D, int V, Tensor(e!)? memory, Tensor(f!) halves, Tensor(g!) floats) -> ()");
   m.def("chunk_supported(int D) -> bool", &chunk_supported);
   m.def("chunk_workspace(int mode, int chunks, int H, int G, int D) -> int[]", &chunk_workspace);
+  m.def("recurrence_step_supported(int D, int V) -> bool", &recurrence_step_supported);
   m.def("recurrence_fused(int D, int V) -> bool", &recurrence_fused);
 }
 

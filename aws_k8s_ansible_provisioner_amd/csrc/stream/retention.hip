@@ -277,10 +277,11 @@ __global__ __launch_bounds__(256) void head_norm_cache_kernel(HeadNormParams p) 
 // The same in 16-byte pieces (D a multiple of 8 with D / 8 a power of two up to 64, Dv a multiple
 // of 8, values not normed): 8 dimensions per thread, D / 8 lanes per query / key head.  The
 // first nqk workgroups take the (row, head) pairs of q and k; the others the values, 8
-// dimensions of 8 neighbouring rows per thread: rows that fill one 8-token group of the cache
+// dimensions of vrows neighbouring rows per thread (8, or 1 for small steps): 8 rows that fill one 8-token group of the cache
 // are transposed in registers and leave as whole 16-byte entries.
 template <typename T>
-__global__ __launch_bounds__(256) void head_norm_cache_vec_kernel(HeadNormParams p, int nqk) {
+__global__ __launch_bounds__(256) void head_norm_cache_vec_kernel(HeadNormParams p, int nqk,
+                                                                  int vrows) {
   const int lph = p.D >> 3;
   if ((int)blockIdx.x < nqk) {
     const int item = (blockIdx.x * 256 + threadIdx.x) / lph, j = threadIdx.x & (lph - 1);
@@ -341,10 +342,10 @@ __global__ __launch_bounds__(256) void head_norm_cache_vec_kernel(HeadNormParams
   }
   const int per = p.G * (p.Dv >> 3);                  // threads of a group of 8 rows
   const int item = (blockIdx.x - nqk) * 256 + threadIdx.x;
-  const int t0 = item / per * 8;
+  const int t0 = item / per * vrows;
   if (t0 >= p.T) return;
   const int e = item % per, g = e / (p.Dv >> 3), c = (e % (p.Dv >> 3)) * 8;
-  const int n = min(8, p.T - t0);
+  const int n = min(vrows, p.T - t0);
   const int64_t s0 = p.slots[t0];
   bool whole = n == 8 && s0 >= 0 && (s0 & 7) == 0;
   for (int i = 1; i < 8 && whole; ++i) whole = p.slots[t0 + i] == s0 + i;
@@ -1013,10 +1014,11 @@ void launch_head_norm_cache(const HeadNormParams& p, bool f32, hipStream_t s) {
       (((uintptr_t)p.proj | (uintptr_t)p.q_out | (uintptr_t)p.k_cache | (uintptr_t)p.v_cache |
         (uintptr_t)p.q_w | (uintptr_t)p.k_w | (uintptr_t)p.cos_sin) & 15) == 0) {
     const int64_t qk = (int64_t)p.T * (p.H + p.G) * lph;
-    const int64_t vt = (int64_t)((p.T + 7) / 8) * p.G * (p.Dv >> 3);
+    const int vrows = p.T >= 512 ? 8 : 1;
+    const int64_t vt = (int64_t)((p.T + vrows - 1) / vrows) * p.G * (p.Dv >> 3);
     const int nqk = (int)((qk + 255) / 256), nvb = (int)((vt + 255) / 256);
-    if (f32) head_norm_cache_vec_kernel<float><<<nqk + nvb, 256, 0, s>>>(p, nqk);
-    else head_norm_cache_vec_kernel<bf16><<<nqk + nvb, 256, 0, s>>>(p, nqk);
+    if (f32) head_norm_cache_vec_kernel<float><<<nqk + nvb, 256, 0, s>>>(p, nqk, vrows);
+    else head_norm_cache_vec_kernel<bf16><<<nqk + nvb, 256, 0, s>>>(p, nqk, vrows);
     return;
   }
   if (f32) head_norm_cache_kernel<float><<<p.T, 256, 0, s>>>(p);

@@ -326,6 +326,10 @@ struct RecurrenceParams {
 bool recurrence_fused(int D, int V);
 bool recurrence_supported(int D, int V);
 void launch_recurrence(RecurrenceParams p, int mode, bool f32, hipStream_t s);
+// steps of single rows (q_start null), sizes, offsets and row strides in fours, 16-byte aligned
+// rows; always holds a whole head
+bool recurrence_step_supported(int D, int V);
+void launch_recurrence_step(RecurrenceParams p, int mode, bool f32, hipStream_t s);
 // chunked matrix-core form for prompt portions (recurrence_mfma.hip, bf16): the sequences of r
 // (q_start given, pointing at the first chunked sequence, whose first row is row0); r.raw takes
 // the heads as they leave the state (the matrix memory's still undivided, with den = n . q and

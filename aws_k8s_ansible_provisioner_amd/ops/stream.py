@@ -953,8 +953,8 @@ def _recurrence(mode: str, out, qkv, q_off, k_off, v_off, act, proj, gates: tupl
                 seq_slot, positions, q_start, H, G, D, V, first_seq) -> None:
     """GPU form of the recurrences below.  Prompt portions in bf16, at head sizes the matrix-core
     kernels take: chunks of 64 tokens prepared side by side, then walked with the state in
-    accumulators, followed by norm_gate.  Everything else (single rows, fp32, other sizes): the
-    scan kernel (one workgroup per sequence, head and block of state columns, state in
+    accumulators, followed by norm_gate.  Steps of single rows: one kernel from q, k, v to the
+    normed and gated heads.  Everything else (fp32 prompts, other sizes): the scan kernel (one workgroup per sequence, head and block of state columns, state in
     registers) with the head norm and the gate fused where a workgroup holds a whole head, else
     followed by norm_gate."""
     ns = torch.ops.akap_stream
@@ -983,10 +983,12 @@ def _recurrence(mode: str, out, qkv, q_off, k_off, v_off, act, proj, gates: tupl
                       gate_act, mem[2, nd:] if mem is not None else None,
                       mem[3, nd:] if mem is not None else None)
             return
-    fuse = not norm_all and ns.recurrence_fused(D, V)
+    step = q_start is None and ns.recurrence_step_supported(D, V) \
+        and (q_off | k_off | v_off | qkv.stride(0)) % 4 == 0 and qkv.data_ptr() % 16 == 0
+    fuse = not norm_all and (step or ns.recurrence_fused(D, V))
     raw = None if fuse else torch.empty(T, H * V, dtype=torch.float32, device=qkv.device)
     ns.recurrence(m, out, raw, *args, norm_w, g_off, 1 if gate_act == "silu" else 0, float(eps),
-                  seq_slot, positions, q_start, H, G, D, V)
+                  seq_slot, positions, q_start, H, G, D, V, step)
     if raw is not None:
         norm_gate(out, raw, proj[:, g_off:g_off + H * V], norm_w, groups, eps, gate_act)
 
