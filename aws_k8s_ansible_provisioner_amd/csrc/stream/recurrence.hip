@@ -644,7 +644,7 @@ int step_shape(int D, int V, int* dp) {
     int p = 1;
     while (p * dreg < D) p <<= 1;
     *dp = p;
-    if (p <= 64 && (V / kVR) * p <= (dreg == 8 ? 512 : 1024)) return dreg;
+    if (p <= 64 && (V / kVR) * p <= 1024) return dreg;
   }
   return 0;
 }
