@@ -299,15 +299,16 @@ def test_sazepel_served_with_sampling_and_no_prefix_cache():
     assert hits == 0
 
 
-def test_mudepel_served_with_sampling_and_no_prefix_cache():
-    """The multi-stream design behind the same OpenAI endpoints: convolution inputs and
-    state-space states live in the scheduler's sequence slots, so a repeated prompt must give
+@pytest.mark.parametrize("design", ["tiny-mudepel", "tiny-papivik"])
+def test_recurrent_design_served_with_sampling_and_no_prefix_cache(design):
+    """Designs with recurrent layers behind the same OpenAI endpoints: convolution inputs and
+    recurrent states live in the scheduler's sequence slots, so a repeated prompt must give
     the same greedy completion WITHOUT reusing cached pages, more prompts than slots are served
     by handing slots on (each new owner starts from zeros), and sampled requests run."""
     from aws_k8s_ansible_provisioner_amd.engine.config import EngineConfig
     from aws_k8s_ansible_provisioner_amd.server.api_server import build_app
 
-    app, ae = build_app(EngineConfig(model="tiny-mudepel", served_model_name="m", device="cpu",
+    app, ae = build_app(EngineConfig(model=design, served_model_name="m", device="cpu",
                                      dtype="float32", max_model_len=256, max_num_seqs=2,
                                      max_num_batched_tokens=48, block_size=32,
                                      num_gpu_blocks=64, enable_prefix_caching=True))
