@@ -253,15 +253,18 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
   }
   if (MODE != kDelta) return;
   __syncthreads();
-  // the inverse of I + A by forward substitution, a column per lane of one wave
+  // The inverse of I + A, by halves: both 32 x 32 diagonal blocks by forward substitution, a
+  // column per lane of one wave (lanes 0 .. 31 the upper, 32 .. 63 the lower block), then the
+  // lower left block as -T22 A21 T11.
   if (wave == 0) {
-    float x[kC];
+    const int o = lane & 32, col = lane & 31;
+    float x[32];
 #pragma unroll
-    for (int i = 0; i < kC; ++i) {
-      float a0 = lane == i ? 1.f : 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
+    for (int i = 0; i < 32; ++i) {
+      float a0 = col == i ? 1.f : 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
 #pragma unroll
       for (int j = 0; j < i; j += 4) {
-        const float4 a = *(const float4*)(am + i * AS + j);
+        const float4 a = *(const float4*)(am + (o + i) * AS + o + j);
         a0 = fmaf(-a.x, x[j], a0);
         if (j + 1 < i) a1 = fmaf(-a.y, x[j + 1], a1);
         if (j + 2 < i) a2 = fmaf(-a.z, x[j + 2], a2);
@@ -270,7 +273,31 @@ __global__ __launch_bounds__(256) void chunk_prep_kernel(ChunkParams p) {
       x[i] = (a0 + a1) + (a2 + a3);
     }
 #pragma unroll
-    for (int i = 0; i < kC; ++i) am[i * AS + lane] = x[i];
+    for (int i = 0; i < 32; ++i) am[(o + i) * AS + o + col] = x[i];
+  }
+  __syncthreads();
+  {
+    constexpr int MS = 36;
+    float* mid = (float*)qs;               // [32][MS]: q is not needed any more
+    static_assert(kC * LS * sizeof(bf16) >= 32 * MS * sizeof(float), "the product fits q's rows");
+    const int row = tid >> 3, c4 = (tid & 7) * 4;
+    auto product = [&](const float* a, const float* b, int bs) {
+      float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 8
+      for (int j = 0; j < 32; ++j) {
+        const float w = a[j];
+        const float4 v = *(const float4*)(b + j * bs + c4);
+        acc.x = fmaf(w, v.x, acc.x);
+        acc.y = fmaf(w, v.y, acc.y);
+        acc.z = fmaf(w, v.z, acc.z);
+        acc.w = fmaf(w, v.w, acc.w);
+      }
+      return acc;
+    };
+    *(float4*)(mid + row * MS + c4) = product(am + (32 + row) * AS, am, AS);
+    __syncthreads();
+    const float4 t = product(am + (32 + row) * AS + 32, mid, MS);
+    *(float4*)(am + (32 + row) * AS + c4) = make_float4(-t.x, -t.y, -t.z, -t.w);
   }
   __syncthreads();
   bf16* tf = (bf16*)p.tf + ch * kPT * kFrag;
