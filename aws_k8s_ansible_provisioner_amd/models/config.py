@@ -19,7 +19,7 @@ from typing import Optional
 class ModelConfig:
     name: str
     hf_id: str
-    arch: str  # "qwen3" | "llama" | "mixtral" | "qwen3_moe" | "bidetar" | "puputar" | "sazepel" (LayeredConfig)
+    arch: str  # "qwen3" | "llama" | "mixtral" | "qwen3_moe" | "bidetar" | "puputar" | "sazepel" | "mudepel" | "papivik" (LayeredConfig)
     vocab_size: int
     hidden_size: int
     intermediate_size: int

@@ -15,9 +15,10 @@ ONE convolution launch serves both mixers' q, k, v (silu from the delta rule's f
 a shorter kernel padded with zero taps), and both write side by side into one buffer, so the
 weighted sum of the two outputs happens in the output GEMM's fp32 accumulator: the left
 constant rides in the fp32 weights of the value convolution (the attention's output is linear
-in the values), the right one in the head norm's weights.  The recurrences share one scan kernel
-(state in registers, one launch from projection to the normed and gated heads) for decode rows
-and for sizes or types the chunked matrix-core form does not take.  The post-norm, the residual
+in the values), the right one in the head norm's weights.  The
+recurrences have one set of kernels: prompt portions in chunks of 64 tokens on the matrix cores
+with the fp32 state in accumulators, single rows in one launch from q, k, v to the normed and
+gated heads, and a scan for other sizes and types.  The post-norm, the residual
 sum and the copy of the stream that the next sublayer reads (or the model's output norm) are
 one kernel.  Decode steps are sync-free and allocation-stable, so the runner captures them in
 hipGraphs.

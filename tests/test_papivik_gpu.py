@@ -315,7 +315,7 @@ OTHER = {
         oracle.mlstm_layer(1, 40, 36, cap=2.0), oracle.lightning_layer(1, 160, 65, (0.95,)),
         oracle.parallel_layer((2, 2, 16, 64), (2, 1, 36, 40), 0.25, 16, conv=(5, 3))]),
     "matrix_core": lambda: oracle.make_config(64, 23, [
-        oracle.mlstm_layer(2, 64, 96, cap=11.0, ff=64), oracle.lightning_layer(2, 96, 32, (0.95, 0.6)),
+        oracle.mlstm_layer(2, 64, 96, cap=11.0, ff=64), oracle.lightning_layer(2, 96, 32, (0.95, 0.0)),
         oracle.parallel_layer((4, 2, 64, 64), (4, 2, 64, 32), 0.15, 32, conv=(4, 4),
                               scales=(0.8, 1.1), ff=32)]),
 }
