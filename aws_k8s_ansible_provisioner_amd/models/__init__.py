@@ -23,6 +23,10 @@ def model_class(cfg: ModelConfig):
         from .papivik import PapivikLM
 
         return PapivikLM
+    if cfg.arch == "venanex":
+        from .venanex import VenanexLM
+
+        return VenanexLM
     from .transformer import DecoderLM
 
     return DecoderLM

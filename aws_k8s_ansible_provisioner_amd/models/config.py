@@ -19,7 +19,8 @@ from typing import Optional
 class ModelConfig:
     name: str
     hf_id: str
-    arch: str  # "qwen3" | "llama" | "mixtral" | "qwen3_moe" | "bidetar" | "puputar" | "sazepel" | "mudepel" | "papivik" (LayeredConfig)
+    arch: str  # "qwen3" | "llama" | "mixtral" | "qwen3_moe" | "bidetar" | "puputar" | "sazepel" | "mudepel" | "papivik" |
+               # "venanex" (LayeredConfig)
     vocab_size: int
     hidden_size: int
     intermediate_size: int
@@ -150,6 +151,16 @@ class AttentionSpec:
     # k carry a weight vector of `dim` entries shared by the heads
     conv: int = 0
     qk_norm_w: bool = False
+    # diff given: differential attention.  A head has two queries and two keys of `dim` entries,
+    # [map 1 | map 2], each a softmax map of its own over the head's values; the second output is
+    # taken off the first lambda times (one learned number per layer, `diff` its constant part),
+    # each head is divided by its root mean square and multiplied by 1 - diff
+    diff: Optional[float] = None
+
+    @property
+    def key_dim(self) -> int:
+        """Entries of a head's query (and of a cached key)."""
+        return self.dim * (2 if self.diff is not None else 1)
 
 
 @dataclasses.dataclass
@@ -301,7 +312,7 @@ class LatentAttentionSpec:
     size kv_rank, plus a rotated key part of rot_dim dimensions shared by all heads.  A head
     has `dim` unrotated and `rot_dim` rotated query/key dimensions and values of size `vdim`.
     gate: "head" (one sigmoid per head) or "element" (one per output dimension), computed from
-    the mixer's input.  kv_from: index of an earlier layer whose cached latent and rotated key
+    the mixer's input, or "none".  kv_from: index of an earlier layer whose cached latent and rotated key
     this layer reads instead of projecting its own."""
     heads: int
     dim: int
@@ -324,6 +335,8 @@ class LatentAttentionSpec:
 
     @property
     def gate_rows(self) -> int:
+        if self.gate == "none":
+            return 0
         return self.heads if self.gate == "head" else self.heads * self.vdim
 
 
@@ -346,6 +359,8 @@ class RouterSpec:
     # renormalisation)
     kind: str = "corrected"
     group_top: int = 1
+    # what an expert's weight multiplies: its "output" or its "input"
+    weigh: str = "output"
 
     @property
     def outputs(self) -> int:
@@ -357,11 +372,16 @@ class MlpSpec:
     kind: str   # "dense": down(act(up h)) | "moe": routed experts of that form
     ff: int
     # "relu2" | "xielu" (two learned numbers per layer) | "gelu" (tanh form) | "swiglu" |
-    # "geglu" (gated, tanh form of gelu on the gate)
+    # "geglu" (gated, tanh form of gelu on the gate) | "clamped" (g = min(gate, limit),
+    # u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1))
     act: str = "relu2"
     bias: bool = False
     router: Optional[RouterSpec] = None
     shared_ff: int = 0              # > 0: a gated expert of this width that every token uses
+    limit: float = 0.0              # "clamped": of the routed experts, of the shared one
+    shared_limit: float = 0.0
+    # the shared expert's output is multiplied by the sigmoid of one projection of the input
+    shared_gate: bool = False
 
 
 @dataclasses.dataclass
@@ -392,6 +412,8 @@ class LayeredConfig(ModelConfig):
     # (hyper-connections) instead of one stream and a plain sum
     streams: int = 0
     logit_softcap: float = 0.0      # > 0: logits <- cap tanh(logits / cap)
+    # every pass of the loop begins with x <- W [x; embedding output]
+    loop_inject: bool = False
 
     def layer_runs(self) -> list:
         """Indices into layer_specs in execution order."""
@@ -413,7 +435,7 @@ class LayeredConfig(ModelConfig):
             elif isinstance(m, ParallelMixerSpec):
                 n += m.left.kv_heads * (m.left.dim + m.left.vdim) * es
             else:
-                n += m.kv_heads * (m.dim + m.vdim) * es
+                n += m.kv_heads * (m.key_dim + m.vdim) * es
                 if m.pool > 0:
                     n += -(-m.kv_heads * (m.dim + m.vdim) * 4 // m.pool)
         return n
@@ -424,6 +446,9 @@ class LayeredConfig(ModelConfig):
         if self.arch == "mudepel":
             return self.vocab_size * d + d + sum(_mudepel_layer_params(d, max(self.streams, 0), ls)
                                                  for ls in self.layer_specs)
+        if self.arch == "venanex":
+            return self.vocab_size * d + d + (2 * d * d if self.loop_inject else 0) + \
+                sum(_venanex_layer_params(d, ls) for ls in self.layer_specs)
         if self.arch == "papivik":
             return n + sum(_papivik_layer_params(d, ls) for ls in self.layer_specs)
         for ls in self.layer_specs:
@@ -495,6 +520,22 @@ def _papivik_layer_params(d: int, ls: "LayerSpec") -> int:
     n += d
     if ls.mlp is not None:
         n += d + 2 * d * ls.mlp.ff
+    return n
+
+
+def _venanex_layer_params(d: int, ls: "LayerSpec") -> int:
+    m = ls.mixer
+    if isinstance(m, LatentAttentionSpec):
+        n = m.q_rank * (d + 1) + m.heads * (m.dim + m.rot_dim) * m.q_rank + m.cache_dim * d \
+            + m.kv_rank + m.heads * (m.dim + m.vdim) * m.kv_rank + d * m.heads * m.vdim
+    else:
+        n = d * ((m.heads + m.kv_heads) * m.key_dim + m.kv_heads * m.vdim
+                 + 2 * m.heads * m.vdim) + 4 * m.dim
+    n += 2 * d
+    ml = ls.mlp
+    if ml is not None:
+        n += 2 * d + ml.router.experts * d * (1 + 3 * ml.ff) + 3 * d * ml.shared_ff \
+            + (d if ml.shared_gate else 0)
     return n
 
 
@@ -955,10 +996,126 @@ def papivik_dict(width: int, layers: list, vocab: int = 32000, eps: float = 1e-6
             "norm": {"eps": eps}, "vocab": vocab, "width": width}
 
 
+def _venanex_latent(m: dict) -> LatentAttentionSpec:
+    rot = m["rot"]
+    if int(rot["dims"]) != int(m["rot_dim"]) or int(m["rot_dim"]) % 2:
+        raise ValueError("Venanex: the rotated part is rotated whole (rot.dims == rot_dim, even)")
+    sc = rot.get("scaling") or None
+    if sc is not None and not all(k in sc for k in ("factor", "original", "fast", "slow")):
+        raise ValueError("Venanex: rot.scaling needs factor, original, fast and slow")
+    return LatentAttentionSpec(
+        heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+        kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), scale=float(m["scale"]),
+        rot=RotarySpec(int(rot["dims"]), float(rot["base"]), sc, layout="half"), gate="none")
+
+
+def _venanex_attention(m: dict) -> AttentionSpec:
+    if m.get("rot"):
+        raise ValueError("Venanex: the differential attention has no rotation")
+    spec = AttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]),
+                         vdim=int(m["vdim"]), scale=float(m["scale"]), rot=None,
+                         chunk=int((m.get("mask") or {}).get("size") or 0), sink=False,
+                         gate=True, gate_per="element", shared_kv=False, diff=float(m["diff"]))
+    if spec.heads % spec.kv_heads:
+        raise ValueError("Venanex: heads must be a multiple of kv_heads")
+    return spec
+
+
+def _venanex_mlp(ml: Optional[dict]) -> Optional[MlpSpec]:
+    if ml is None:
+        return None
+    if ml.get("kind") != "moe":
+        raise ValueError(f"Venanex: unknown feed-forward kind {ml.get('kind')!r}")
+    rt, sh = ml["router"], ml.get("shared")
+    router = RouterSpec(experts=int(rt["experts"]), top=int(rt["top"]), kind="sigmoid",
+                        weigh="input")
+    if not 1 <= router.top <= router.experts:
+        raise ValueError(f"Venanex: bad router {rt}")
+    spec = MlpSpec("moe", int(ml["expert"]["ff"]), act="clamped", router=router,
+                   limit=float(ml["expert"]["limit"]), shared_ff=int(sh["ff"]) if sh else 0,
+                   shared_limit=float(sh["limit"]) if sh else 0.0, shared_gate=bool(sh))
+    if spec.limit < 0 or spec.shared_limit < 0:
+        raise ValueError("Venanex: the experts' limit must not be negative")
+    return spec
+
+
+def venanex_config(name: str, d: dict, max_position: int = 1 << 20) -> LayeredConfig:
+    """A Venanex config.json: sequential layers with a layer norm (weight, no bias) before and
+    after each sublayer, mixers "latent_attention" (no output gate, rotate-half positions under
+    YaRN scaling on the shared key part) or "attention" (differential, chunked, without
+    positions, a sigmoid gate per output entry), routed feed-forwards of clamped gated experts
+    whose weights multiply the experts' inputs, beside a gated shared expert (or none), a loop
+    over a span of layers every pass of which mixes the embedding back in, tied embeddings."""
+    readers = {"latent_attention": _venanex_latent, "attention": _venanex_attention}
+    specs = []
+    for ly in d["layers"]:
+        if ly["type"] not in readers:
+            raise ValueError(f"Venanex: unknown mixer type {ly['type']!r}")
+        specs.append(LayerSpec(ly["type"], readers[ly["type"]](ly["mixer"]),
+                               _venanex_mlp(ly.get("mlp"))))
+    lp, loop = d.get("loop"), None
+    if lp:
+        loop = (int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not (0 <= loop[0] < loop[1] <= len(specs)) or loop[2] < 1:
+            raise ValueError(f"Venanex: bad loop {lp}")
+    att = [ls.mixer for ls in specs if isinstance(ls.mixer, AttentionSpec)]
+    lat = [ls.mixer for ls in specs if isinstance(ls.mixer, LatentAttentionSpec)]
+    cfg = LayeredConfig(
+        name=name, hf_id=name, arch="venanex", vocab_size=int(d["vocab"]),
+        hidden_size=int(d["width"]),
+        intermediate_size=max([ls.mlp.ff for ls in specs if ls.mlp is not None] or [0]),
+        num_layers=0, num_heads=max(ls.mixer.heads for ls in specs),
+        num_kv_heads=max([a.kv_heads for a in att] + [1]),
+        head_dim=max([max(a.key_dim, a.vdim) for a in att] + [m.cache_dim for m in lat]),
+        rms_eps=float(d["norm"]["eps"]), max_position=max_position, bos_id=0, eos_id=-1,
+        tie_embeddings=True, layer_specs=specs, loop=loop, loop_inject=loop is not None)
+    cfg.num_layers = len(cfg.layer_runs())
+    return cfg
+
+
+def venanex_dict(width: int, layers: list, vocab: int = 32000, eps: float = 1e-6,
+                 loop: Optional[tuple] = None) -> dict:
+    """A Venanex config.json dictionary from short layer dicts (random-init benchmarks and
+    tests).  A layer gives `latent` = (heads, dim, rot_dim, vdim, kv_rank, q_rank) with optional
+    base, yarn (a scaling dict), scale, or `att` = (heads, kv_heads, dim, vdim) with optional
+    chunk, diff, scale; and experts / expert_ff / top / limit with optional shared_ff /
+    shared_limit, or neither (no feed-forward).  loop = (start, stop, times)."""
+    out = []
+    for ly in layers:
+        if "latent" in ly:
+            h, dd, r, vv, R, Q = ly["latent"]
+            kind = "latent_attention"
+            m = {"heads": h, "dim": dd, "rot_dim": r, "vdim": vv, "kv_rank": R, "q_rank": Q,
+                 "rot": {"base": float(ly.get("base", 10000.0)), "dims": r,
+                         "scaling": ly.get("yarn")},
+                 "scale": float(ly.get("scale", (dd + r) ** -0.5))}
+        else:
+            h, g, dd, vv = ly["att"]
+            kind = "attention"
+            m = {"heads": h, "kv_heads": g, "dim": dd, "vdim": vv,
+                 "diff": float(ly.get("diff", 0.8)), "scale": float(ly.get("scale", dd ** -0.5))}
+            if ly.get("chunk"):
+                m["mask"] = {"size": int(ly["chunk"])}
+        mlp = None
+        if ly.get("experts"):
+            mlp = {"kind": "moe",
+                   "expert": {"ff": ly["expert_ff"], "limit": float(ly.get("limit", 7.0))},
+                   "router": {"experts": ly["experts"], "top": ly["top"]}}
+            if ly.get("shared_ff"):
+                mlp["shared"] = {"ff": ly["shared_ff"],
+                                 "limit": float(ly.get("shared_limit", 7.0))}
+        out.append({"type": kind, "mixer": m, "mlp": mlp})
+    d = {"architecture": "Venanex", "layers": out, "norm": {"eps": eps}, "vocab": vocab,
+         "width": width}
+    if loop:
+        d["loop"] = {"start": loop[0], "stop": loop[1], "times": loop[2]}
+    return d
+
+
 # config.json readers of designs that do not use the HF key set, by their "architecture" value
 _NATIVE_READERS = {"Bidetar": bidetar_config, "Puputar": puputar_config,
                    "Sazepel": sazepel_config, "Mudepel": mudepel_config,
-                   "Papivik": papivik_config}
+                   "Papivik": papivik_config, "Venanex": venanex_config}
 
 _REGISTRY: dict[str, ModelConfig] = {}
 
@@ -1256,6 +1413,43 @@ TINY_PAPIVIK = register(_papivik_stack(
     "tiny-papivik", width=128, n=5, att=(4, 2, 32, 16), delta=(4, 2, 16, 32), mlstm=(2, 16, 24),
     lightning=(3, 16, 32), ff=192, vocab=512, rot_dims=16, scales=(1.2, 0.8), conv=(3, 4),
     embed_scale=0.5))
+
+
+def _venanex_stack(name: str, width: int, n: int, latent: tuple, att: tuple, experts: int,
+                   expert_ff: int, top: int, shared_ff: int, chunk: int, loop: tuple,
+                   vocab: int = 32000, yarn: Optional[dict] = None, limit: float = 7.0
+                   ) -> LayeredConfig:
+    """n layers alternating latent attention and chunked differential attention, all with a
+    routed feed-forward and a shared expert except the last."""
+    layers = []
+    for i in range(n):
+        ly = dict(att=att, chunk=chunk, diff=0.8 - 0.6 * math.exp(-0.3 * i)) if i % 2 else \
+            dict(latent=latent, base=500000.0, yarn=yarn)
+        if i + 1 < n:
+            ly.update(experts=experts, expert_ff=expert_ff, top=top, shared_ff=shared_ff,
+                      limit=limit, shared_limit=1.5 * limit)
+        layers.append(ly)
+    cfg = venanex_config(name, venanex_dict(width, layers, vocab=vocab, loop=loop))
+    cfg.hf_id = "test/" + name
+    return cfg
+
+
+# Venanex at layer sizes of real models (random weights; bench.py --compare-design venanex):
+# 16 latent heads of 128 + 64 over a 512 + 64 cache, 16 / 4 differential heads of 2 x 64 over
+# 128-entry values, 8 experts of which 2 per token beside a shared one; the middle half of the
+# stack runs twice
+VENANEX_W2048 = register(_venanex_stack(
+    "venanex-w2048", width=2048, n=12, latent=(16, 128, 64, 128, 512, 768),
+    att=(16, 4, 64, 128), experts=8, expert_ff=1408, top=2, shared_ff=1408, chunk=8192,
+    loop=(4, 8, 2), yarn=_YARN))
+VENANEX_W4096 = register(_venanex_stack(
+    "venanex-w4096", width=4096, n=6, latent=(32, 128, 64, 128, 512, 1536),
+    att=(32, 8, 64, 128), experts=8, expert_ff=3584, top=2, shared_ff=3584, chunk=8192,
+    loop=(2, 4, 2), yarn=_YARN))
+TINY_VENANEX = register(_venanex_stack(
+    "tiny-venanex", width=128, n=4, latent=(4, 16, 8, 24, 40, 48), att=(4, 2, 16, 32), experts=6,
+    expert_ff=64, top=2, shared_ff=48, chunk=40, vocab=512, loop=(1, 3, 2), limit=1.5,
+    yarn={"factor": 2.0, "original": 64, "fast": 8.0, "slow": 1.0}))
 
 
 def get_config(name: str) -> ModelConfig:

@@ -27,7 +27,6 @@ residual update, the deferred biases and both norms of the next layer are one ke
 from __future__ import annotations
 
 import dataclasses
-import math
 from typing import Optional
 
 import torch
@@ -37,6 +36,7 @@ from .. import ops
 from ..ops import stream as sops
 from ..parallel.state import ParallelState, get_state
 from .config import LatentAttentionSpec, LayeredConfig, LayerSpec
+from .latent import LatentPaths
 from .routed import MOE_DENSE_ROWS, routed_sorted
 from .transformer import AttnBatch
 
@@ -64,11 +64,13 @@ class LatentLayerWeights:
     b_up: Optional[torch.Tensor] = None
     act: Optional[torch.Tensor] = None      # fp32 [2]
     w_down: Optional[torch.Tensor] = None   # routed [d, E F] (experts side by side)
+    w_uk_t: Optional[torch.Tensor] = None   # [H, D, R], [H, R, V]: w_uk and w_uv with the two last
+    w_uv_t: Optional[torch.Tensor] = None   # sizes exchanged (derived; the library's batched GEMM)
     router: Optional[torch.Tensor] = None   # fp32 [n, d]
     correction: Optional[torch.Tensor] = None
 
 
-class PuputarLM:
+class PuputarLM(LatentPaths):
     """Weights + forward of one replica (same surface as DecoderLM for the model runner)."""
 
     supports_v_tail = False
@@ -103,8 +105,6 @@ class PuputarLM:
         self.vocab_start, self.vocab_end = 0, cfg.vocab_size
         self._tables: dict = {}
         self.state: Optional[torch.Tensor] = None
-        self._ws: Optional[tuple] = None
-        self._ws_kept: list = []
         self._seg_map: dict = {}
         self._init_weights(seed)
 
@@ -170,6 +170,7 @@ class PuputarLM:
             self.layers.append(lw)
         self.final_norm = rand(d, s=0.1, mean=1.0, dt=f32)
         self.lm_head = rand(cfg.vocab_size, d)
+        self._derive_latent()
 
     def _names(self, i: int, lw: LatentLayerWeights):
         """(checkpoint name, destination view, transform of the checkpoint tensor) of layer i."""
@@ -243,6 +244,7 @@ class PuputarLM:
                 raise ValueError(f"{name}: checkpoint shape {tuple(sd[name].shape)} does not fit "
                                  f"the config (wanted {tuple(dst.shape)} after layout)")
             dst.copy_(src.to(dst.dtype))
+        self._derive_latent()
 
     @property
     def graph_safe(self) -> bool:
@@ -252,7 +254,8 @@ class PuputarLM:
         seen = [self.embed, self.embed_norm, self.final_norm, self.lm_head]
         for lw in self.layers:
             seen += [getattr(lw, f.name) for f in dataclasses.fields(lw)
-                     if f.name != "cos_sin" and isinstance(getattr(lw, f.name), torch.Tensor)]
+                     if f.name not in ("cos_sin", "w_uk_t", "w_uv_t")
+                     and isinstance(getattr(lw, f.name), torch.Tensor)]
         return sum(t.numel() * t.element_size() for t in seen)
 
     # ------------------------------------------------------------------ cache and state
@@ -260,14 +263,6 @@ class PuputarLM:
         """(q rows per token, rows per tile, rows per tile of short steps) of the scheduler's
         prefill tile map (the latent attention kernel takes its grid from the token rows)."""
         return 1, 128, 0
-
-    def _grouped(self, m: LatentAttentionSpec, block_size: int) -> bool:
-        """Does the layer keep the grouped second copy of its latents (the operand layout of
-        the matrix-core attention kernels: bf16 on the GPU, sizes they are built for)?"""
-        if self.device.type != "cuda" or self.dtype != torch.bfloat16 or block_size % 32:
-            return False
-        sops.load_native(required=True)
-        return bool(torch.ops.akap_stream.latent_mfma_supported(m.kv_rank, m.rot_dim))
 
     def kv_block_bytes(self, block_size: int, kv_dtype: str = "auto") -> int:
         es = torch.empty(0, dtype=self.dtype).element_size()
@@ -325,57 +320,6 @@ class PuputarLM:
         if self.dtype == torch.bfloat16:
             return ops.linear(x, w)
         return F.linear(x, w)
-
-    def _decode_parts(self, rows: int, heads: int) -> int:
-        """Key partitions of a decode row: static in the batch size and the model length
-        (hipGraph-capturable).  One workgroup per (row, 32 heads, partition); about one
-        workgroup per CU measured best (64 rows x 2112 keys, 16 heads, latent 512 + 64: 138 us
-        unsplit, 64 us at 4 partitions, 80 at 8, 87 at 16), a partition never under 128 keys."""
-        max_parts = max(1, math.ceil(self.max_model_len / 128))
-        groups = max(1, rows * math.ceil(heads / 32))
-        return min(max_parts, 64, max(1, math.ceil(256 / groups)))
-
-    def _workspace(self, rows: int, heads: int, kv_rank: int, parts: int):
-        """Partial softmax state of the split decode: (max, sum) per (row, head, partition) and
-        the unnormalised latent output.  Layers differ in heads and latent size, so both
-        buffers are checked; a buffer that has to grow (eager steps only: the runner warms a
-        bucket before capturing it) is kept alive, since captured graphs may still point at
-        it."""
-        n_ml, n_o = 2 * rows * heads * parts, rows * heads * parts * kv_rank
-        if self._ws is None or self._ws[0].numel() < n_ml or self._ws[1].numel() < n_o:
-            if self._ws is not None:
-                self._ws_kept.append(self._ws)
-                n_ml, n_o = max(n_ml, self._ws[0].numel()), max(n_o, self._ws[1].numel())
-            self._ws = (torch.empty(n_ml, dtype=torch.float32, device=self.device),
-                        torch.empty(n_o, dtype=torch.float32, device=self.device))
-        return self._ws
-
-    def _attention(self, m: LatentAttentionSpec, o_lat, q_lat, q, batch: AttnBatch, cache,
-                   groups) -> None:
-        T = q.shape[0]
-        nd = batch.num_decode if batch.is_prefill else T
-        if nd:
-            parts, ws = 1, None
-            if groups is not None:
-                parts = self._decode_parts(nd, m.heads)
-                ws = self._workspace(nd, m.heads, m.kv_rank, parts) if parts > 1 else None
-            # the leading nd rows are contiguous slices of the head-major buffers only when
-            # they are all rows; a mixed step's decode rows go through narrow copies
-            if nd == T:
-                sops.latent_attention_decode(o_lat, q_lat, q, m.dim, cache, groups,
-                                             batch.block_tables[:nd], batch.seq_lens[:nd],
-                                             batch.positions[:nd], m.scale, ws, parts)
-            else:
-                od = torch.empty(m.heads, nd, m.kv_rank, dtype=o_lat.dtype, device=o_lat.device)
-                sops.latent_attention_decode(od, q_lat[:, :nd].contiguous(), q[:nd], m.dim, cache,
-                                             groups, batch.block_tables[:nd], batch.seq_lens[:nd],
-                                             batch.positions[:nd], m.scale, ws, parts)
-                o_lat[:, :nd] = od
-        if batch.is_prefill:
-            sops.latent_attention_prefill(o_lat, q_lat, q, m.dim, cache, groups,
-                                          batch.block_tables, batch.seq_lens, batch.q_start,
-                                          batch.positions, batch.tile_seq, batch.tile_row,
-                                          batch.tile_rows, m.scale, first_seq=nd)
 
     def _routed(self, lw: LatentLayerWeights, h2: torch.Tensor, small: bool) -> torch.Tensor:
         """The routed feed-forward of h2 [T, d] as fp32 [T, d]."""
@@ -439,10 +383,11 @@ class PuputarLM:
                              0, lw.kv_off, eps, v_caches[r] if lw.kv_off >= 0 else None)
             q = self._linear(cq, lw.w_uq).view(T, H, D + rd)
             sops.rotate_heads_(q, batch.positions, lw.cos_sin, D)
-            q_lat = sops.head_matmul(q[:, :, :D].transpose(0, 1), lw.w_uk)    # [H, T, R]
+            q_lat = sops.head_matmul(q[:, :, :D].transpose(0, 1), lw.w_uk,     # [H, T, R]
+                                     lw.w_uk_t)
             o_lat = torch.empty(H, T, R, dtype=dt, device=dev)
-            self._attention(m, o_lat, q_lat, q, batch, k_caches[r], v_caches[r])
-            o = sops.head_matmul(o_lat, lw.w_uv)                               # [H, T, V]
+            self._latent_attention(m, o_lat, q_lat, q, batch, k_caches[r], v_caches[r])
+            o = sops.head_matmul(o_lat, lw.w_uv, lw.w_uv_t)                    # [H, T, V]
             cat = torch.empty(T, lw.hv + lw.ff, dtype=dt, device=dev)
             sops.head_gate(o, proj[:, lw.g_off:lw.g_off + m.gate_rows], cat[:, :lw.hv])
             ml = lw.spec.mlp

@@ -20,12 +20,13 @@ MOE_DENSE_ROWS = 256
 
 
 def routed_sorted(h2: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, experts: int,
-                  outputs: int, expert_fn: Callable[[int, torch.Tensor], torch.Tensor]
-                  ) -> torch.Tensor:
+                  outputs: int, expert_fn: Callable[[int, torch.Tensor], torch.Tensor],
+                  weigh: str = "output") -> torch.Tensor:
     """The routed feed-forward of h2 [T, d] by expert-sorted rows, as fp32 [T, d].  ids / w
     [T, top]: chosen outputs and their weights; outputs >= experts are identity outputs (they
     return their input and run no expert).  expert_fn(e, rows) is expert e applied to its rows
-    [c, d] -> [c, d]."""
+    [c, d] -> [c, d].  weigh "input": a weight multiplies the row an expert reads instead of the
+    one it returns."""
     T, d = h2.shape
     top = ids.shape[1]
     flat = ids.reshape(-1).long()
@@ -35,6 +36,9 @@ def routed_sorted(h2: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, experts:
     inv[order] = torch.arange(T * top, dtype=torch.int32, device=h2.device)
     n_real = sum(counts)
     xs = h2.index_select(0, order[:n_real] // top)
+    if weigh == "input":
+        xs = (xs.float() * w.reshape(-1)[order[:n_real], None]).to(h2.dtype)
+        w = torch.ones_like(w)
     ys = torch.empty(max(1, n_real), d, dtype=h2.dtype, device=h2.device)
     a = 0
     for e, c in enumerate(counts):

@@ -387,7 +387,7 @@ def latent_prep(proj: torch.Tensor, cq_out: torch.Tensor, cache: Optional[torch.
                 positions: torch.Tensor, slots: torch.Tensor, cos_sin: torch.Tensor,
                 q_w: torch.Tensor, kv_w: Optional[torch.Tensor], q_rank: int, kv_rank: int,
                 rot_dim: int, q_off: int, kv_off: int, eps: float,
-                vgroups: Optional[torch.Tensor] = None) -> None:
+                vgroups: Optional[torch.Tensor] = None, half: bool = False) -> None:
     """Per token t of the fused down-projection proj [T, N]: the query latent
     proj[t, q_off : q_off + q_rank] is RMS-normalised (weights q_w, fp32) into cq_out
     [T, q_rank]; the key/value latent proj[t, kv_off : kv_off + kv_rank] is RMS-normalised
@@ -396,19 +396,20 @@ def latent_prep(proj: torch.Tensor, cq_out: torch.Tensor, cache: Optional[torch.
     cache [NB, BS, kv_rank + rot_dim] at slots[t] (-1: nothing).  cache None: the layer reads
     another layer's cache and projects no latent of its own.  vgroups
     [NB, BS / 8, kv_rank, 8]: the normed latent once more, in groups of 8 tokens
-    (dimension-major inside a group: the operand layout of the matrix-core attention)."""
+    (dimension-major inside a group: the operand layout of the matrix-core attention).  half:
+    the rotated entries pair up as (i, i + rot_dim / 2) instead of (2i, 2i + 1)."""
     if _native(proj):
         torch.ops.akap_stream.latent_prep(proj, cq_out, cache, positions, slots, cos_sin, q_w,
                                           kv_w, q_rank, kv_rank, rot_dim, q_off, kv_off,
-                                          float(eps), vgroups)
+                                          float(eps), vgroups, bool(half))
         return
     cq = _rms(proj[:, q_off:q_off + q_rank].float(), eps) * q_w.float()
     cq_out.copy_(cq.to(cq_out.dtype))
     if cache is None:
         return
     c = _rms(proj[:, kv_off:kv_off + kv_rank].float(), eps) * kv_w.float()
-    kr = _rotate_pairs(proj[:, kv_off + kv_rank:kv_off + kv_rank + rot_dim].float(),
-                       cos_sin[positions.long()])
+    kr, cs = proj[:, kv_off + kv_rank:kv_off + kv_rank + rot_dim].float(), cos_sin[positions.long()]
+    kr = rotate_half_(kr[:, None].clone(), cs)[:, 0] if half else _rotate_pairs(kr, cs)
     BS = cache.shape[1]
     ok = slots >= 0
     sl = slots[ok].long()
@@ -418,15 +419,17 @@ def latent_prep(proj: torch.Tensor, cq_out: torch.Tensor, cache: Optional[torch.
 
 
 def rotate_heads_(q: torch.Tensor, positions: torch.Tensor, cos_sin: torch.Tensor,
-                  offset: int) -> None:
+                  offset: int, half: bool = False) -> None:
     """In place: the cos_sin.shape[1] entries from `offset` of every head of q [T, H, n] are
-    rotated in interleaved pairs by the angle row of positions[t] (fp32 arithmetic)."""
+    rotated in interleaved pairs (half: in pairs of the first and the second half of them) by the
+    angle row of positions[t] (fp32 arithmetic)."""
     if _native(q):
-        torch.ops.akap_stream.rotate_heads(q, positions, cos_sin, int(offset))
+        torch.ops.akap_stream.rotate_heads(q, positions, cos_sin, int(offset), bool(half))
         return
     dims = cos_sin.shape[1]
-    part = q[:, :, offset:offset + dims].float()
-    q[:, :, offset:offset + dims] = _rotate_pairs(part, cos_sin[positions.long()]).to(q.dtype)
+    part, cs = q[:, :, offset:offset + dims].float(), cos_sin[positions.long()]
+    q[:, :, offset:offset + dims] = (rotate_half_(part.clone(), cs) if half
+                                     else _rotate_pairs(part, cs)).to(q.dtype)
 
 
 def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q: torch.Tensor, rot_off: int,
@@ -528,20 +531,26 @@ def latent_attention_decode(out: torch.Tensor, q_lat: torch.Tensor, q: torch.Ten
 HEAD_MATMUL_ROWS = 256
 
 
-def head_matmul(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+def head_matmul(a: torch.Tensor, w: torch.Tensor, wt: Optional[torch.Tensor] = None,
+                token_major: bool = False) -> torch.Tensor:
     """out[h] = a[h] @ w[h]^T for every head: a [H, T, K] (any head / row strides, unit stride in
     k: a view of [T, H, n] rows is fine), w [H, N, K].  A few rows of bf16 on the GPU (decode
-    steps) run a small matrix-core kernel; everything else the library's batched GEMM."""
+    steps) run a small matrix-core kernel; everything else the library's batched GEMM, which takes
+    the weights as wt [H, K, N] (contiguous; made from w on the spot when not given: the library's
+    bf16 batched product must not see a transposed view).  token_major: the result lies in memory
+    as [T, H, N] (returned as the [H, T, N] view of it)."""
     H, T, K = a.shape
     N = w.shape[1]
+    out = torch.empty((T, H, N) if token_major else (H, T, N), dtype=a.dtype, device=a.device)
+    if token_major:
+        out = out.transpose(0, 1)
     if (a.is_cuda and a.dtype == torch.bfloat16 and 0 < T <= HEAD_MATMUL_ROWS and K % 16 == 0
             and N % 32 == 0 and a.stride(2) == 1 and a.stride(0) % 8 == 0 and a.stride(1) % 8 == 0
             and a.data_ptr() % 16 == 0 and w.is_contiguous()):
         load_native(required=True)
-        out = torch.empty(H, T, N, dtype=a.dtype, device=a.device)
         torch.ops.akap_stream.head_matmul(out, a, w)
         return out
-    return torch.bmm(a, w.transpose(1, 2))
+    return torch.bmm(a, wt if wt is not None else w.transpose(1, 2).contiguous(), out=out)
 
 
 def head_gate(o: torch.Tensor, gate: torch.Tensor, out: torch.Tensor) -> None:
@@ -1543,21 +1552,26 @@ def gate_group_norm(out: torch.Tensor, y: torch.Tensor, gate: torch.Tensor, w: t
 
 # ----------------------------------------------------------------------------- sigmoid group routing
 def route_sigmoid(h: torch.Tensor, router: torch.Tensor, top: int, groups: int = 1,
-                  keep: int = 1, group_top: int = 2):
+                  keep: int = 1, group_top: int = 2, gates: int = 0):
     """Routing by sigmoid scores: s = sigmoid(router h) (fp32, from h's stored values); experts
     form `groups` equal groups of neighbours, a group scores the sum of its `group_top` largest
     s, only experts of the `keep` best groups can be chosen (ties: the lower index); the `top`
     largest s among them win (ties: the lower index) and weigh their experts as they are.
     Returns ids int32 [T, top] (by falling score) and weights fp32 [T, top].  router fp32
-    [E, d]."""
-    T, E = h.shape[0], router.shape[0]
+    [E, d].  gates > 0: the router has that many rows more, which are no experts; their sigmoids
+    are returned too, fp32 [T, gates]."""
+    T, E = h.shape[0], router.shape[0] - gates
     ids = torch.empty(T, top, dtype=torch.int32, device=h.device)
     w = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    gw = torch.empty(T, gates, dtype=torch.float32, device=h.device) if gates else None
     if _native(h):
         torch.ops.akap_stream.route_sigmoid(ids, w, h, router, int(groups), int(keep),
-                                            int(group_top))
-        return ids, w
+                                            int(group_top), gw)
+        return (ids, w, gw) if gates else (ids, w)
     s = torch.sigmoid(h.float() @ router.float().T)
+    if gates:
+        gw.copy_(s[:, E:])
+        s = s[:, :E].contiguous()
     choice = s.clone()
     per = E // groups
     if groups > 1:
@@ -1569,7 +1583,7 @@ def route_sigmoid(h: torch.Tensor, router: torch.Tensor, top: int, groups: int =
     idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
     ids.copy_(idx)
     w.copy_(s.gather(1, idx))
-    return ids, w
+    return (ids, w, gw) if gates else (ids, w)
 
 
 def gated_act(gu: torch.Tensor, out: torch.Tensor, act: str = "silu",
@@ -1597,3 +1611,161 @@ def gated_act(gu: torch.Tensor, out: torch.Tensor, act: str = "silu",
         full.scatter_(1, ids.long(), w)
         r = r * full[:, :, None]
     out.copy_(r.reshape(T, experts * F_).to(out.dtype))
+
+
+CLAMPED_ALPHA = 1.702
+
+
+def clamped_glu(gu: torch.Tensor, out: torch.Tensor, limit: float,
+                ids: Optional[torch.Tensor] = None, w: Optional[torch.Tensor] = None,
+                experts: int = 1, shared_ff: int = 0, shared_limit: float = 0.0,
+                shared_w: Optional[torch.Tensor] = None, alpha: float = CLAMPED_ALPHA) -> None:
+    """Clamped gated units, f(g, u; L) = g' sigmoid(alpha g') (u' + 1) with g' = min(g, L) and
+    u' = clamp(u, -L, L).  gu [T, E 2F (+ 2 Fs)] = per expert [gate | up], then the shared expert's;
+    out [T, E F (+ Fs)].  Routed experts: out[t, e F + i] = f(c g, c u; limit) with the routing
+    weight c = w_e(t) on the INPUT (the units are linear up to the clamps and have no biases, so
+    scaling both projections is scaling the expert's input) and 0 for experts not chosen; ids / w
+    None: one plain layer, c = 1.  Shared expert (the last shared_ff columns of out):
+    shared_w[t] f(g, u; shared_limit) (shared_w fp32 [T]; None: 1).  fp32 arithmetic; both tensors
+    may be column slices of wider rows."""
+    if _native(gu):
+        torch.ops.akap_stream.clamped_glu(out, gu, ids, w, int(experts), float(limit),
+                                          int(shared_ff), float(shared_limit), shared_w,
+                                          float(alpha))
+        return
+    T = gu.shape[0]
+    F_ = (out.shape[1] - shared_ff) // experts if experts else 0
+
+    def unit(g, u, lim):
+        g, u = torch.clamp(g, max=lim), torch.clamp(u, min=-lim, max=lim)
+        return g * torch.sigmoid(alpha * g) * (u + 1.0)
+
+    if F_:
+        g3 = gu[:, :experts * 2 * F_].float().reshape(T, experts, 2, F_)
+        if ids is not None:
+            c = torch.zeros(T, experts, dtype=torch.float32)
+            c.scatter_(1, ids.long(), w)
+            g3 = g3 * c[:, :, None, None]
+        r = unit(g3[:, :, 0], g3[:, :, 1], limit)
+        out[:, :experts * F_] = r.reshape(T, experts * F_).to(out.dtype)
+    if shared_ff:
+        s2 = gu[:, experts * 2 * F_:].float().reshape(T, 2, shared_ff)
+        r = unit(s2[:, 0], s2[:, 1], shared_limit)
+        if shared_w is not None:
+            r = r * shared_w.float().reshape(T, 1)
+        out[:, experts * F_:] = r.to(out.dtype)
+
+
+# ----------------------------------------------------------------------------- layer norms
+def _layer_norm(x: torch.Tensor, eps: float) -> torch.Tensor:
+    c = x - x.mean(dim=-1, keepdim=True)
+    return c / torch.sqrt(c.pow(2).mean(dim=-1, keepdim=True) + eps)
+
+
+def stream_layer_norm_step(x: torch.Tensor, ya: torch.Tensor, yb: Optional[torch.Tensor],
+                           post_w: Optional[torch.Tensor], next_w: Optional[torch.Tensor],
+                           eps: float, out: torch.Tensor, fresh: bool = False) -> None:
+    """stream_post_norm_add_norm with layer norms (weights, no biases): with m = ya (+ yb),
+    x <- x + ln(m) post_w (fresh: x is not read and counts as zero; post_w None: m itself);
+    out = ln(x) next_w (next_w None: x itself).  ln(v) = (v - mean(v)) / sqrt(mean((v -
+    mean(v))^2) + eps) over the row.  x fp32 [T, d] (updated in place); ya and yb [T, d] each in
+    the activation type or fp32; weights fp32 [d].  All arithmetic is fp32; out (may be a column
+    slice of wider rows) is rounded once."""
+    if _native(x):
+        torch.ops.akap_stream.layer_norm_step(out, x, ya, yb, post_w, next_w, float(eps),
+                                              bool(fresh))
+        return
+    m = ya.float() if yb is None else ya.float() + yb.float()
+    if post_w is not None:
+        m = _layer_norm(m, eps) * post_w.float()
+    x.copy_(m if fresh else x + m)
+    out.copy_((_layer_norm(x, eps) * next_w.float() if next_w is not None else x).to(out.dtype))
+
+
+# ----------------------------------------------------------------------------- differential attention
+def _diff_rows(out, q, k_cache, v_cache, bt_row, rows: slice, pos, kv_len: int, gate, lam: float,
+               diff: float, scale: float, chunk: int, eps: float, H: int) -> None:
+    G, BS, Dv = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    D = k_cache.shape[3] // 2
+    nb = -(-kv_len // BS)
+    blocks = bt_row[:nb].long()
+    K = k_cache[blocks].permute(1, 0, 2, 3).reshape(G, nb * BS, 2, D)[:, :kv_len].float()
+    V = v_tokens(v_cache[blocks]).permute(1, 0, 2, 3).reshape(G, nb * BS, Dv)[:, :kv_len].float()
+    i, j = pos[:, None], torch.arange(kv_len)[None, :]
+    ok = j <= i
+    if chunk > 0:
+        ok &= (i // chunk) == (j // chunk)
+    n = i.shape[0]
+    qf = q[rows].float().reshape(n, H, 2, D)
+    o = torch.empty(n, H, Dv)
+    for h in range(H):
+        g = h // (H // G)
+        a = [torch.softmax(((qf[:, h, m] @ K[g, :, m].T) * scale).masked_fill(~ok, float("-inf")),
+                           dim=-1) @ V[g] for m in (0, 1)]
+        o[:, h] = _rms(a[0] - lam * a[1], eps) * (1.0 - diff)
+    o = o.reshape(n, H * Dv)
+    if gate is not None:
+        o = o * torch.sigmoid(gate[rows].float())
+    out[rows] = o.to(out.dtype)
+
+
+def diff_mfma_ok(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, scale: float
+                 ) -> bool:
+    """The matrix-core kernels take bf16 on the GPU at the head sizes they are built for."""
+    if not (q.is_cuda and q.dtype == torch.bfloat16 and scale > 0):
+        return False
+    load_native(required=True)
+    return (torch.ops.akap_stream.diff_mfma_supported(k_cache.shape[3] // 2, v_cache.shape[3],
+                                                      k_cache.shape[2])
+            and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0)
+
+
+def diff_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
+                   v_cache: torch.Tensor, batch, gate: Optional[torch.Tensor], heads: int,
+                   lam: float, diff: float, scale: float, chunk: int, eps: float, max_len: int,
+                   workspace=None) -> None:
+    """Paged differential attention of the token rows of a step (batch: the runner's AttnBatch).
+    q [T, H 2 D]: per query head [map 1 | map 2] (may be a column slice of the projection); K
+    [NB, G, BS, 2 D] (a cached key is [map 1 | map 2]), V [NB, G, BS / 8, Dv, 8].  Each map is a
+    causal softmax over scale q.k of its own, restricted (chunk > 0) to keys of the query's chunk
+    floor(position / chunk); with their outputs a1, a2 over the same values,
+    o = a1 - lam a2, divided by its root mean square over the head's Dv entries (eps inside the
+    root), times 1 - diff, times sigmoid(gate) per entry (gate [T, H Dv] or None):
+    out[t, h Dv ...].  Query head h reads key/value head h // (H / G).  Scores, softmax, the
+    difference, its norm and the gate are fp32.  Decode rows on the matrix cores cut the visible
+    range into partitions merged by a second launch (workspace: callable (rows, parts) ->
+    decode_workspace buffers for 2 H heads of Dv)."""
+    T = q.shape[0]
+    nd = batch.num_decode if batch.is_prefill else T
+    if _native(q):
+        ns = torch.ops.akap_stream
+        args = (k_cache, v_cache, batch.block_tables, batch.seq_lens)
+        tail = (gate, heads, float(lam), float(diff), float(scale), int(chunk), float(eps))
+        if not diff_mfma_ok(q, k_cache, v_cache, scale):
+            ns.diff_attention(out, q, *args, batch.q_start if batch.is_prefill else None,
+                              batch.positions, *tail)
+            return
+        if nd:
+            parts = diff_attention_parts(nd, heads, k_cache.shape[1], chunk, max_len)
+            ws = workspace(nd, parts) if parts > 1 else (None, None)
+            ns.diff_attention_decode_mfma(out[:nd], q[:nd], k_cache, v_cache,
+                                          batch.block_tables[:nd], batch.seq_lens[:nd],
+                                          gate[:nd] if gate is not None else None, *tail[1:],
+                                          ws[0], ws[1], parts)
+        if batch.is_prefill:
+            ns.diff_attention_prefill_mfma(out, q, *args, batch.q_start, batch.tile_seq,
+                                           batch.tile_row, int(batch.tile_rows), *tail)
+        return
+    for b, (r0, r1) in enumerate(_row_sequences(T, batch.q_start if batch.is_prefill else None)):
+        if r1 > r0 and int(batch.seq_lens[b]) > 0:
+            _diff_rows(out, q, k_cache, v_cache, batch.block_tables[b], slice(r0, r1),
+                       batch.positions[r0:r1].long(), int(batch.seq_lens[b]), gate, lam, diff,
+                       scale, chunk, eps, heads)
+
+
+def diff_attention_parts(rows: int, heads: int, kv_heads: int, chunk: int, max_len: int) -> int:
+    """Key partitions of a decode row: static in the batch size, the model length and the mask
+    (hipGraph-capturable).  About four waves per CU, a partition never under DECODE_PART keys."""
+    span = min(max_len, chunk) if chunk > 0 else max_len
+    wgs = max(1, rows * kv_heads * -(-(heads // kv_heads) // 16))
+    return 1 if wgs >= 1024 else min(max(1, -(-span // DECODE_PART)), 64, -(-1024 // wgs))
