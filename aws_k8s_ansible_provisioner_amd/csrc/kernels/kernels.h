@@ -223,10 +223,15 @@ void launch_argmax(const void* logits, int ld, int V, int is_bf16, int64_t* out,
 // Grouped expert GEMM for MoE decode: 32|64-row x 128-col tiles, k-pipelined, optional
 // activation-row gather and SwiGLU epilogue over gate/up-interleaved weight rows.
 bool moe_dgemm_supported(int N, int K, int pf, int silu, int splitk);
+// w given (with gather and silu): the epilogue forms clamped units of the weighted inputs
+struct MoeClamp {
+  const float* w;        // [n_flat] routing weight of every (token, choice) pair, or null
+  float limit, alpha;
+};
 void launch_moe_dgemm(const void* A, const void* W, void* Y, const int32_t* sorted_ids,
                       const int32_t* tile_expert, int max_tiles, int n_flat, int topk, int N,
                       int K, int lda, int ldy, int gather, int silu, int pf, int bm, int splitk,
-                      float* partials, bool nt_weights, hipStream_t s);
+                      float* partials, bool nt_weights, const MoeClamp& clamp, hipStream_t s);
 // out[t] = sum_k w[t,k] * sum_z P[z, inv[t*K+k], :]  (split-K fp32 partials of the down GEMM)
 void launch_moe_combine_split(const float* P, const float* wts, const int32_t* inv, void* out,
                               int T, int topk, int d, int S, int rows, hipStream_t s);

@@ -16,7 +16,10 @@
 //            their outputs are never combined), else row(r) = r
 //   SILU     W = [gate; up] (N = 2F) read gate/up-interleaved in 16-row groups (dgemm.hip
 //            EPI_SILU): Y[r, f] = bf16(bf16(silu(g)) * u), Y is [rows, F] -- the SwiGLU of
-//            the expert FFN happens in the w13 GEMM's epilogue.
+//            the expert FFN happens in the w13 GEMM's epilogue.  SILU == 2: clamped units instead,
+//            g' sigmoid(alpha g') (u' + 1) with g' = min(c g, limit), u' = clamp(c u, -limit,
+//            limit), c the routing weight of the row's (token, choice) pair: a weight on the
+//            expert's input (W has no biases).
 #include "common.h"
 #include "kernels.h"
 
@@ -30,7 +33,7 @@ __device__ __forceinline__ int mswz(int row, int chunk) { return row * 8 + (chun
 // 32-row x (128/WN)-col sub-tile = 2 x JN 16x16 MFMA tiles.
 // SPLIT: K is split over gridDim.z; each slice writes fp32 partials P[z, row, col] (ldy = N)
 // that moe_combine_split_kernel sums while combining (no extra launch).
-template <int BM, bool GATHER, bool SILU, int PF, bool SPLIT, bool NTW = false>
+template <int BM, bool GATHER, int SILU, int PF, bool SPLIT, bool NTW = false>
 __global__ __launch_bounds__(256, 2) void moe_dgemm_kernel(const bf16* __restrict__ A,
                                                            const bf16* __restrict__ W,
                                                            bf16* __restrict__ Y,
@@ -38,7 +41,8 @@ __global__ __launch_bounds__(256, 2) void moe_dgemm_kernel(const bf16* __restric
                                                            const int32_t* __restrict__ sorted_ids,
                                                            const int32_t* __restrict__ tile_expert,
                                                            int n_flat, int topk, int N, int K,
-                                                           int lda, int ldy, int rows) {
+                                                           int lda, int ldy, int rows,
+                                                           const MoeClamp clamp) {
   constexpr int WM = BM / 32, WN = 4 / WM, WCOLS = MBN / WN, JN = WCOLS / 16;
   constexpr int AR = BM / 32;  // A rows staged per thread
   // one __shared__ object: [buf 2][A BM rows | W 128 rows][8 chunks] bf16x8
@@ -68,7 +72,7 @@ __global__ __launch_bounds__(256, 2) void moe_dgemm_kernel(const bf16* __restric
   for (int c = 0; c < 4; ++c) {
     const int v = n0 + s_r + 32 * c;  // virtual column
     int wrow = v < N ? v : 0;
-    if constexpr (SILU) wrow = v < N ? ((v >> 4) & 1) * (N >> 1) + (v >> 5) * 16 + (v & 15) : 0;
+    if constexpr (SILU != 0) wrow = v < N ? ((v >> 4) & 1) * (N >> 1) + (v >> 5) * 16 + (v & 15) : 0;
     wb[c] = W + ((size_t)e * N + wrow) * K;
   }
 
@@ -141,11 +145,23 @@ __global__ __launch_bounds__(256, 2) void moe_dgemm_kernel(const bf16* __restric
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = m0 + wm * 32 + i * 16 + fg * 4 + r;
-      if constexpr (SILU) {
+      if constexpr (SILU != 0) {
+        float c = 0.f;
+        if constexpr (SILU == 2) {
+          const int sid = sorted_ids[row];
+          c = sid >= 0 && sid < n_flat ? clamp.w[sid] : 0.f;
+        }
 #pragma unroll
         for (int jj = 0; jj < JN / 2; ++jj) {  // sub-tiles 2jj / 2jj+1 = gate / up
           const int vb = n0 + wn * WCOLS + 32 * jj;
           if (vb + 16 + fr < N) {
+            if constexpr (SILU == 2) {
+              const float g = fminf(c * acc[i][2 * jj][r], clamp.limit);
+              const float u = fminf(fmaxf(c * acc[i][2 * jj + 1][r], -clamp.limit), clamp.limit);
+              Y[(size_t)row * ldy + (vb >> 1) + fr] =
+                  f2bf(g / (1.f + __expf(-clamp.alpha * g)) * (u + 1.f));
+              continue;
+            }
             const float g = bf2f(f2bf(acc[i][2 * jj][r]));
             const float u = bf2f(f2bf(acc[i][2 * jj + 1][r]));
             const float sg = bf2f(f2bf(g / (1.f + __expf(-g))));
@@ -226,12 +242,12 @@ void launch_moe_combine_split(const float* P, const float* wts, const int32_t* i
                                                        rows);
 }
 
-template <int BM, bool G, bool S, bool SPL>
+template <int BM, bool G, int S, bool SPL>
 static void moe_dgemm_pf(dim3 grid, int pf, bool ntw, hipStream_t s, const bf16* A, const bf16* W, bf16* Y,
                          float* P, const int32_t* sid, const int32_t* te, int n_flat, int topk,
-                         int N, int K, int lda, int ldy, int rows) {
+                         int N, int K, int lda, int ldy, int rows, const MoeClamp& cl) {
 #define MOE_L(PFV, NT) moe_dgemm_kernel<BM, G, S, PFV, SPL, NT><<<grid, 256, 0, s>>>( \
-      A, W, Y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows)
+      A, W, Y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows, cl)
   switch (pf) {
     case 4: if (ntw) MOE_L(4, true); else MOE_L(4, false); break;
     case 2: if (ntw) MOE_L(2, true); else MOE_L(2, false); break;
@@ -243,26 +259,26 @@ static void moe_dgemm_pf(dim3 grid, int pf, bool ntw, hipStream_t s, const bf16*
 template <int BM>
 static void moe_dgemm_bm(dim3 grid, int gather, int silu, int pf, bool ntw, hipStream_t s, const bf16* a,
                          const bf16* w, bf16* y, float* P, const int32_t* sid, const int32_t* te,
-                         int n_flat, int topk, int N, int K, int lda, int ldy, int rows) {
+                         int n_flat, int topk, int N, int K, int lda, int ldy, int rows,
+                         const MoeClamp& cl) {
   const bool spl = grid.z > 1;
-  if (gather && silu)
-    moe_dgemm_pf<BM, true, true, false>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
-  else if (silu)
-    moe_dgemm_pf<BM, false, true, false>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
-  else if (gather && spl)
-    moe_dgemm_pf<BM, true, false, true>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
-  else if (gather)
-    moe_dgemm_pf<BM, true, false, false>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
-  else if (spl)
-    moe_dgemm_pf<BM, false, false, true>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
-  else
-    moe_dgemm_pf<BM, false, false, false>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, rows);
+#define MOE_P(G, S, SPL)                                                                        \
+  moe_dgemm_pf<BM, G, S, SPL>(grid, pf, ntw, s, a, w, y, P, sid, te, n_flat, topk, N, K, lda, ldy, \
+                              rows, cl)
+  if (gather && silu && cl.w) MOE_P(true, 2, false);
+  else if (gather && silu) MOE_P(true, 1, false);
+  else if (silu) MOE_P(false, 1, false);
+  else if (gather && spl) MOE_P(true, 0, true);
+  else if (gather) MOE_P(true, 0, false);
+  else if (spl) MOE_P(false, 0, true);
+  else MOE_P(false, 0, false);
+#undef MOE_P
 }
 
 void launch_moe_dgemm(const void* A, const void* W, void* Y, const int32_t* sorted_ids,
                       const int32_t* tile_expert, int max_tiles, int n_flat, int topk, int N,
                       int K, int lda, int ldy, int gather, int silu, int pf, int bm, int splitk,
-                      float* partials, bool ntw, hipStream_t s) {
+                      float* partials, bool ntw, const MoeClamp& cl, hipStream_t s) {
   if (max_tiles == 0) return;
   dim3 grid(max_tiles, (N + MBN - 1) / MBN, splitk);
   const bf16* a = (const bf16*)A;
@@ -270,9 +286,11 @@ void launch_moe_dgemm(const void* A, const void* W, void* Y, const int32_t* sort
   bf16* y = (bf16*)Y;
   const int rows = max_tiles * bm;
   if (bm == 64)
-    moe_dgemm_bm<64>(grid, gather, silu, pf, ntw, s, a, w, y, partials, sorted_ids, tile_expert, n_flat, topk, N, K, lda, ldy, rows);
+    moe_dgemm_bm<64>(grid, gather, silu, pf, ntw, s, a, w, y, partials, sorted_ids, tile_expert,
+                     n_flat, topk, N, K, lda, ldy, rows, cl);
   else
-    moe_dgemm_bm<32>(grid, gather, silu, pf, ntw, s, a, w, y, partials, sorted_ids, tile_expert, n_flat, topk, N, K, lda, ldy, rows);
+    moe_dgemm_bm<32>(grid, gather, silu, pf, ntw, s, a, w, y, partials, sorted_ids, tile_expert,
+                     n_flat, topk, N, K, lda, ldy, rows, cl);
 }
 
 }  // namespace akap

@@ -679,7 +679,7 @@ void moe_gemm(Tensor out, Tensor a, Tensor w, Tensor sorted_ids, Tensor tile_exp
 // [splitk, rows, N] consumed by moe_combine_split.
 void moe_dgemm(Tensor out, Tensor a, Tensor w, Tensor sorted_ids, Tensor tile_expert,
                int64_t n_flat, int64_t topk, bool gather, bool silu, int64_t pf, int64_t bm,
-               int64_t splitk) {
+               int64_t splitk, std::optional<Tensor> clamp_w, double limit, double alpha) {
   CHECK_GPU(a); CHECK_BF16(a); CHECK_BF16(w); CHECK_CONTIG(w); CHECK_CONTIG(out);
   CHECK_LAST_CONTIG(a);
   TORCH_CHECK(w.dim() == 3, "expert weights [E, N, K]");
@@ -712,13 +712,21 @@ void moe_dgemm(Tensor out, Tensor a, Tensor w, Tensor sorted_ids, Tensor tile_ex
     return e ? std::atoi(e) : -1;
   }();
   const bool ntw = nt_env >= 0 ? nt_env != 0 : (bm == 64 && n_flat <= 40 * w.size(0));
+  akap::MoeClamp clamp{nullptr, (float)limit, (float)alpha};
+  if (clamp_w.has_value()) {
+    CHECK_GPU(*clamp_w); CHECK_CONTIG(*clamp_w);
+    TORCH_CHECK(gather && silu && splitk == 1 && limit >= 0 &&
+                    clamp_w->scalar_type() == at::kFloat && clamp_w->numel() == n_flat,
+                "moe_dgemm: clamped units need gather, silu and one fp32 weight per pair");
+    clamp.w = clamp_w->data_ptr<float>();
+  }
   const c10::DeviceGuard g(a.device());
   akap::launch_moe_dgemm(a.data_ptr(), w.data_ptr(), splitk > 1 ? nullptr : out.data_ptr(),
                          sorted_ids.data_ptr<int32_t>(), tile_expert.data_ptr<int32_t>(),
                          max_tiles, n_flat, topk, N, K, a.stride(0),
                          splitk > 1 ? N : out.stride(0), gather ? 1 : 0, silu ? 1 : 0, (int)pf,
                          (int)bm, (int)splitk, splitk > 1 ? out.data_ptr<float>() : nullptr, ntw,
-                         cur_stream());
+                         clamp, cur_stream());
 }
 
 void moe_combine_split(Tensor partials, Tensor wts, Tensor inv, Tensor out, int64_t splitk,
@@ -1360,7 +1368,8 @@ TORCH_LIBRARY(akap, m) {
   m.def("moe_combine(Tensor y, Tensor wts, Tensor inv, Tensor(a!) out) -> ()");
   m.def(
       "moe_dgemm(Tensor(a!) out, Tensor a, Tensor w, Tensor sorted_ids, Tensor tile_expert, "
-      "int n_flat, int topk, bool gather, bool silu, int pf, int bm=32, int splitk=1) -> ()");
+      "int n_flat, int topk, bool gather, bool silu, int pf, int bm=32, int splitk=1, "
+      "Tensor? clamp_w=None, float limit=0, float alpha=0) -> ()");
   m.def(
       "moe_combine_split(Tensor partials, Tensor wts, Tensor inv, Tensor(a!) out, int splitk, "
       "int rows) -> ()");

@@ -240,7 +240,8 @@ __global__ __launch_bounds__(256) void route_sigmoid_kernel(int32_t* __restrict_
                                                             const T* __restrict__ h, int h_stride,
                                                             const float* __restrict__ router, int d,
                                                             int E, int top, int groups, int keep,
-                                                            int group_top) {
+                                                            int group_top, float* __restrict__ gw,
+                                                            int gates) {
   extern __shared__ __align__(16) float lds[];   // [d] row (padded to 4), [E] scores, [E] choice
   float* hs = lds;                               // values, [groups] group scores
   float* sc = lds + ((d + 3) & ~3);
@@ -250,7 +251,7 @@ __global__ __launch_bounds__(256) void route_sigmoid_kernel(int32_t* __restrict_
   const T* hr = h + (size_t)t * h_stride;
   for (int c = threadIdx.x; c < d; c += 256) hs[c] = ldf(hr + c);
   __syncthreads();
-  for (int e = wave; e < E; e += 4) {
+  for (int e = wave; e < E + gates; e += 4) {
     const float* r = router + (size_t)e * d;
     float acc = 0.f;
     if ((d & 3) == 0 && ((uintptr_t)router & 15) == 0) {
@@ -267,8 +268,12 @@ __global__ __launch_bounds__(256) void route_sigmoid_kernel(int32_t* __restrict_
     acc = wave_sum(acc);
     if (lane == 0) {
       const float s = 1.0f / (1.0f + expf(-acc));
-      sc[e] = s;
-      ch[e] = s;
+      if (e >= E) {
+        gw[(size_t)t * gates + e - E] = s;
+      } else {
+        sc[e] = s;
+        ch[e] = s;
+      }
     }
   }
   __syncthreads();
@@ -966,15 +971,17 @@ void launch_gate_group_norm(void* out, int out_stride, const float* y, const voi
 
 void launch_route_sigmoid(int32_t* ids, float* w, const void* h, int h_stride, bool f32,
                           const float* router, int rows, int d, int E, int top, int groups,
-                          int keep, int group_top, hipStream_t s) {
+                          int keep, int group_top, float* gate_w, int gates, hipStream_t s) {
   if (rows <= 0) return;
   const size_t lds = (size_t)(((d + 3) & ~3) + 2 * E + groups) * sizeof(float);
   if (f32)
     route_sigmoid_kernel<float><<<rows, 256, lds, s>>>(ids, w, (const float*)h, h_stride, router,
-                                                       d, E, top, groups, keep, group_top);
+                                                       d, E, top, groups, keep, group_top, gate_w,
+                                                       gates);
   else
     route_sigmoid_kernel<bf16><<<rows, 256, lds, s>>>(ids, w, (const bf16*)h, h_stride, router, d,
-                                                      E, top, groups, keep, group_top);
+                                                      E, top, groups, keep, group_top, gate_w,
+                                                      gates);
 }
 
 void launch_conv_silu(void* out, bool out_f32, const void* proj, int proj_stride, int off, bool f32,

@@ -100,13 +100,22 @@ void gate_group_norm(Tensor out, Tensor y, Tensor gate, Tensor w, int64_t groups
 }
 
 void route_sigmoid(Tensor ids, Tensor w, Tensor h, Tensor router, int64_t groups, int64_t keep,
-                   int64_t group_top) {
+                   int64_t group_top, std::optional<Tensor> gate_w) {
   CHECK_GPU(ids); CHECK_GPU(w); CHECK_GPU(h); CHECK_GPU(router);
   CHECK_I32(ids); CHECK_F32(w); CHECK_CONTIG(ids); CHECK_CONTIG(w); CHECK_LAST_CONTIG(h);
   CHECK_F32(router); CHECK_CONTIG(router);
   TORCH_CHECK(h.dim() == 2 && router.dim() == 2 && router.size(1) == h.size(1) && ids.dim() == 2 &&
                   ids.size(0) == h.size(0) && w.sizes() == ids.sizes(), "route_sigmoid: shapes");
-  const int64_t E = router.size(0), d = h.size(1), top = ids.size(1);
+  int64_t gates = 0;
+  float* gw = nullptr;
+  if (gate_w.has_value()) {
+    CHECK_GPU(*gate_w); CHECK_F32(*gate_w); CHECK_CONTIG(*gate_w);
+    TORCH_CHECK(gate_w->dim() == 2 && gate_w->size(0) == h.size(0) &&
+                    gate_w->size(1) < router.size(0), "route_sigmoid: gate_w [T, gates]");
+    gates = gate_w->size(1);
+    gw = gate_w->data_ptr<float>();
+  }
+  const int64_t E = router.size(0) - gates, d = h.size(1), top = ids.size(1);
   TORCH_CHECK(E >= 1 && E <= 2048 && d <= 12000, "route_sigmoid: at most 2048 experts, rows of at "
               "most 12000 entries");
   TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && group_top >= 1 &&
@@ -115,7 +124,7 @@ void route_sigmoid(Tensor ids, Tensor w, Tensor h, Tensor router, int64_t groups
   akap_stream::launch_route_sigmoid(ids.data_ptr<int32_t>(), w.data_ptr<float>(), h.data_ptr(),
                                     (int)h.stride(0), is_f32(h, "h"), router.data_ptr<float>(),
                                     (int)h.size(0), (int)d, (int)E, (int)top, (int)groups,
-                                    (int)keep, (int)group_top, cur_stream());
+                                    (int)keep, (int)group_top, gw, (int)gates, cur_stream());
 }
 
 // rows, sequences and the checks shared by the ops that walk sequences of a step
@@ -396,7 +405,7 @@ TORCH_LIBRARY_FRAGMENT(akap_stream, m) {
   m.def("gate_group_norm(Tensor(a!) out, Tensor y, Tensor gate, Tensor w, int groups, float eps) "
         "-> ()");
   m.def("route_sigmoid(Tensor(a!) ids, Tensor(b!) w, Tensor h, Tensor router, int groups, "
-        "int keep, int group_top) -> ()");
+        "int keep, int group_top, Tensor(c!)? gate_w=None) -> ()");
   m.def("conv_silu(Tensor(a!) out, Tensor proj, int off, Tensor conv_w, Tensor? conv_b, "
         "Tensor(b!) state, Tensor seq_slot, Tensor positions, Tensor? q_start, "
         "int silu_from=0) -> ()");

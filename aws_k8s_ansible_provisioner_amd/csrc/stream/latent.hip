@@ -189,10 +189,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrepParams p) {
   const int half = p.rot_dim / 2;
   const T* kr = kv + p.kv_rank;
   for (int i = threadIdx.x; i < half; i += 256) {
-    const float u = ldf(kr + 2 * i), v = ldf(kr + 2 * i + 1);
+    const int a = p.half_pairs ? i : 2 * i, b = p.half_pairs ? i + half : 2 * i + 1;
+    const float u = ldf(kr + a), v = ldf(kr + b);
     const float c = cs[i], s = cs[half + i];
-    stf(dst + p.kv_rank + 2 * i, u * c - v * s);
-    stf(dst + p.kv_rank + 2 * i + 1, v * c + u * s);
+    stf(dst + p.kv_rank + a, u * c - v * s);
+    stf(dst + p.kv_rank + b, v * c + u * s);
   }
 }
 
@@ -201,7 +202,7 @@ __global__ __launch_bounds__(256) void rotate_heads_kernel(T* __restrict__ q, in
                                                            int n, int offset, int dims,
                                                            const int64_t* __restrict__ positions,
                                                            const float* __restrict__ cos_sin,
-                                                           int max_pos) {
+                                                           int max_pos, int half_pairs) {
   const int t = blockIdx.x;
   int64_t pos = positions[t];
   pos = pos < 0 ? 0 : (pos >= max_pos ? max_pos - 1 : pos);
@@ -210,11 +211,12 @@ __global__ __launch_bounds__(256) void rotate_heads_kernel(T* __restrict__ q, in
   T* row = q + (size_t)t * q_stride;
   for (int i = threadIdx.x; i < H * half; i += 256) {
     const int h = i / half, j = i % half;
-    T* e = row + (size_t)h * n + offset + 2 * j;
-    const float u = ldf(e), v = ldf(e + 1);
+    T* a = row + (size_t)h * n + offset + (half_pairs ? j : 2 * j);
+    T* b = a + (half_pairs ? half : 1);
+    const float u = ldf(a), v = ldf(b);
     const float c = cs[j], s = cs[half + j];
-    stf(e, u * c - v * s);
-    stf(e + 1, v * c + u * s);
+    stf(a, u * c - v * s);
+    stf(b, v * c + u * s);
   }
 }
 
@@ -762,14 +764,14 @@ void launch_latent_prep(const LatentPrepParams& p, bool f32, hipStream_t s) {
 
 void launch_rotate_heads(void* q, int q_stride, int T, int H, int n, int offset, int dims,
                          const int64_t* positions, const float* cos_sin, int max_pos, bool f32,
-                         hipStream_t s) {
+                         bool half_pairs, hipStream_t s) {
   if (T <= 0) return;
   if (f32)
     rotate_heads_kernel<float><<<T, 256, 0, s>>>((float*)q, q_stride, H, n, offset, dims,
-                                                 positions, cos_sin, max_pos);
+                                                 positions, cos_sin, max_pos, half_pairs);
   else
     rotate_heads_kernel<bf16><<<T, 256, 0, s>>>((bf16*)q, q_stride, H, n, offset, dims, positions,
-                                                cos_sin, max_pos);
+                                                cos_sin, max_pos, half_pairs);
 }
 
 template <typename T>

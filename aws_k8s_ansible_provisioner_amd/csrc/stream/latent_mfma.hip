@@ -642,10 +642,11 @@ void launch_decode(const LatentAttnParams& p, hipStream_t s) {
 // 32 x 32 tile of one head, both operands contiguous in k (16-byte fragment loads), k in
 // batches of 8 MFMA steps whose loads go out together.  The library's batched GEMM takes
 // 12-14 us for these 0.1 GFLOP products at 64 rows.
-__global__ __launch_bounds__(64) void head_matmul_kernel(bf16* __restrict__ out,
-                                                         const bf16* __restrict__ a, int64_t a_hs,
-                                                         int64_t a_ts, const bf16* __restrict__ w,
-                                                         int T, int N, int K) {
+__global__ __launch_bounds__(64) void head_matmul_kernel(bf16* __restrict__ out, int64_t o_hs,
+                                                         int64_t o_ts, const bf16* __restrict__ a,
+                                                         int64_t a_hs, int64_t a_ts,
+                                                         const bf16* __restrict__ w, int T, int N,
+                                                         int K) {
   const int lane = threadIdx.x;
   const int col = lane & 31, hf = lane >> 5;
   const int ntn = N / 32;
@@ -672,18 +673,18 @@ __global__ __launch_bounds__(64) void head_matmul_kernel(bf16* __restrict__ out,
 #pragma unroll
   for (int i = 0; i < 16; ++i) {
     const int r = mt * 32 + 8 * (i >> 2) + 4 * hf + (i & 3);
-    if (r < T) out[((size_t)h * T + r) * N + nt * 32 + col] = (bf16)acc[i];
+    if (r < T) out[(size_t)h * o_hs + (size_t)r * o_ts + nt * 32 + col] = (bf16)acc[i];
   }
 }
 
 }  // namespace
 
-void launch_head_matmul(void* out, const void* a, int64_t a_hs, int64_t a_ts, const void* w, int H,
-                        int T, int N, int K, hipStream_t s) {
+void launch_head_matmul(void* out, int64_t o_hs, int64_t o_ts, const void* a, int64_t a_hs,
+                        int64_t a_ts, const void* w, int H, int T, int N, int K, hipStream_t s) {
   if (H <= 0 || T <= 0) return;
   const dim3 grid((N / 32) * ((T + 31) / 32), H);
-  head_matmul_kernel<<<grid, 64, 0, s>>>((bf16*)out, (const bf16*)a, a_hs, a_ts, (const bf16*)w, T,
-                                         N, K);
+  head_matmul_kernel<<<grid, 64, 0, s>>>((bf16*)out, o_hs, o_ts, (const bf16*)a, a_hs, a_ts,
+                                         (const bf16*)w, T, N, K);
 }
 
 // the latent / rotated sizes the matrix kernels are built for

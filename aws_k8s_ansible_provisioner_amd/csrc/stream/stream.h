@@ -106,12 +106,14 @@ struct LatentPrepParams {
   int T, q_rank, kv_rank, rot_dim, q_off, kv_off;
   int64_t num_slots;
   float eps;
+  int half_pairs;        // rotated pairs (i, i + rot_dim / 2) instead of (2i, 2i + 1)
 };
 void launch_latent_prep(const LatentPrepParams& p, bool f32, hipStream_t s);
-// in place: `dims` entries from `offset` of each of the H heads (n entries per head) of a row
+// in place: `dims` entries from `offset` of each of the H heads (n entries per head) of a row; pairs
+// (2i, 2i + 1), or (i, i + dims / 2) with half_pairs
 void launch_rotate_heads(void* q, int q_stride, int T, int H, int n, int offset, int dims,
                          const int64_t* positions, const float* cos_sin, int max_pos, bool f32,
-                         hipStream_t s);
+                         bool half_pairs, hipStream_t s);
 
 struct LatentAttnParams {
   void* out;            // [H, T, R]
@@ -143,10 +145,11 @@ bool latent_mfma_sizes(int R, int r);
 void launch_latent_prefill_mfma(const LatentAttnParams& p, hipStream_t s);
 void launch_latent_decode_mfma(const LatentAttnParams& p, hipStream_t s);
 
-// out [H, T, N] = a [H, T, K] (strides a_hs / a_ts, unit in k) x w [H, N, K]^T, bf16, K % 16 == 0,
-// N % 32 == 0, 16-byte aligned rows; meant for a few rows (one wave per 32 x 32 tile)
-void launch_head_matmul(void* out, const void* a, int64_t a_hs, int64_t a_ts, const void* w, int H,
-                        int T, int N, int K, hipStream_t s);
+// out [H, T, N] (strides o_hs / o_ts) = a [H, T, K] (strides a_hs / a_ts, unit in k) x
+// w [H, N, K]^T, bf16, K % 16 == 0, N % 32 == 0, 16-byte aligned rows; meant for a few rows (one
+// wave per 32 x 32 tile)
+void launch_head_matmul(void* out, int64_t o_hs, int64_t o_ts, const void* a, int64_t a_hs,
+                        int64_t a_ts, const void* w, int H, int T, int N, int K, hipStream_t s);
 void launch_head_gate(void* out, int out_stride, const void* o, const void* gate, int gate_stride,
                       bool per_head, int rows, int H, int V, bool f32, hipStream_t s);
 void launch_xielu(void* out, int out_stride, const void* x, int x_stride, const void* bias,
@@ -275,9 +278,11 @@ void launch_softcap(void* x, bool f32, size_t n, float cap, hipStream_t s);
 void launch_gate_group_norm(void* out, int out_stride, const float* y, const void* gate,
                             int gate_stride, const float* w, bool f32, int rows, int n,
                             int groups, float eps, hipStream_t s);
+// gates > 0: the router has that many rows after the E experts', whose sigmoids go to gate_w
+// [rows, gates]
 void launch_route_sigmoid(int32_t* ids, float* w, const void* h, int h_stride, bool f32,
                           const float* router, int rows, int d, int E, int top, int groups,
-                          int keep, int group_top, hipStream_t s);
+                          int keep, int group_top, float* gate_w, int gates, hipStream_t s);
 // causal per-channel convolution of columns [off, off + C) of proj (b null: no bias; silu on the
 // channels from silu_from on), then the sequences' last taps - 1 inputs to their slots; out fp32
 // or proj's type; B sequences (q_start null: B = T, one row each)
@@ -415,5 +420,69 @@ void launch_pooled_window_prefill_mfma(const PoolAttnParams& p, const int32_t* t
 // query heads of a key/value head are the columns of a tile, the key range is split over the
 // workgroup's waves
 void launch_pooled_window_decode_mfma(const PoolAttnParams& p, int rows, hipStream_t s);
+
+// ---- layer norms, clamped gated units, differential attention (diff.hip, diff_mfma.hip) --------
+// m = ya + yb; x (fp32 rows of d) <- x + ln(m) post_w (fresh: x is not read; post_w null: m itself);
+// out = ln(x) next_w (next_w null: out = x), ln over the row with the mean taken off
+struct LayerNormStepParams {
+  void* out;
+  int out_stride;
+  float* x;
+  const void* ya;        // rows of bf16 or fp32
+  int ya_stride, ya_f32;
+  const void* yb;        // or null
+  int yb_stride, yb_f32;
+  const float* post_w;   // [d] or null
+  const float* next_w;
+  int rows, d, fresh;
+  float eps;
+};
+void launch_layer_norm_step(const LayerNormStepParams& p, bool out_f32, hipStream_t s);
+
+// out [rows, E F + Fs] from gu [rows, E 2F + 2 Fs] (per expert [gate | up], then the shared one):
+// g' sigmoid(alpha g') (u' + 1), g' = min(c g, limit), u' = clamp(c u, -limit, limit), c the routing
+// weight (0: not chosen; ids null: 1); the shared one times shared_w (null: 1)
+struct ClampedGluParams {
+  void* out;
+  int out_stride;
+  const void* gu;
+  int gu_stride;
+  const int32_t* ids;    // [rows, top] or null
+  const float* w;
+  const float* shared_w; // [rows] or null
+  int rows, top, E, F, Fs;
+  float limit, shared_limit, alpha;
+};
+void launch_clamped_glu(const ClampedGluParams& p, bool f32, hipStream_t s);
+
+struct DiffAttnParams {
+  void* out;             // rows of out_stride; head h at columns [h Dv, (h + 1) Dv)
+  int out_stride;
+  const void* q;         // rows of q_stride; head h at [h 2D, (h + 1) 2D): [map 1 | map 2]
+  int q_stride;
+  const void* k_cache;   // [NB, G, BS, 2 D]
+  const void* v_cache;   // [NB, G, BS / 8, Dv, 8]
+  const int32_t* block_tables;  // [B, max_blocks]
+  int max_blocks;
+  const int32_t* seq_lens;      // [B]
+  const int32_t* q_start;       // [B + 1] or null (row t is sequence t)
+  const int64_t* positions;     // [T] (row form)
+  const int32_t* tile_seq;      // prefill tile map (matrix-core form)
+  const int32_t* tile_row;
+  int num_tiles, tile_rows;
+  const void* gate;             // [T, H Dv] logits, or null
+  int gate_stride;
+  float lam, out_mult, scale, eps;   // out_mult: 1 - diff
+  int chunk, T, B, H, G, D, Dv, BS, NB;
+  // decode split: (max, sum) [B, H, 2, parts, 2] and unnormalised outputs [B, H, 2, parts, Dv]
+  float* ws_ml;
+  float* ws_o;
+  int num_parts;
+};
+void launch_diff_attention(const DiffAttnParams& p, bool f32, hipStream_t s);
+// bf16, sizes among the built ones, pages of a multiple of 32 keys
+bool diff_mfma_supported(int D, int Dv, int BS);
+void launch_diff_prefill_mfma(const DiffAttnParams& p, hipStream_t s);
+void launch_diff_decode_mfma(const DiffAttnParams& p, hipStream_t s);
 
 }  // namespace akap_stream

@@ -354,7 +354,7 @@ void token_shift(Tensor out, Tensor h, Tensor mu, Tensor state, Tensor seq_slot,
 void latent_prep(Tensor proj, Tensor cq_out, std::optional<Tensor> cache, Tensor positions,
                  Tensor slots, Tensor cos_sin, Tensor q_w, std::optional<Tensor> kv_w,
                  int64_t q_rank, int64_t kv_rank, int64_t rot_dim, int64_t q_off, int64_t kv_off,
-                 double eps, std::optional<Tensor> vgroups) {
+                 double eps, std::optional<Tensor> vgroups, bool half) {
   CHECK_GPU(proj); CHECK_LAST_CONTIG(proj); CHECK_GPU(cq_out); CHECK_CONTIG(cq_out);
   CHECK_GPU(positions); CHECK_GPU(slots); CHECK_CONTIG(positions); CHECK_CONTIG(slots);
   CHECK_GPU(cos_sin); CHECK_F32(cos_sin); CHECK_CONTIG(cos_sin);
@@ -379,6 +379,7 @@ void latent_prep(Tensor proj, Tensor cq_out, std::optional<Tensor> cache, Tensor
   p.T = T; p.q_rank = q_rank; p.kv_rank = kv_rank; p.rot_dim = rot_dim; p.q_off = q_off;
   p.kv_off = kv_off;
   p.eps = (float)eps;
+  p.half_pairs = half;
   if (cache.has_value()) {
     CHECK_GPU(*cache); CHECK_CONTIG(*cache);
     TORCH_CHECK(kv_w.has_value(), "latent_prep: a cache needs kv_w");
@@ -404,7 +405,7 @@ void latent_prep(Tensor proj, Tensor cq_out, std::optional<Tensor> cache, Tensor
   akap_stream::launch_latent_prep(p, f32, cur_stream());
 }
 
-void rotate_heads(Tensor q, Tensor positions, Tensor cos_sin, int64_t offset) {
+void rotate_heads(Tensor q, Tensor positions, Tensor cos_sin, int64_t offset, bool half) {
   CHECK_GPU(q); CHECK_GPU(positions); CHECK_GPU(cos_sin); CHECK_F32(cos_sin); CHECK_CONTIG(cos_sin);
   CHECK_CONTIG(positions);
   TORCH_CHECK(q.dim() == 3 && q.stride(2) == 1 && q.stride(1) == q.size(2), "q must be [T, H, n]");
@@ -416,7 +417,7 @@ void rotate_heads(Tensor q, Tensor positions, Tensor cos_sin, int64_t offset) {
   akap_stream::launch_rotate_heads(q.data_ptr(), (int)q.stride(0), (int)q.size(0), (int)q.size(1),
                                    (int)q.size(2), (int)offset, (int)dims,
                                    positions.data_ptr<int64_t>(), cos_sin.data_ptr<float>(),
-                                   (int)cos_sin.size(0), is_f32(q, "q"), cur_stream());
+                                   (int)cos_sin.size(0), is_f32(q, "q"), half, cur_stream());
 }
 
 void latent_attention(Tensor out, Tensor q_lat, Tensor q, int64_t rot_off, Tensor cache,
@@ -569,7 +570,7 @@ bool latent_mfma_supported(int64_t R, int64_t r) {
 }
 
 void head_matmul(Tensor out, Tensor a, Tensor w) {
-  CHECK_GPU(out); CHECK_GPU(a); CHECK_GPU(w); CHECK_CONTIG(out); CHECK_CONTIG(w);
+  CHECK_GPU(out); CHECK_GPU(a); CHECK_GPU(w); CHECK_LAST_CONTIG(out); CHECK_CONTIG(w);
   TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && out.dim() == 3 && a.stride(2) == 1, "head_matmul: ranks");
   const int64_t H = a.size(0), T = a.size(1), K = a.size(2), N = w.size(1);
   TORCH_CHECK(w.size(0) == H && w.size(2) == K && out.size(0) == H && out.size(1) == T &&
@@ -581,8 +582,9 @@ void head_matmul(Tensor out, Tensor a, Tensor w) {
               "head_matmul: sizes / alignment");
   TORCH_CHECK(H <= 65535 && (N / 32) * ((T + 31) / 32) < (1LL << 31), "head_matmul: grid");
   const c10::DeviceGuard g(a.device());
-  akap_stream::launch_head_matmul(out.data_ptr(), a.data_ptr(), a.stride(0), a.stride(1),
-                                  w.data_ptr(), (int)H, (int)T, (int)N, (int)K, cur_stream());
+  akap_stream::launch_head_matmul(out.data_ptr(), out.stride(0), out.stride(1), a.data_ptr(),
+                                  a.stride(0), a.stride(1), w.data_ptr(), (int)H, (int)T, (int)N,
+                                  (int)K, cur_stream());
 }
 
 void head_gate(Tensor out, Tensor o, Tensor gate) {
@@ -740,7 +742,7 @@ void head_norm_cache(Tensor proj, Tensor q_out, Tensor k_cache, Tensor v_cache, 
                   v_cache.scalar_type() == proj.scalar_type(), "head_norm_cache: dtypes differ");
   TORCH_CHECK(slots.scalar_type() == at::kLong, "slots must be int64");
   const int64_t T = proj.size(0), N = proj.size(1);
-  TORCH_CHECK(proj.dim() == 2 && H > 0 && G > 0 && D > 0 && Dv > 0 && q_off >= 0 && k_off >= 0 &&
+  TORCH_CHECK(proj.dim() == 2 && H >= 0 && G > 0 && D > 0 && Dv > 0 && q_off >= 0 && k_off >= 0 &&
                   v_off >= 0 && q_off + H * D <= N && k_off + G * D <= N && v_off + G * Dv <= N,
               "head_norm_cache: slices outside the projection");
   TORCH_CHECK(q_out.numel() == T * H * D && slots.numel() == T, "head_norm_cache: q_out / slots");
@@ -1050,7 +1052,7 @@ TORCH_LIBRARY(akap_stream, m) {
         "Tensor positions, bool single=False) -> ()");
   m.def("latent_prep(Tensor proj, Tensor(a!) cq_out, Tensor(b!)? cache, Tensor positions, "
         "Tensor slots, Tensor cos_sin, Tensor q_w, Tensor? kv_w, int q_rank, int kv_rank, "
-        "int rot_dim, int q_off, int kv_off, float eps, Tensor(c!)? vgroups=None) -> ()");
+        "int rot_dim, int q_off, int kv_off, float eps, Tensor(c!)? vgroups=None, bool half=False) -> ()");
   m.def("latent_attention_prefill_mfma(Tensor(a!) out, Tensor q_lat, Tensor q, int rot_off, "
         "Tensor cache, Tensor vgroups, Tensor block_tables, Tensor seq_lens, Tensor q_start, "
         "Tensor tile_seq, Tensor tile_row, int tile_rows, float scale) -> ()");
@@ -1058,7 +1060,8 @@ TORCH_LIBRARY(akap_stream, m) {
         "Tensor cache, Tensor vgroups, Tensor block_tables, Tensor seq_lens, float scale, "
         "Tensor(b!)? ws_ml, Tensor(c!)? ws_o, int num_parts) -> ()");
   m.def("latent_mfma_supported(int R, int r) -> bool", &latent_mfma_supported);
-  m.def("rotate_heads(Tensor(a!) q, Tensor positions, Tensor cos_sin, int offset) -> ()");
+  m.def("rotate_heads(Tensor(a!) q, Tensor positions, Tensor cos_sin, int offset, "
+        "bool half=False) -> ()");
   m.def("latent_attention(Tensor(a!) out, Tensor q_lat, Tensor q, int rot_off, Tensor cache, "
         "Tensor block_tables, Tensor seq_lens, Tensor? q_start, Tensor positions, float scale) "
         "-> ()");

@@ -745,14 +745,16 @@ def l2_prefetch(tensors) -> None:
         torch.ops.akap.l2_prefetch(ts[i:i + 8], sink)
 
 
-def fused_moe(h, w13, w2, topk_w, topk_ids, out=None):
+def fused_moe(h, w13, w2, topk_w, topk_ids, out=None, clamp=None):
     """Graph-safe fused expert FFN: out[t] = sum_k w[t,k] * W2_e . silu_mul(W13_e . h[t]).
 
     GPU: moe_align (device-side sort + tile->expert map, 32-row tiles) -> grouped k-pipelined
     MFMA GEMM gathering token rows with the SwiGLU in its epilogue (csrc/kernels/
     moe_dgemm.hip) -> grouped GEMM -> deterministic gather-combine.  All buffer shapes depend
     only on (T, top_k, E), so the whole block captures in a hipGraph.
-    w13 [E, 2F, d], w2 [E, d, F]."""
+    w13 [E, 2F, d], w2 [E, d, F].  clamp = (limit, alpha): clamped gated units instead of SwiGLU,
+    with the routing weight on the expert's input -- g = min(w[t,k] gate, limit), u =
+    clamp(w[t,k] up, -limit, limit), g sigmoid(alpha g) (u + 1) -- and a plain sum over k."""
     T, d = h.shape
     K = topk_ids.shape[1]
     E = w13.shape[0]
@@ -760,9 +762,13 @@ def fused_moe(h, w13, w2, topk_w, topk_ids, out=None):
     if out is None:
         out = torch.empty(T, d, dtype=h.dtype, device=h.device)
     if not _native(h):
-        out.copy_(ref.fused_moe(h, w13, w2, topk_w, topk_ids))
+        out.copy_(ref.fused_moe(h, w13, w2, topk_w, topk_ids, clamp))
         return out
     n = T * K
+    units = ()
+    if clamp is not None:
+        units = (1, topk_w.contiguous(), float(clamp[0]), float(clamp[1]))
+        topk_w = torch.ones_like(topk_w)
     bm = moe_tile_rows(n, E)
     cap = moe_capacity(n, E, bm)
     tiles = cap // bm
@@ -772,7 +778,7 @@ def fused_moe(h, w13, w2, topk_w, topk_ids, out=None):
     sorted_ids, _, _ = moe_align(topk_ids, E, bm, inv=inv, tile_expert=tile_expert)
     act = torch.empty(cap, F, dtype=h.dtype, device=dev)
     torch.ops.akap.moe_dgemm(act, h, w13, sorted_ids, tile_expert, n, K, True, True,
-                             _moe_pf(d), bm)
+                             _moe_pf(d), bm, *units)
     S = moe_down_splitk(n, E, bm, F)
     if S > 1:
         # fp32 K-slices of the down projection, summed by the combine (no extra launch)

@@ -255,10 +255,11 @@ def moe_align(topk_ids, E, block, cap):
     return sorted_ids.to(topk_ids.device), offsets.to(topk_ids.device), acc
 
 
-def fused_moe(h, w13, w2, topk_w, topk_ids):
+def fused_moe(h, w13, w2, topk_w, topk_ids, clamp=None):
     """fp32 reference of the fused expert FFN (bf16 rounding at the same points as the
     kernels: after each GEMM and after silu_and_mul).  Expert ids outside [0, E) -- the
-    padding rows of the expert-parallel dispatch -- contribute nothing (as in moe_align)."""
+    padding rows of the expert-parallel dispatch -- contribute nothing (as in moe_align).
+    clamp = (limit, alpha): clamped units of the weighted inputs (ops.fused_moe)."""
     T, d = h.shape
     E = w13.shape[0]
     out = torch.zeros(T, d, dtype=torch.float32, device=h.device)
@@ -267,10 +268,18 @@ def fused_moe(h, w13, w2, topk_w, topk_ids):
         t_idx, k_idx = (ids == e).nonzero(as_tuple=True)
         if t_idx.numel() == 0:
             continue
-        y1 = (h[t_idx].float() @ w13[e].float().t()).to(h.dtype)
-        a = silu_and_mul(y1)
+        y1 = h[t_idx].float() @ w13[e].float().t()
+        wk = topk_w[t_idx, k_idx].float()[:, None]
+        if clamp is not None:
+            limit, alpha = clamp
+            g, u = (y1 * wk).chunk(2, dim=-1)
+            g, u = torch.clamp(g, max=limit), torch.clamp(u, min=-limit, max=limit)
+            a = (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(h.dtype)
+            wk = torch.ones_like(wk)
+        else:
+            a = silu_and_mul(y1.to(h.dtype))
         y2 = (a.float() @ w2[e].float().t()).to(h.dtype)
-        out.index_add_(0, t_idx, topk_w[t_idx, k_idx].float()[:, None] * y2.float())
+        out.index_add_(0, t_idx, wk * y2.float())
     return out.to(h.dtype)
 
 
