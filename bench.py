@@ -90,7 +90,7 @@ def parse():
     ap.add_argument("--profile-steps", type=int, default=0,
                     help="extra untimed waves run after timing (for rocprofv3 captures)")
     ap.add_argument("--compare-design", default=None, choices=["bidetar", "puputar", "sazepel", "mudepel",
-                                                               "papivik"],
+                                                               "papivik", "venanex"],
                     help="instead of the serving wave: prefill and decode throughput of this "
                          "design at real layer sizes (random weights) beside the closest "
                          "existing model of equal size; prints one JSON line with the table")
@@ -121,6 +121,11 @@ COMPARE_SETS = {
     # matrix-memory, linear-attention and attention + delta-rule layers beside the framework's
     # two other hybrids of a recurrent state and an attention at the same width and depth
     "papivik": [("papivik-w2048", "sazepel-w2048"), ("papivik-w4096", "sazepel-w4096"),
+                ("mudepel-w2048", None)],
+    # latent + differential attention with routed experts in every layer beside the framework's
+    # other latent design (its routed variant) and the one whose every second layer has the same
+    # kind of router and a shared expert, at the same width and number of layer runs
+    "venanex": [("venanex-w2048", "puputar-w2048-moe"), ("venanex-w4096", "mudepel-w4096"),
                 ("mudepel-w2048", None)],
 }
 

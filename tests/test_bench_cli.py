@@ -112,7 +112,8 @@ def test_bench_gpus_n_without_launcher_starts_n_ranks():
                                            ("puputar", "tiny-puputar,tiny-bidetar"),
                                            ("sazepel", "tiny-sazepel,tiny-bidetar"),
                                            ("mudepel", "tiny-mudepel,tiny-sazepel"),
-                                           ("papivik", "tiny-papivik,tiny-mudepel")])
+                                           ("papivik", "tiny-papivik,tiny-mudepel"),
+                                           ("venanex", "tiny-venanex,tiny-puputar")])
 def test_bench_compare_design_option(design, models):
     """--compare-design prints one JSON line with prefill and decode throughput per model and
     leaves the default output alone."""

@@ -335,3 +335,32 @@ def test_recurrent_design_served_with_sampling_and_no_prefix_cache(design):
     hits = sum(float(ln.rsplit(" ", 1)[1]) for ln in text.splitlines()
                if ln.startswith("vllm:prefix_cache_hits_total"))
     assert hits == 0
+
+
+def test_latent_and_differential_design_served_with_prefix_cache():
+    """A design whose sequences own nothing but pages, behind the OpenAI endpoints with the prefix
+    cache on: a repeated prompt reuses its pages (latents of every pass of the loop, keys and
+    values) and gives the same greedy completion; more prompts than slots; sampling."""
+    from aws_k8s_ansible_provisioner_amd.engine.config import EngineConfig
+    from aws_k8s_ansible_provisioner_amd.server.api_server import build_app
+
+    app, ae = build_app(EngineConfig(model="tiny-venanex", served_model_name="m", device="cpu",
+                                     dtype="float32", max_model_len=256, max_num_seqs=2,
+                                     max_num_batched_tokens=48, block_size=32,
+                                     num_gpu_blocks=64, enable_prefix_caching=True))
+    prompt = list(range(10, 110))
+    with TestClient(app) as c:
+        def text(p, **kw):
+            r = c.post("/v1/completions", json={"prompt": p, "max_tokens": 6, "temperature": 0.0,
+                                                **kw})
+            assert r.status_code == 200, r.text
+            return [ch["text"] for ch in sorted(r.json()["choices"], key=lambda ch: ch["index"])]
+
+        assert text(prompt) == text(prompt)
+        short = [[50, 51, 52], list(range(200, 233)), [7] * 7]
+        assert text(short) == [text(p)[0] for p in short]
+        assert len(text(prompt[:50], temperature=0.8, top_p=0.9, seed=3)) == 1
+        metrics = c.get("/metrics").text
+    hits = sum(float(ln.rsplit(" ", 1)[1]) for ln in metrics.splitlines()
+               if ln.startswith("vllm:prefix_cache_hits_total"))
+    assert hits > 0

@@ -188,3 +188,89 @@ def forward(cfg, W, tokens):
         x = layer(x, W, f"l{i}.", cfg["layers"][i], eps)
         after.append(x)
     return layer_norm(x, W["final.norm"], eps) @ W["embed"].T, torch.stack(after)
+
+
+# ------------------------------------------------------------------------------------- test models
+def latent_layer(heads, dim, rot_dim, vdim, kv_rank, q_rank, scale=None, base=100.0, yarn=None,
+                 mlp=None):
+    """yarn = (factor, original, fast, slow) or None."""
+    sc = dict(zip(("factor", "original", "fast", "slow"), yarn)) if yarn else None
+    return {"type": "latent_attention", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim,
+                      "kv_rank": kv_rank, "q_rank": q_rank,
+                      "scale": scale if scale is not None else (dim + rot_dim) ** -0.5,
+                      "rot": {"base": base, "dims": rot_dim, "scaling": sc}}}
+
+
+def diff_layer(heads, kv_heads, dim, vdim, chunk, diff=0.6, scale=None, mlp=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "diff": diff,
+         "scale": scale if scale is not None else dim ** -0.5}
+    if chunk:
+        m["mask"] = {"size": chunk}
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def experts(n, top, ff, limit=1.0, shared=None, shared_limit=2.0):
+    ml = {"kind": "moe", "expert": {"ff": ff, "limit": limit},
+          "router": {"experts": n, "top": top}}
+    if shared:
+        ml["shared"] = {"ff": shared, "limit": shared_limit}
+    return ml
+
+
+def make_config(width, vocab, layers, loop=None, eps=1e-5):
+    cfg = {"architecture": "Venanex", "layers": layers, "norm": {"eps": eps}, "vocab": vocab,
+           "width": width}
+    if loop:
+        cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return cfg
+
+
+def random_weights(cfg, seed=0):
+    """Random tensors under the checkpoint's names, values that bfloat16 holds exactly.  The rows
+    of the stream get a mean far from zero, so that a norm without its subtraction shows."""
+    g = torch.Generator().manual_seed(seed)
+    d = cfg["width"]
+
+    def rnd(*shape, s=1.0, mean=0.0):
+        return (torch.randn(*shape, generator=g) * s + mean).to(torch.bfloat16)
+
+    def lin(rows, cols, s=1.0):
+        return rnd(rows, cols, s=s * cols ** -0.5)
+
+    def gain(n):
+        return rnd(n, s=0.2, mean=1.0)
+
+    W = {"embed": rnd(cfg["vocab"], d, mean=0.5), "final.norm": gain(d)}
+    if cfg.get("loop"):
+        W["loop.in"] = lin(d, 2 * d, 1.2)
+    for i, ly in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", ly["mixer"]
+        H, D, V = m["heads"], m["dim"], m["vdim"]
+        W[p + "norm1"], W[p + "norm1b"] = gain(d), rnd(d, s=0.2, mean=0.8)
+        if ly["type"] == "latent_attention":
+            R, r, Q = m["kv_rank"], m["rot_dim"], m["q_rank"]
+            W[p + "mix.dq"], W[p + "mix.dq.norm"] = lin(Q, d), gain(Q)
+            W[p + "mix.uq"] = lin(H * (D + r), Q, 1.6)
+            W[p + "mix.dkv"], W[p + "mix.dkv.norm"] = lin(R + r, d), gain(R)
+            W[p + "mix.uk"], W[p + "mix.uv"] = lin(H * D, R, 1.6), lin(H * V, R)
+        else:
+            G = m["kv_heads"]
+            W[p + "mix.q"], W[p + "mix.k"] = lin(H * 2 * D, d, 1.4), lin(G * 2 * D, d, 1.4)
+            W[p + "mix.v"], W[p + "mix.g"] = lin(G * V, d), lin(H * V, d)
+            for n in ("lq1", "lk1", "lq2", "lk2"):
+                W[p + "mix." + n] = rnd(D, s=0.5 * D ** -0.25)
+        W[p + "mix.o"] = lin(d, H * V)
+        ml = ly.get("mlp")
+        if ml is None:
+            continue
+        W[p + "norm2"], W[p + "norm2b"] = gain(d), rnd(d, s=0.2, mean=0.8)
+        W[p + "mlp.router"] = lin(ml["router"]["experts"], d, 2.0)
+        names = [(f"e{e}.", ml["expert"]["ff"]) for e in range(ml["router"]["experts"])]
+        if ml.get("shared"):
+            names.append(("shared.", ml["shared"]["ff"]))
+            W[p + "mlp.shared.sg"] = lin(1, d)
+        for n, ff in names:
+            W[p + f"mlp.{n}gate"], W[p + f"mlp.{n}up"] = lin(ff, d, 1.5), lin(ff, d, 1.5)
+            W[p + f"mlp.{n}down"] = lin(d, ff, 2.0)
+    return W
