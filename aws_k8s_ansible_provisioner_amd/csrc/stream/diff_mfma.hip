@@ -82,24 +82,28 @@ __device__ __forceinline__ void softmax_block(f32x16& s, bf16x8 (&pb)[2], f32x16
   }
 }
 
-// o1 * f1 - o2 * f2 -> head norm, 1 - diff, gate, store.  Register i of tile k: entry
-// 32 k + 8 (i >> 2) + 4 hf + (i & 3) of the head's output.  v is the difference.
+// 1 / rms of a head's difference v (registers of this lane, its other half and, for split heads,
+// `other`: the share of the wave that holds the rest) times 1 - diff
 template <int DVT>
-__device__ __forceinline__ void finish(f32x16 (&v)[DVT], const DiffAttnParams& p, int t, int h,
-                                       bool store) {
-  constexpr int Dv = 32 * DVT;
-  const int hf = (threadIdx.x & 63) >> 5;
+__device__ __forceinline__ float sum_squares(const f32x16 (&v)[DVT]) {
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < DVT; ++k)
 #pragma unroll
     for (int i = 0; i < 16; ++i) ss += v[k][i] * v[k][i];
-  ss += __shfl_xor(ss, 32, 64);
-  if (!store) return;
-  const float f = p.out_mult / sqrtf(ss * (1.0f / Dv) + p.eps);
-  bf16* o = (bf16*)p.out + (size_t)t * p.out_stride + (size_t)h * Dv + 4 * hf;
-  const bf16* gt = p.gate ? (const bf16*)p.gate + (size_t)t * p.gate_stride + (size_t)h * Dv + 4 * hf
-                          : nullptr;
+  return ss + __shfl_xor(ss, 32, 64);
+}
+
+// scale, gate, store DVT tiles of head h from value entry d0 on.  Register i of tile k: entry
+// d0 + 32 k + 8 (i >> 2) + 4 hf + (i & 3).
+template <int DVT>
+__device__ __forceinline__ void store_head(const f32x16 (&v)[DVT], float ss, const DiffAttnParams& p,
+                                           int t, int h, int d0) {
+  const int hf = (threadIdx.x & 63) >> 5;
+  const float f = p.out_mult / sqrtf(ss / (float)p.Dv + p.eps);
+  const size_t c = (size_t)h * p.Dv + d0 + 4 * hf;
+  bf16* o = (bf16*)p.out + (size_t)t * p.out_stride + c;
+  const bf16* gt = p.gate ? (const bf16*)p.gate + (size_t)t * p.gate_stride + c : nullptr;
 #pragma unroll
   for (int k = 0; k < DVT; ++k)
 #pragma unroll
@@ -118,16 +122,24 @@ __device__ __forceinline__ void finish(f32x16 (&v)[DVT], const DiffAttnParams& p
 }
 
 // Flat grid: (tile of 128 tokens, key/value head) units dealt over the XCDs longest first, the
-// query heads of a unit are consecutive workgroups of ONE XCD; four waves of 32 queries each.
-template <int KS, int DVT>
-__global__ __launch_bounds__(256) void diff_prefill_mfma_kernel(DiffAttnParams p) {
-  constexpr int D = 16 * KS, Dv = 32 * DVT;
+// query heads of a unit are consecutive workgroups of ONE XCD; 32 queries per wave.  SPLIT 2: two
+// waves share a query tile, each with half of the value entries (DVT tiles of 32 per wave), so
+// that wide values fit the registers; both compute the scores.  The maps take turns (one score
+// tile and one map's K fragments live at a time, the queries in LDS), which leaves room for two
+// waves per SIMD: the fragments of map 2 are requested ahead of map 1's softmax, those of the next
+// block's map 1 ahead of map 2's, the V fragments at the start of the block.
+template <int KS, int DVT, int SPLIT>
+__global__ __launch_bounds__(256 * SPLIT, 2) void diff_prefill_mfma_kernel(DiffAttnParams p) {
+  constexpr int D = 16 * KS, Dv = 32 * DVT * SPLIT;
+  __shared__ bf16x8 qs_all[4][2 * KS][64];           // [query tile][map, step][lane]
+  __shared__ float share[4 * SPLIT][32];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int qt = wave / SPLIT, d0 = (wave % SPLIT) * 32 * DVT;
   const int col = lane & 31, hf = lane >> 5;
   const int rep = p.H / p.G;
   const int xcd = blockIdx.x & 7, jx = blockIdx.x >> 3;
   const int unit = (jx / rep) * 8 + xcd;
-  if (unit >= p.num_tiles * p.G) return;
+  if (unit >= p.num_tiles * p.G) return;             // (workgroup-uniform, like the next two)
   const int tile = p.num_tiles - 1 - unit / p.G;     // the map is sorted by rising work
   const int g = unit % p.G, h = g * rep + jx % rep;
   const int b = p.tile_seq[tile];
@@ -135,30 +147,32 @@ __global__ __launch_bounds__(256) void diff_prefill_mfma_kernel(DiffAttnParams p
   const int qs0 = p.q_start[b];
   const int qlen = p.q_start[b + 1] - qs0;
   const int kv = p.seq_lens[b];
+  if (kv < qlen) return;
   const int rend = min(p.tile_row[tile] + p.tile_rows, qlen);
   const float sc2 = p.scale * kLog2e;
   const int32_t* bt = p.block_tables + (size_t)b * p.max_blocks;
   const bf16* kc = (const bf16*)p.k_cache;
   const bf16* vc = (const bf16*)p.v_cache;
   const int krow = swap23(col);
-  const int r0 = p.tile_row[tile] + wave * 32;
-  if (r0 >= rend || kv < qlen) return;
+  const int r0 = p.tile_row[tile] + qt * 32;
+  const bool active = r0 < rend;                     // the others only meet the barriers
   const int r = r0 + col;
   const bool valid = r < rend;
-  const int t = qs0 + (valid ? r : r0);
+  const int t = qs0 + (valid ? r : active ? r0 : 0);
   const int pos = kv - qlen + r;
   const int lo = chunk_start(pos, p.chunk);
-  bf16x8 qf[2][KS];
-  {
+  bf16x8 (&qs)[2 * KS][64] = qs_all[qt];
+  if (wave % SPLIT == 0) {
     const bf16* qp = (const bf16*)p.q + (size_t)t * p.q_stride + (size_t)h * 2 * D + 8 * hf;
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
-#pragma unroll
-      for (int c = 0; c < KS; ++c) qf[k][c] = *(const bf16x8*)(qp + k * D + 16 * c);
+    for (int c = 0; c < 2 * KS; ++c) qs[c][lane] = *(const bf16x8*)(qp + 16 * c);
   }
+  __syncthreads();
   // the wave's range; columns past the tile's end compute like real ones and are not stored
-  const int first = kv - qlen + r0, end = kv - qlen + min(r0 + 31, rend - 1);
-  const int lo_first = chunk_start(first, p.chunk), lo_last = chunk_start(first + 31, p.chunk);
+  const int first = kv - qlen + r0;
+  const int end = active ? kv - qlen + min(r0 + 31, rend - 1) : -1;
+  const int lo_last = chunk_start(first + 31, p.chunk);
+  const int jb = active ? chunk_start(first, p.chunk) & ~31 : 0;
   f32x16 o[2][DVT];
   float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
 #pragma unroll
@@ -168,61 +182,71 @@ __global__ __launch_bounds__(256) void diff_prefill_mfma_kernel(DiffAttnParams p
 #pragma unroll
       for (int i = 0; i < 16; ++i) o[k][d][i] = 0.f;
 
-  // K fragments of the next block are requested before this block's softmax, its block-table
-  // entry one block earlier still; this block's V fragments before its Q K^T products
-  const int jb = lo_first & ~31;
-  int row0 = key_row(p, bt, g, jb);
-  int row1 = jb + 32 <= end ? key_row(p, bt, g, jb + 32) : 0;
-  bf16x8 kf[2][KS];
-  auto load_k = [&](int row) {
-    const bf16* kp = kc + ((size_t)row + krow) * (2 * D) + 8 * hf;
+  if (active) {
+    int row0 = key_row(p, bt, g, jb);
+    int row1 = jb + 32 <= end ? key_row(p, bt, g, jb + 32) : 0;
+    bf16x8 kf[KS];
+    auto load_k = [&](int row, int map) {
+      const bf16* kp = kc + ((size_t)row + krow) * (2 * D) + map * D + 8 * hf;
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
+      for (int c = 0; c < KS; ++c) kf[c] = *(const bf16x8*)(kp + 16 * c);
+    };
+    load_k(row0, 0);
+    for (int j0 = jb; j0 <= end; j0 += 32) {
+      const bf16* vp = vc + (((size_t)(row0 >> 3) + hf) * Dv + d0 + col) * 8;
+      bf16x8 vf[DVT][2];
+      auto load_v = [&] {
 #pragma unroll
-      for (int c = 0; c < KS; ++c) kf[k][c] = *(const bf16x8*)(kp + k * D + 16 * c);
-  };
-  load_k(row0);
-  for (int j0 = jb; j0 <= end; j0 += 32) {
-    const bf16* vp = vc + (((size_t)(row0 >> 3) + hf) * Dv + col) * 8;
-    bf16x8 vf[DVT][2];
+        for (int d = 0; d < DVT; ++d)
 #pragma unroll
-    for (int d = 0; d < DVT; ++d)
+          for (int sl = 0; sl < 2; ++sl)
+            vf[d][sl] = *(const bf16x8*)(vp + ((size_t)(2 * sl) * Dv + 32 * d) * 8);
+      };
+      if (KS <= 4) load_v();
+      const bool full = j0 + 31 <= first && j0 >= lo_last;
 #pragma unroll
-      for (int sl = 0; sl < 2; ++sl)
-        vf[d][sl] = *(const bf16x8*)(vp + ((size_t)(2 * sl) * Dv + 32 * d) * 8);
-    f32x16 s[2];
+      for (int k = 0; k < 2; ++k) {
+        f32x16 s;
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
+        for (int i = 0; i < 16; ++i) s[i] = 0.f;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) s[k][i] = 0.f;
+        for (int c = 0; c < KS; ++c)
+          s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[c], qs[k * KS + c][lane], s, 0, 0, 0);
+        if (k == 0) {
+          if (KS > 4) {                              // long rows: not beside the score products
+            __builtin_amdgcn_sched_barrier(0);
+            load_v();
+          }
+          load_k(row0, 1);
+        } else if (j0 + 32 <= end) {
+          row0 = row1;
+          load_k(row0, 0);
+          if (j0 + 64 <= end) row1 = key_row(p, bt, g, j0 + 64);
+        }
+        bf16x8 pb[2];
+        softmax_block<DVT>(s, pb, o[k], m[k], l[k], j0, full, pos, lo, sc2);
 #pragma unroll
-      for (int c = 0; c < KS; ++c)
-        s[k] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[k][c], qf[k][c], s[k], 0, 0, 0);
+        for (int d = 0; d < DVT; ++d)
+#pragma unroll
+          for (int sl = 0; sl < 2; ++sl)
+            o[k][d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[d][sl], pb[sl], o[k][d], 0, 0, 0);
+      }
     }
-    if (j0 + 32 <= end) {
-      row0 = row1;
-      load_k(row0);
-      if (j0 + 64 <= end) row1 = key_row(p, bt, g, j0 + 64);
-    }
-    const bool full = j0 + 31 <= first && j0 >= lo_last;
-    bf16x8 pb[2][2];
-#pragma unroll
-    for (int k = 0; k < 2; ++k)
-      softmax_block<DVT>(s[k], pb[k], o[k], m[k], l[k], j0, full, pos, lo, sc2);
-#pragma unroll
-    for (int d = 0; d < DVT; ++d)
-#pragma unroll
-      for (int sl = 0; sl < 2; ++sl)
-#pragma unroll
-        for (int k = 0; k < 2; ++k)
-          o[k][d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[d][sl], pb[k][sl], o[k][d], 0, 0, 0);
   }
   const float f1 = l[0] > 0.f ? 1.0f / l[0] : 0.f, f2 = l[1] > 0.f ? p.lam / l[1] : 0.f;
 #pragma unroll
   for (int d = 0; d < DVT; ++d)
 #pragma unroll
     for (int i = 0; i < 16; ++i) o[0][d][i] = o[0][d][i] * f1 - o[1][d][i] * f2;
-  finish<DVT>(o[0], p, t, h, valid);
+  float ss = sum_squares<DVT>(o[0]);
+  if constexpr (SPLIT > 1) {
+    if (hf == 0) share[wave][col] = ss;
+    __syncthreads();
+    ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < SPLIT; ++k) ss += share[qt * SPLIT + k][col];
+  }
+  if (valid) store_head<DVT>(o[0], ss, p, t, h, d0);
 }
 
 // grid (B, G * ceil(rep / 16), parts), one wave
@@ -333,7 +357,8 @@ __global__ __launch_bounds__(64) void diff_decode_mfma_kernel(DiffAttnParams p) 
       const float a = o[d][i] * f;
       o[d][i] = a - __shfl_xor(a, 16, 64);
     }
-  finish<DVT>(o, p, b, h, valid && map == 0);
+  const float ss = sum_squares<DVT>(o);
+  if (valid && map == 0) store_head<DVT>(o, ss, p, b, h, 0);
 }
 
 // grid (B, H), 128 threads: the partitions of one (row, head) under both maps
@@ -395,8 +420,11 @@ bool diff_mfma_supported(int D, int Dv, int BS) {
 void launch_diff_prefill_mfma(const DiffAttnParams& p, hipStream_t s) {
   if (p.num_tiles <= 0) return;
   const unsigned grid = (unsigned)((p.num_tiles * p.G + 7) / 8 * 8) * (p.H / p.G);
-#define F(a, c) \
-  if (p.D == a && p.Dv == c) diff_prefill_mfma_kernel<a / 16, c / 32><<<grid, 256, 0, s>>>(p);
+#define F(a, c)                                                                       \
+  if (p.D == a && p.Dv == c) {                                                        \
+    constexpr int sp = c > 128 ? 2 : 1;                                               \
+    diff_prefill_mfma_kernel<a / 16, c / 32 / sp, sp><<<grid, 256 * sp, 0, s>>>(p);   \
+  }
   DIFF_SIZES(F)
 #undef F
 }
