@@ -317,7 +317,7 @@ class DecoderLM:
         On the GPU every allocation's size is kept hipIpc-safe (`ipc_safe_alloc_bytes`): the
         HIP runtime PyTorch bundles (ROCm 7.0.2) hangs in hipIpcOpenMemHandle when bit 31 of
         the allocation size is set (size mod 4 GiB >= 2 GiB; 1.5 / 5 / 8 / 9.5 / 36 GiB map,
-        2 / 2.5 / 6.6 GiB hang, at any occupancy -- bench/ipc_import_repro.cpp,
+        2 / 2.5 / 6.6 GiB hang, at any occupancy --
         profiles/r6_ipc_import_sweep.md; ROCm 7.2's runtime maps them all).  That was the
         round-4/5 "hang once the device is mostly allocated": big caches made such sizes.
         The layers per segment are chosen to avoid padding where possible; otherwise the

@@ -210,7 +210,7 @@ def timed_graphs(fns, iters=10):
 def run_fresh(halves, pool):
     """Alternating attention with only forward stream dependencies: every cross-stream wait
     continues on a brand-new stream (hipGraph capture on ROCm 7 segfaults when a stream waits
-    on a stream that earlier waited on it: bench/graph_multistream_probe.py)."""
+    on a stream that earlier waited on it: profiles/r2_graph_capture_segfault.md)."""
     main = torch.cuda.current_stream()
     it = iter(pool)
     L = len(halves[0].m.layers)

@@ -10,5 +10,4 @@ run sk_t 400 python -u -m pytest -x -v --timeout 120 --timeout-method thread tes
 run sk_b 400 python -u tools/pgemm_m256_probe.py &&
 run slope 400 python -u tools/gemm_slope.py &&
 run car 700 python -u -m pytest -x -v --timeout 240 --timeout-method thread tests/test_custom_allreduce_gpu.py &&
-run ipc3seg 150 python -u tools/ipc_multi_open_probe.py --mode serial --gb 86 --segments 3 --world 3 &&
 echo done
