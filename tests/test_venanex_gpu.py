@@ -52,7 +52,7 @@ def test_layer_norm_step_kernel(dtype, d):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("E,F_,Fs,top", [(4, 5, 3, 2), (6, 64, 48, 1), (1, 8, 0, 1), (16, 96, 128, 4),
+@pytest.mark.parametrize("E,F_,Fs,top", [(4, 5, 3, 2), (6, 64, 48, 1), (1, 8, 0, 1), (12, 80, 112, 4),
                                          (8, 1408, 1408, 2), (0, 0, 40, 1)])
 def test_clamped_glu_kernel(dtype, E, F_, Fs, top):
     g, dt = gen(E * F_ + Fs), DT[dtype]
@@ -75,7 +75,7 @@ def test_clamped_glu_kernel(dtype, E, F_, Fs, top):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("E,d,top", [(5, 36, 2), (16, 192, 1), (8, 2048, 2), (3, 7, 3)])
+@pytest.mark.parametrize("E,d,top", [(5, 36, 2), (12, 160, 1), (8, 2048, 2), (3, 7, 3)])
 def test_router_with_gate_row_kernel(dtype, E, d, top):
     g = gen(E * d)
     h, router = torch.randn(9, d, generator=g).to(DT[dtype]), torch.randn(E + 1, d, generator=g) / d ** 0.5
@@ -170,7 +170,7 @@ def attention_close(got, want, dtype):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("H,G,D,Dv,chunk", [
     (4, 2, 6, 10, 20), (3, 3, 5, 3, 0), (6, 1, 24, 40, 7), (2, 2, 1, 1, 1), (2, 1, 80, 320, 0),
-    (4, 2, 16, 32, 64), (4, 4, 16, 64, 0), (6, 2, 32, 32, 100), (8, 2, 32, 64, 64),
+    (4, 2, 16, 32, 64), (4, 4, 16, 64, 0), (6, 2, 32, 32, 100), (8, 2, 32, 64, 96),
     (4, 1, 32, 128, 0), (2, 2, 64, 64, 33), (8, 2, 64, 128, 0), (20, 1, 64, 128, 90),
     (2, 1, 64, 256, 128), (4, 2, 128, 128, 0), (2, 2, 128, 256, 50), (40, 1, 16, 32, 0)])
 def test_differential_attention_kernels(dtype, H, G, D, Dv, chunk):
@@ -209,7 +209,7 @@ def test_split_of_decode_rows(max_len):
 def test_one_key_at_a_chunk_edge_kernels(dtype, far, single):
     """One key takes nearly all the weight wherever it is seen: rows of its own chunk from its
     position on carry its value, no other row notices."""
-    H, G, D, Dv, chunk, dt = 4, 2, 32, 64, 64, DT[dtype]
+    H, G, D, Dv, chunk, dt = 6, 3, 64, 64, 64, DT[dtype]
     seqs = [(p + 1, 1) for p in (62, 63, 64, 100, 127, 128, 129, 220)] if single else [(221, 221)]
     batch, kc, vt, gather, where = attention_case(seqs, G, D, Dv, 32, seed=far, dtype=dt)
     T = sum(n for _, n in seqs)
@@ -370,7 +370,7 @@ def test_mid_size_engine_against_the_cpu_ops(tmp_path, dtype, core):
     grouped expert GEMMs then take the prompt portions."""
     if core:
         ops.load_native(required=True)
-    cfg = oracle.make_config(width=192, vocab=301, loop=(0, 2, 2), layers=[
+    cfg = oracle.make_config(width=160, vocab=301, loop=(0, 2, 2), layers=[
         oracle.latent_layer(6, 64, 32, 64, 128, 160, base=9000.0, yarn=(4.0, 128, 16.0, 1.0),
                             mlp=oracle.experts(6, 2, 128, limit=1.5, shared=192)),
         oracle.diff_layer(8, 2, 64, 128, chunk=128, scale=0.11,
