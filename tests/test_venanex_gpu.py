@@ -367,14 +367,16 @@ def test_mid_size_engine_against_the_cpu_ops(tmp_path, dtype, core):
     """Sizes between the tiny oracle models and the benchmark's (matrix-core attention, 16-byte
     paths everywhere, portions above the small-batch threshold): the engine on the GPU against the
     same engine on the CPU ops, over a mixed schedule; core: with the core library loaded, whose
-    grouped expert GEMMs then take the prompt portions."""
+    grouped expert GEMMs then take the prompt portions.  bf16 chooses every expert, so that no
+    close routing choice can turn over and the comparison can be tight."""
+    top = (2, 1) if dtype == "float32" else (6, 5)
     if core:
         ops.load_native(required=True)
     cfg = oracle.make_config(width=160, vocab=301, loop=(0, 2, 2), layers=[
         oracle.latent_layer(6, 64, 32, 64, 128, 160, base=9000.0, yarn=(4.0, 128, 16.0, 1.0),
-                            mlp=oracle.experts(6, 2, 128, limit=1.5, shared=192)),
+                            mlp=oracle.experts(6, top[0], 128, limit=1.5, shared=192)),
         oracle.diff_layer(8, 2, 64, 128, chunk=128, scale=0.11,
-                          mlp=oracle.experts(5, 1, 64, shared=96, shared_limit=1.0)),
+                          mlp=oracle.experts(5, top[1], 64, shared=96, shared_limit=1.0)),
         oracle.diff_layer(4, 4, 32, 64, chunk=0, diff=0.3, scale=0.2)])
     W = oracle.random_weights(cfg, seed=11)
     path = write_model(tmp_path, cfg, W)
@@ -385,8 +387,5 @@ def test_mid_size_engine_against_the_cpu_ops(tmp_path, dtype, core):
     got = replay(engine(path, dtype=dtype, max_tokens=1024, device="cuda"), reqs, sched)
     for n in reqs:
         e = rel_err(got[n], want[n])
-        if dtype == "float32":
-            assert e.max().item() < 2e-4, f"{n}: position {int(e.argmax())} off by {e.max().item():.2e}"
-        else:
-            assert e.median().item() < 0.05 and (e > 0.3).float().mean().item() < 0.1, (
-                n, e.median().item(), e.max().item())
+        assert e.max().item() < (2e-4 if dtype == "float32" else 0.06), \
+            f"{n}: position {int(e.argmax())} off by {e.max().item():.2e}"
